@@ -397,6 +397,115 @@ int lr_ladder_decode_step_fp8(const lr_ladder_model_t* model, int batch, const i
 int lr_sample_topk(const void* logits, int64_t ldl, const void* noise, int64_t ldn, int B, int V, float temperature,
                    int top_k, void* probs, int64_t ldp, int32_t* next_token, lr_stream_t stream);
 
+/* ---------------------------------------------------------------------------------------------
+ * Models with an fp32 residual stream and token mixers of other kinds (the Lasivik family).  No
+ * counterpart in the reference.  `dtype` selects the storage of weights and activations: bf16 as
+ * everywhere above, or fp32 for running such a model in true 32-bit throughout; the arithmetic
+ * named fp32 below is fp32 in both. */
+enum { LR_BF16 = 0, LR_F32 = 1 };
+
+/* x[t, :] = table[idx[t], :] * scale in fp32; x_compute (may be NULL): the same in the compute type.
+ * idx as in lr_embed; dim % 8 == 0. */
+int lr_embed_residual(const void* table, const void* idx, int idx_is_i64, float* x, void* x_compute, int64_t n_tokens,
+                      int dim, int vocab, float scale, int dtype, lr_stream_t stream);
+
+/* r = alpha * x + d (fp32; d in the compute type, may be NULL), then
+ *     out = r / sqrt(mean(r^2) + eps) * (gain_offset + gain)
+ * into x_out (fp32, may be NULL, may alias x) and / or x_compute (compute type, may be NULL).  With gain_offset 1 the
+ * gain is stored around zero.  Rows are dense with `dim` columns (dim % 8 == 0, <= 16384), of which the first
+ * `width` count for the mean; the others must be zero in x, d and gain. */
+int lr_residual_rmsnorm(const float* x, float alpha, const void* d, const void* gain, float gain_offset, float* x_out,
+                        void* x_compute, int rows, int dim, int width, float eps, int dtype, lr_stream_t stream);
+
+/* logits = cap * tanh(scale * logits / cap) in place (cap <= 0: the scale alone); [rows, V], row stride ldl. */
+int lr_logit_cap(void* logits, int64_t ldl, int rows, int V, float scale, float cap, int dtype, lr_stream_t stream);
+
+/* lr_linear / lr_swiglu / lr_argmax on fp32 tensors (fp32 matrix-core products, no reduced-precision mode; any sizes). */
+int lr_linear_f32(const float* x, int64_t ldx, const float* w, float* y, int64_t ldy, int M, int N, int K,
+                  lr_stream_t stream);
+int lr_swiglu_f32(const float* h, int64_t ldh, float* out, int rows, int I, lr_stream_t stream);
+int lr_argmax_f32(const float* logits, int64_t ldl, int32_t* out, int B, int V, lr_stream_t stream);
+
+/* Linear attention with decay over S consecutive tokens per sequence, the state carried from call to call:
+ *     S_t = diag(a_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t          per head, S [dk, dv] fp32
+ *     y = o / sqrt(mean(o^2) + eps) * norm * silu(g)                  per head over dv (norm NULL: no gain)
+ * q, k [B*S, H*dk], v, g [B*S, H*dv] are column ranges of one buffer with row stride ld (row b * S + s); y [B*S, H*dv].
+ * Decay: lowrank != NULL -- a = sigmoid(a2 t + a_bias)^(1/tau) per key channel, t [B*S, rank] another column range of
+ * the buffer, a2 [H*dk, rank], a_bias [H*dk]; else e^head_decay[h] (fp32 logs on the device).
+ * rope != NULL: q and k are first rotated, pairs (i, i + rot_dims / 2) of a head's first rot_dims dimensions by the angle
+ * whose (cos, sin) is rope[position][i], fp32 [rope_len, rot_dims / 2, 2].  Then q *= q_scale, k *= k_scale.
+ * pos [>= 1] int32 on the device: position of the call's first token; 0 starts from a zero state, whatever `state`
+ * ([B, H, dk, dv]) holds, anything else continues from it.  A position outside the rope table sets *err and leaves
+ * everything untouched.  dk, dv <= 256.  S == 1 is one launch; else scratch of lr_linear_attention_scratch_bytes()
+ * bytes (0: none needed). */
+typedef struct lr_linear_attention {
+  const void *q, *k, *v, *g;
+  int64_t ld;
+  const void *lowrank, *a2, *a_bias;
+  const float* head_decay;
+  const float* rope;
+  const int32_t* pos;
+  float* state;
+  const void* norm;
+  void* y;
+  int64_t ldy;
+  int32_t* err; /* may be NULL */
+  void* scratch;
+  size_t scratch_bytes;
+  int32_t B, S, H, dk, dv, rank, rot_dims, rope_len, dtype;
+  float tau, q_scale, k_scale, eps;
+} lr_linear_attention_t;
+size_t lr_linear_attention_scratch_bytes(int B, int S, int H, int dk, int dv, int gated);
+int lr_linear_attention(const lr_linear_attention_t* desc, lr_stream_t stream);
+
+/* Latent cache of a low-rank attention: cache[b, pos[s], :] = c[row] / sqrt(mean(c^2) + eps) * gain for row b * S + s,
+ * c [B*S, rank] with row stride ld, cache [Bmax, Smax, ldc] (ldc % 8 == 0, columns from `rank` on are set to zero).
+ * A position outside the cache sets *err = LR_DEV_POS_RANGE. */
+int lr_latent_update(const void* c, int64_t ld, const void* gain, const int32_t* pos, void* cache, int B, int S, int rank,
+                     int ldc, int Smax, float eps, int dtype, int32_t* err, lr_stream_t stream);
+
+/* The n cache rows a portion of S tokens at positions pos[0] .. pos[0] + S - 1 can see through a sliding window, n =
+ * min(S + window - 1, Smax), as a dense [B, n, ldc]: row j is position base + j with base = max(0, pos[0] - window + 1),
+ * or 0 when n == Smax. */
+int lr_latent_window(const void* cache, const int32_t* pos, void* rows, int B, int n, int window, int ldc, int Smax,
+                     int dtype, lr_stream_t stream);
+
+/* Sliding-window softmax attention of S queries per sequence over keys and values expanded from such rows: position i
+ * sees positions i - window + 1 .. i.  q [B*S, H*dk] (row stride ldq), k and v: column ranges [B * n_keys, H*dk] and
+ * [B * n_keys, H*dv] of buffers with row stride ldk, rows as lr_latent_window orders them; y [B*S, H*dv].
+ * score = (q . k) * scale; scores, softmax and sums in fp32. */
+typedef struct lr_window_attention {
+  const void* q;
+  int64_t ldq;
+  const void *k, *v;
+  int64_t ldk;
+  void* y;
+  int64_t ldy;
+  const int32_t* pos;
+  int32_t B, S, H, dk, dv, window, n_keys, Smax, dtype;
+  float scale;
+} lr_window_attention_t;
+int lr_window_attention(const lr_window_attention_t* desc, lr_stream_t stream);
+
+/* The same attention straight on the latent cache, for single tokens and short portions: with k = W_uk c and v = W_uv c
+ * per head, scores are ((W_uk^T q) . c) * scale and the output W_uv (sum of weights times c).  uk [H*dk, ldr], uv
+ * [H*dv, ldr], cache [Bmax, Smax, ldr] (columns beyond the rank zero in all three); the portion's own latents must be in
+ * the cache.  ldr <= 1024. */
+typedef struct lr_latent_attention {
+  const void* q;
+  int64_t ldq;
+  const void *uk, *uv, *cache;
+  void* y;
+  int64_t ldy;
+  const int32_t* pos;
+  void* scratch;
+  size_t scratch_bytes;
+  int32_t B, S, H, dk, dv, ldr, window, Smax, dtype;
+  float scale;
+} lr_latent_attention_t;
+size_t lr_latent_attention_scratch_bytes(int B, int S, int H, int ldr, int Smax);
+int lr_latent_attention(const lr_latent_attention_t* desc, lr_stream_t stream);
+
 #ifdef __cplusplus
 }
 #endif

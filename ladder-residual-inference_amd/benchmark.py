@@ -8,7 +8,8 @@ generations; prefill and decode timed separately between device synchronisations
 metric lines.  Added: --greedy (argmax on the device, lowest index on ties), --seed (weights
 N(0, 0.02) for every parameter and the prompt come from one seeded device generator),
 --virtual_tp / --tp_rank / --shard_vocab (build the layers at 1/N size without any process group),
---last_logits_only, --json.
+--last_logits_only, --checkpoint (a folder with config.json and weights instead of a named shape and random
+weights), --json.
 
 There is no compiler in this build: --compile and --cuda_graph both select hipGraph replay of a
 captured decode step (the captured step also copies the new token and advances the position on
@@ -26,7 +27,7 @@ import torch
 
 sys.path.insert(0, str(Path(__file__).parent.resolve()))
 
-from gpt_fast import GPTDense, GPTDesync, GPTLadder, GPTParallel, _hip, set_virtual_tp  # noqa: E402
+from gpt_fast import GPTDense, GPTDesync, GPTLadder, GPTLasivik, GPTParallel, _hip, set_virtual_tp  # noqa: E402
 from gpt_fast.utils import _get_model_size, set_flash_attention  # noqa: E402
 
 default_device = "cuda" if torch.cuda.is_available() else "cpu"
@@ -36,6 +37,7 @@ _MODELS = {
     "gpt_desync": GPTDesync,
     "gpt_parallel": GPTParallel,
     "gpt_ladder": GPTLadder,
+    "gpt_lasivik": GPTLasivik,
 }
 
 HBM_PEAK_GBPS = 8000.0  # MI355X HBM3E, vendor figure
@@ -171,6 +173,8 @@ class DecodeGraph:
             _hip.advance(self.cur_token, nxt.contiguous(), self.input_pos, batch_size, self.history, pos0=prompt_len)
             return nxt
 
+        # the warm-up steps are real steps: a recurrent state they advance is put back
+        states = [(s, s.clone()) for s in getattr(model, "recurrent_states", list)()]
         side = torch.cuda.Stream()
         side.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(side):
@@ -180,6 +184,8 @@ class DecodeGraph:
         self.graph = torch.cuda.CUDAGraph()
         with torch.cuda.graph(self.graph):
             self.next_token = step()
+        for s, kept in states:
+            s.copy_(kept)
 
     def reset(self, first_token: torch.Tensor):
         self.cur_token.copy_(first_token.view(self.B, 1))
@@ -278,7 +284,10 @@ def _load_model(model_name, device, precision, seed: Optional[int] = None, verbo
 
 def decode_bytes_per_step(cfg, batch_size: int, pos: int) -> int:
     """Algorithmic HBM bytes of one decode step at position `pos` (bf16): every weight and gain of
-    the shard once, the valid K and V rows, the new K/V rows, the embedding rows."""
+    the shard once, the valid K and V rows, the new K/V rows, the embedding rows.  `cfg`: a ModelArgs, or a model that
+    counts its own (decode_bytes)."""
+    if hasattr(cfg, "decode_bytes"):
+        return cfg.decode_bytes(batch_size, pos)
     D, L, hd = cfg.dim, cfg.n_layer, cfg.head_dim
     Hq, Hkv, I, V = cfg.n_head_local, cfg.n_kv_local, cfg.ffn_local, cfg.output_rows
     weights = L * (D * (Hq + 2 * Hkv) * hd + D * Hq * hd + D * 2 * I + I * D + 2 * D) + V * D + D
@@ -297,7 +306,7 @@ def main(model_name: str, prompt_length: int = 1, num_samples: int = 5, max_new_
          compile_prefill: bool = False, profile: Optional[Path] = None, device=default_device,
          use_cuda_graphs: bool = False, greedy: bool = False, seed: Optional[int] = None,
          precision=torch.bfloat16, last_logits_only: bool = False, json_path: Optional[Path] = None,
-         warmup: int = 5):
+         warmup: int = 5, checkpoint: Optional[Path] = None):
     from gpt_fast import maybe_init_dist
 
     rank = maybe_init_dist()
@@ -307,7 +316,13 @@ def main(model_name: str, prompt_length: int = 1, num_samples: int = 5, max_new_
     print_rank_0(f"Using device={device}")
     print_rank_0("Loading model ...")
     t0 = time.time()
-    model = _load_model(model_name, device, precision, seed)
+    if checkpoint is not None:
+        from gpt_fast.checkpoint import load_pretrained
+
+        model = load_pretrained(str(checkpoint), device, precision)
+        print_rank_0(model)
+    else:
+        model = _load_model(model_name, device, precision, seed)
     model.last_logits_only = last_logits_only
     device_sync(device)
     print_rank_0(f"Time to load model: {time.time() - t0:.02f} seconds")
@@ -406,7 +421,7 @@ def main(model_name: str, prompt_length: int = 1, num_samples: int = 5, max_new_
     steps = max(max_new_tokens - 1, 1)
     ms_per_token = mean("decode_latency") / steps * 1e3
     mid_pos = prompt_length + steps // 2
-    step_bytes = decode_bytes_per_step(cfg, batch_size, mid_pos)
+    step_bytes = decode_bytes_per_step(model if hasattr(model, "decode_bytes") else cfg, batch_size, mid_pos)
     gbps = step_bytes / (ms_per_token * 1e-3) / 1e9
     print_rank_0("==========")
     print_rank_0(f"Batch Size: {batch_size}")
@@ -419,7 +434,7 @@ def main(model_name: str, prompt_length: int = 1, num_samples: int = 5, max_new_
     print_rank_0(f"Decode: {ms_per_token:.3f} ms/token, {batch_size * 1e3 / ms_per_token:.1f} tok/s, "
                  f"{gbps:.0f} GB/s algorithmic = {100 * gbps / HBM_PEAK_GBPS:.1f} % of {HBM_PEAK_GBPS:.0f} GB/s")
     print_rank_0(f"Memory used: {torch.cuda.max_memory_reserved() / 1e9:.02f} GB")
-    result = dict(model_name=model_name, batch_size=batch_size, prompt_length=prompt_length,
+    result = dict(model_name=model_name or str(checkpoint), batch_size=batch_size, prompt_length=prompt_length,
                   max_new_tokens=max_new_tokens, ms_per_token=ms_per_token,
                   decode_tok_per_s=batch_size * 1e3 / ms_per_token, prefill_latency_s=mean("prefill_latency"),
                   decode_latency_s=mean("decode_latency"), algorithmic_bytes_per_step=step_bytes,
@@ -433,7 +448,11 @@ def main(model_name: str, prompt_length: int = 1, num_samples: int = 5, max_new_
 
 def build_parser():
     p = argparse.ArgumentParser(description="Per-rank Ladder-Residual inference benchmark on MI355X (HIP backend).")
-    p.add_argument("--model_name", type=str, required=True, help="family:config, e.g. gpt_ladder:ladder-70b-tp8")
+    p.add_argument("--model_name", type=str, default=None, help="family:config, e.g. gpt_ladder:ladder-70b-tp8")
+    p.add_argument("--checkpoint", type=Path, default=None,
+                   help="folder with config.json and weights; the model is chosen by config.json")
+    p.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16",
+                   help="float32: families that run in true 32-bit (gpt_lasivik)")
     p.add_argument("--prompt_length", type=int, required=True, help="Input prompt length")
     p.add_argument("--num_samples", type=int, default=5, help="Number of samples.")
     p.add_argument("--max_new_tokens", type=int, default=200, help="Maximum number of new tokens.")
@@ -460,6 +479,8 @@ def build_parser():
 
 if __name__ == "__main__":
     args = build_parser().parse_args()
+    if (args.model_name is None) == (args.checkpoint is None):
+        raise SystemExit("give either --model_name or --checkpoint")
     if args.cuda_graph:
         assert not args.compile
     if args.shard_vocab and not args.virtual_tp:
@@ -471,4 +492,4 @@ if __name__ == "__main__":
         main(args.model_name, args.prompt_length, args.num_samples, args.max_new_tokens, args.batch_size, args.top_k,
              args.temperature, args.compile, args.compile_prefill, args.profile, args.device, args.cuda_graph,
              greedy=args.greedy, seed=args.seed, last_logits_only=args.last_logits_only, json_path=args.json,
-             warmup=args.warmup)
+             warmup=args.warmup, checkpoint=args.checkpoint, precision=getattr(torch, args.dtype))

@@ -1,7 +1,8 @@
 """Builds libladder_hip.so (gfx950) from csrc/*.hip with plain hipcc: no torch headers, no cmake.
 
-    python build.py            # compile what changed, link
-    python build.py --force    # recompile everything
+    python build.py                    # compile what changed, link
+    python build.py --force            # recompile everything
+    python build.py --family lasivik   # only what one model family calls, as a library of its own
 
 The shared library lands next to the Python package (gpt_fast/libladder_hip.so), in-tree, so that
 it travels with the sources to a GPU machine.  hipcc cross-compiles without a GPU."""
@@ -17,10 +18,17 @@ OBJ = os.path.join(HERE, "build")
 LIB = os.path.join(HERE, "gpt_fast", "libladder_hip.so")
 PROF_LIB = os.path.join(HERE, "gpt_fast", "libladder_hip_prof.so")
 BAND_PROF_LIB = os.path.join(HERE, "gpt_fast", "libladder_hip_bandprof.so")
-HEADERS = [os.path.join(CSRC, h) for h in ("lr_common.h", "attn_decode_item.h", "stream_band.h")] + \
+HEADERS = [os.path.join(CSRC, h) for h in ("lr_common.h", "mixer_common.h", "attn_decode_item.h", "stream_band.h")] + \
     [os.path.join(HERE, "..", "include", "ladder_hip.h")]
 # sources that compile another source under a switch
 INCLUDES = {"ladder_step_fp8.hip": [os.path.join(CSRC, "ladder_step.hip")]}
+
+# the sources behind a model family's kernels: a checkout without a built library serves such a model
+# after compiling these
+FAMILY_SOURCES = {
+    "lasivik": ("attention.hip", "elementwise.hip", "gemm.hip", "gemv.hip", "latent_attention.hip", "linear_attention.hip",
+                "residual.hip", "sample.hip", "stream_gemm.hip"),
+}
 
 FLAGS = [
     "--offload-arch=gfx950", "-O3", "-fPIC", "-std=c++17",
@@ -72,6 +80,39 @@ def build(force=False, verbose=True):
     return LIB
 
 
+def build_family(family, force=False, verbose=True):
+    """gpt_fast/libladder_hip_<family>.so: the entry points one model family uses."""
+    os.makedirs(OBJ, exist_ok=True)
+    srcs = [os.path.join(CSRC, f) for f in FAMILY_SOURCES[family]]
+    lib = LIB.replace(".so", f"_{family}.so")
+    with ThreadPoolExecutor(max_workers=min(8, len(srcs))) as ex:
+        res = list(ex.map(lambda s: _compile(s, force), srcs))
+    objs = [o for o, _ in res]
+    if force or any(c for _, c in res) or _stale(lib, objs):
+        part = lib + f".{os.getpid()}"
+        r = subprocess.run(["hipcc", "--offload-arch=gfx950", "-shared", "-fPIC", "-o", part] + objs,
+                           capture_output=True, text=True)
+        if r.returncode != 0:
+            raise RuntimeError("link failed:\n" + r.stderr)
+        os.replace(part, lib)
+    if verbose:
+        print(f"built {lib}")
+    return lib
+
+
+def ready_for(family, verbose=True):
+    """Path of a library that serves `family`: the full one if it is there and up to date, else the family's own, compiled
+    if need be (the full one for a family that has no list of its own)."""
+    deps = sorted(os.path.join(CSRC, f) for f in os.listdir(CSRC)) + HEADERS
+    if not _stale(LIB, deps):
+        return LIB
+    if family not in FAMILY_SOURCES:
+        return build(verbose=verbose)
+    own = LIB.replace(".so", f"_{family}.so")
+    srcs = [os.path.join(CSRC, f) for f in FAMILY_SOURCES[family]]
+    return build_family(family, verbose=verbose) if _stale(own, srcs + HEADERS) else own
+
+
 def _build_variant(lib, sources, define, suffix, force, verbose):
     """`lib` = the product objects, with `sources` recompiled under `define`."""
     build(force=force, verbose=False)
@@ -110,7 +151,11 @@ if __name__ == "__main__":
                     help="also build libladder_hip_prof.so (decode-step kernel with per-phase time stamps)")
     ap.add_argument("--profile-bands", action="store_true",
                     help="also build libladder_hip_bandprof.so (band kernel with per-wave time stamps)")
+    ap.add_argument("--family", choices=sorted(FAMILY_SOURCES), help="build only this family's library")
     args = ap.parse_args()
+    if args.family:
+        build_family(args.family, force=args.force)
+        sys.exit(0)
     build(force=args.force)
     if args.profile_step:
         build_step_profile(force=args.force)

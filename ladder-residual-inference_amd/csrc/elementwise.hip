@@ -384,21 +384,30 @@ __device__ __forceinline__ void amax_merge(float& bv, int& bi, float v, int i) {
   if (v > bv || (v == bv && i < bi)) { bv = v; bi = i; }
 }
 
-__global__ __launch_bounds__(1024) void k_argmax(const u16* __restrict__ logits, int64_t ldl,
+__device__ __forceinline__ void logits8(const u16* p, float* f) { unpack8(ld16(p), f); }
+__device__ __forceinline__ void logits8(const float* p, float* f) {
+#pragma unroll
+  for (int j = 0; j < 8; ++j) f[j] = p[j];
+}
+__device__ __forceinline__ float logit1(const u16* p) { return bf_to_f(*p); }
+__device__ __forceinline__ float logit1(const float* p) { return *p; }
+
+template <typename T>
+__global__ __launch_bounds__(1024) void k_argmax(const T* __restrict__ logits, int64_t ldl,
                                                  int32_t* __restrict__ out, int V) {
   __shared__ float sv[16];
   __shared__ int si[16];
-  const u16* row = logits + (int64_t)blockIdx.x * ldl;
+  const T* row = logits + (int64_t)blockIdx.x * ldl;
   float bv = -INFINITY;
   int bi = 0x7fffffff;
   const int V8 = V & ~7;
   for (int c = threadIdx.x * 8; c < V8; c += 1024 * 8) {
     float f[8];
-    unpack8(ld16(row + c), f);
+    logits8(row + c, f);
 #pragma unroll
     for (int j = 0; j < 8; ++j) amax_merge(bv, bi, f[j], c + j);
   }
-  for (int c = V8 + threadIdx.x; c < V; c += 1024) amax_merge(bv, bi, bf_to_f(row[c]), c);
+  for (int c = V8 + threadIdx.x; c < V; c += 1024) amax_merge(bv, bi, logit1(row + c), c);
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) {
     const float ov = __shfl_xor(bv, o, LR_WAVE);
@@ -418,7 +427,15 @@ extern "C" int lr_argmax(const void* logits, int64_t ldl, int32_t* out, int B, i
   if (out == nullptr) return LR_E_NULL;
   if (B <= 0 || V <= 0 || ldl < V) return LR_E_SHAPE;
   if (ldl % 8) return LR_E_ALIGN;
-  k_argmax<<<dim3(B), dim3(1024), 0, (hipStream_t)stream>>>((const u16*)logits, ldl, out, V);
+  k_argmax<u16><<<dim3(B), dim3(1024), 0, (hipStream_t)stream>>>((const u16*)logits, ldl, out, V);
+  return lr_launch_status();
+}
+
+extern "C" int lr_argmax_f32(const float* logits, int64_t ldl, int32_t* out, int B, int V, lr_stream_t stream) {
+  LR_REQUIRE_PTR(logits);
+  if (out == nullptr) return LR_E_NULL;
+  if (B <= 0 || V <= 0 || ldl < V) return LR_E_SHAPE;
+  k_argmax<float><<<dim3(B), dim3(1024), 0, (hipStream_t)stream>>>(logits, ldl, out, V);
   return lr_launch_status();
 }
 

@@ -3,7 +3,8 @@
 from .gpt_dense_TP import GPTDense
 from .gpt_desync_TP import GPTDesync
 from .gpt_ladder_TP import GPTLadder
+from .gpt_lasivik import GPTLasivik
 from .gpt_parallel_TP import GPTParallel
 from .tp import maybe_init_dist, set_virtual_tp
 
-__all__ = ["GPTDense", "GPTDesync", "GPTLadder", "GPTParallel", "maybe_init_dist", "set_virtual_tp"]
+__all__ = ["GPTDense", "GPTDesync", "GPTLadder", "GPTLasivik", "GPTParallel", "maybe_init_dist", "set_virtual_tp"]

@@ -63,6 +63,22 @@ _PROTOS = {
                                           c_void_p, c_void_p, c_int64, c_int, c_int, c_void_p, c_size_t, c_void_p]),
     "lr_ladder_step_fail_offset": (c_size_t, []),
     "lr_ladder_step_resident_workgroups": (c_int, [c_void_p, c_int]),
+    "lr_embed_residual": (c_int, [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int64, c_int, c_int, c_float, c_int,
+                                  c_void_p]),
+    "lr_residual_rmsnorm": (c_int, [c_void_p, c_float, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_int, c_int,
+                                    c_int, c_float, c_int, c_void_p]),
+    "lr_logit_cap": (c_int, [c_void_p, c_int64, c_int, c_int, c_float, c_float, c_int, c_void_p]),
+    "lr_linear_f32": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_void_p]),
+    "lr_swiglu_f32": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_int, c_void_p]),
+    "lr_argmax_f32": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_int, c_void_p]),
+    "lr_linear_attention_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
+    "lr_linear_attention": (c_int, [c_void_p, c_void_p]),
+    "lr_latent_update": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
+                                 c_float, c_int, c_void_p, c_void_p]),
+    "lr_latent_window": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p]),
+    "lr_window_attention": (c_int, [c_void_p, c_void_p]),
+    "lr_latent_attention_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int]),
+    "lr_latent_attention": (c_int, [c_void_p, c_void_p]),
 }
 
 
@@ -84,6 +100,14 @@ def lib_path() -> str:
     return _LIB_PATH
 
 
+def use_library(path: str):
+    """Load `path` instead of the full library: one that holds the entry points of a single model family (build.py
+    --family).  Before the first call only; calling an entry point it lacks raises AttributeError."""
+    global _LIB_PATH
+    assert _lib is None or path == _LIB_PATH, "a library is loaded already"
+    _LIB_PATH = path
+
+
 def load():
     """Load the shared library once.  Raises if it has not been built."""
     global _lib
@@ -93,7 +117,10 @@ def load():
                 f"{_LIB_PATH} is missing: build it with `python {os.path.dirname(os.path.dirname(_LIB_PATH))}/build.py` "
                 "(hipcc, gfx950).  This package has no CPU or PyTorch fallback.")
         lib = ctypes.CDLL(_LIB_PATH)
+        whole = os.path.basename(_LIB_PATH) == "libladder_hip.so"
         for name, (res, args) in _PROTOS.items():
+            if not whole and not hasattr(lib, name):
+                continue
             fn = getattr(lib, name)
             fn.restype = res
             fn.argtypes = args
@@ -186,7 +213,11 @@ def linear(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, act_swiglu: bool
     assert w.is_contiguous() and xc == (2 * K if act_swiglu else K), (x.shape, w.shape, act_swiglu)
     Mo, No, ldy = _rows_ld(out)
     assert (Mo, No) == (M, N), (out.shape, M, N)
-    if gemv_cfg:
+    if w.dtype == torch.float32:
+        assert not act_swiglu and not gemv_cfg
+        f = torch.float32
+        _check(load().lr_linear_f32(_dev(x, f), ldx, _dev(w, f), _dev(out, f), ldy, M, N, K, _stream()), "lr_linear_f32")
+    elif gemv_cfg:
         _check(load().lr_linear_tuned(_dev(x), ldx, _dev(w), _dev(out), ldy, M, N, K, int(act_swiglu), int(gemv_cfg),
                                       _stream()), "lr_linear_tuned")
     else:
@@ -393,6 +424,10 @@ def module_linear_swiglu(h: torch.Tensor, mod, out: torch.Tensor, act: torch.Ten
 def swiglu(h: torch.Tensor, out: torch.Tensor):
     rows, two_i, ldh = _rows_ld(h)
     assert out.is_contiguous() and out.numel() == rows * (two_i // 2)
+    if h.dtype == torch.float32:
+        _check(load().lr_swiglu_f32(_dev(h, h.dtype), ldh, _dev(out, h.dtype), rows, two_i // 2, _stream()),
+               "lr_swiglu_f32")
+        return out
     _check(load().lr_swiglu(_dev(h), ldh, _dev(out), rows, two_i // 2, _stream()), "lr_swiglu")
     return out
 
@@ -522,6 +557,9 @@ def stream_read(buf: torch.Tensor, sink: torch.Tensor):
 def argmax(logits: torch.Tensor, out: torch.Tensor):
     B, V, ld = _rows_ld(logits)
     assert out.dtype == torch.int32 and out.numel() == B and out.is_cuda
+    if logits.dtype == torch.float32:
+        _check(load().lr_argmax_f32(_dev(logits, logits.dtype), ld, out.data_ptr(), B, V, _stream()), "lr_argmax_f32")
+        return out
     _check(load().lr_argmax(_dev(logits), ld, out.data_ptr(), B, V, _stream()), "lr_argmax")
     return out
 
@@ -550,6 +588,176 @@ def advance(cur_token, next_token, pos, B, history=None, pos0=0):
     ld, n = (history.stride(0), history.shape[1]) if history is not None else (0, 0)
     _check(load().lr_advance(p(cur_token), p(next_token), p(pos), B, p(history), ld, n, int(pos0), _stream()),
            "lr_advance")
+
+
+# ------------------------------------------------------------------------------------------------
+# fp32 residual stream, linear attention, latent attention
+# ------------------------------------------------------------------------------------------------
+
+_DTYPES = {torch.bfloat16: 0, torch.float32: 1}   # LR_BF16, LR_F32
+
+
+def _opt(t, dtype):
+    return None if t is None else _dev(t, dtype)
+
+
+def embed_residual(table, idx, x, x_compute, scale: float):
+    """x = table[idx] * scale in fp32 and x_compute (may be None) the same in the table's dtype."""
+    assert idx.dtype in (torch.int64, torch.int32) and idx.is_contiguous() and idx.is_cuda and table.is_contiguous()
+    vocab, dim = table.shape
+    for t in (x, x_compute):
+        assert t is None or (t.is_contiguous() and t.numel() == idx.numel() * dim)
+    _check(load().lr_embed_residual(_dev(table, table.dtype), idx.data_ptr(), int(idx.dtype == torch.int64),
+                                    _dev(x, torch.float32), _opt(x_compute, table.dtype), idx.numel(), dim, vocab,
+                                    float(scale), _DTYPES[table.dtype], _stream()), "lr_embed_residual")
+
+
+def residual_rmsnorm(x, alpha: float, d, gain, x_out, x_compute, eps: float, width: int = None, gain_offset: float = 0.0):
+    """rms_norm(alpha * x + d) * (gain_offset + gain); x and x_out fp32, d, gain and x_compute in the compute type."""
+    dim = x.shape[-1]
+    rows = x.numel() // dim
+    for t in (x, d, x_out, x_compute):
+        assert t is None or (t.is_contiguous() and t.numel() == rows * dim)
+    assert gain.numel() == dim and gain.is_contiguous()
+    _check(load().lr_residual_rmsnorm(_dev(x, torch.float32), float(alpha), _opt(d, gain.dtype), _dev(gain, gain.dtype),
+                                      float(gain_offset), _opt(x_out, torch.float32), _opt(x_compute, gain.dtype), rows, dim,
+                                      dim if width is None else width, float(eps), _DTYPES[gain.dtype], _stream()),
+           "lr_residual_rmsnorm")
+
+
+def logit_cap(logits, scale: float, cap: float):
+    """logits = cap * tanh(scale * logits / cap) in place (cap 0: the scale alone)."""
+    rows, V, ld = _rows_ld(logits)
+    _check(load().lr_logit_cap(_dev(logits, logits.dtype), ld, rows, V, float(scale), float(cap), _DTYPES[logits.dtype],
+                               _stream()), "lr_logit_cap")
+    return logits
+
+
+class _LinearAttention(ctypes.Structure):   # lr_linear_attention_t
+    _fields_ = [("q", c_void_p), ("k", c_void_p), ("v", c_void_p), ("g", c_void_p), ("ld", c_int64),
+                ("lowrank", c_void_p), ("a2", c_void_p), ("a_bias", c_void_p), ("head_decay", c_void_p), ("rope", c_void_p),
+                ("pos", c_void_p), ("state", c_void_p), ("norm", c_void_p), ("y", c_void_p), ("ldy", c_int64),
+                ("err", c_void_p), ("scratch", c_void_p), ("scratch_bytes", c_size_t)] + \
+               [(n, c_int32) for n in ("B", "S", "H", "dk", "dv", "rank", "rot_dims", "rope_len", "dtype")] + \
+               [(n, c_float) for n in ("tau", "q_scale", "k_scale", "eps")]
+
+
+def linear_attention_scratch_bytes(B, S, H, dk, dv, gated) -> int:
+    return int(load().lr_linear_attention_scratch_bytes(B, S, H, dk, dv, int(gated)))
+
+
+def linear_attention(proj, y, state, pos, B, S, H, dk, dv, eps, scratch=None, q_scale=1.0, k_scale=1.0, norm=None,
+                     gate=None, head_decay=None, rope=None):
+    """Linear attention with decay over S tokens of B sequences (lr_linear_attention).  proj [B * S, ld]: columns
+    q [H dk] | k [H dk] | v [H dv] | g [H dv] | low-rank decay input; y [B * S, >= H dv]; state fp32 [>= B, H, dk, dv].
+    gate = (a2 [H dk, rank], bias [H dk], tau): a decay per key channel; else head_decay, fp32 [H] log-decays.
+    rope fp32 [positions, dims / 2, 2] or None; norm [dv] or None."""
+    f32 = torch.float32
+    rows, cols, ld = _rows_ld(proj)
+    yrows, ycols, ldy = _rows_ld(y)
+    nq, nv = H * dk, H * dv
+    dt = proj.dtype
+    rank, tau, a2, bias = 0, 1.0, None, None
+    if gate is not None:
+        a2, bias, tau = gate
+        rank = a2.shape[1]
+        assert a2.is_contiguous() and a2.shape[0] == nq and bias.numel() == nq and bias.is_contiguous()
+    else:
+        assert head_decay is not None and head_decay.numel() == H
+    assert rows == yrows == B * S and cols >= 2 * nq + 2 * nv + rank and ycols >= nv and y.dtype == dt
+    assert state.is_contiguous() and state.shape[0] >= B and tuple(state.shape[1:]) == (H, dk, dv)
+    assert pos.dtype == torch.int32 and pos.is_cuda and pos.numel() == S
+    assert norm is None or (norm.numel() == dv and norm.is_contiguous())
+    rot_dims, rope_len = 0, 0
+    if rope is not None:
+        assert rope.is_contiguous() and rope.shape[2] == 2
+        rope_len, rot_dims = rope.shape[0], 2 * rope.shape[1]
+    es = proj.element_size()
+    p = _dev(proj, dt)
+    d = _LinearAttention(
+        q=p, k=p + nq * es, v=p + 2 * nq * es, g=p + (2 * nq + nv) * es, ld=ld,
+        lowrank=None if gate is None else p + (2 * nq + 2 * nv) * es, a2=_opt(a2, dt), a_bias=_opt(bias, dt),
+        head_decay=_opt(head_decay, f32) if gate is None else None, rope=_opt(rope, f32), pos=pos.data_ptr(),
+        state=_dev(state, f32), norm=_opt(norm, dt), y=_dev(y, dt), ldy=ldy,
+        err=device_error_word(proj.device).data_ptr(),
+        scratch=None if scratch is None else scratch.data_ptr(),
+        scratch_bytes=0 if scratch is None else scratch.numel() * scratch.element_size(),
+        B=B, S=S, H=H, dk=dk, dv=dv, rank=rank, rot_dims=rot_dims, rope_len=rope_len, dtype=_DTYPES[dt],
+        tau=tau, q_scale=q_scale, k_scale=k_scale, eps=eps)
+    _check(load().lr_linear_attention(ctypes.byref(d), _stream()), "lr_linear_attention")
+    return y
+
+
+def latent_update(c, gain, pos, cache, B, S, rank, eps: float):
+    """Normalised latents of B * S rows c [B * S, >= rank] into cache [>= B, Smax, ldc] at their positions."""
+    rows, cols, ld = _rows_ld(c)
+    assert rows == B * S and cols >= rank and pos.dtype == torch.int32 and pos.numel() == S and cache.is_contiguous()
+    assert cache.shape[0] >= B and gain.numel() >= rank and cache.dtype == c.dtype
+    assert c.is_cuda
+    _check(load().lr_latent_update(c.data_ptr(), ld, _dev(gain, c.dtype), pos.data_ptr(), _dev(cache, c.dtype), B, S, rank,
+                                   cache.shape[2], cache.shape[1], float(eps), _DTYPES[c.dtype],
+                                   device_error_word(c.device).data_ptr(), _stream()), "lr_latent_update")
+
+
+def latent_window(cache, pos, rows, B, window: int):
+    """The cache rows [B, n, ldc] a portion starting at pos[0] can see (n = rows.shape[1])."""
+    assert cache.is_contiguous() and rows.is_contiguous() and rows.shape[0] == B and rows.shape[2] == cache.shape[2]
+    assert pos.dtype == torch.int32 and pos.is_cuda and cache.shape[0] >= B
+    _check(load().lr_latent_window(_dev(cache, cache.dtype), pos.data_ptr(), _dev(rows, cache.dtype), B, rows.shape[1],
+                                   int(window), cache.shape[2], cache.shape[1], _DTYPES[cache.dtype], _stream()),
+           "lr_latent_window")
+    return rows
+
+
+class _WindowAttention(ctypes.Structure):   # lr_window_attention_t
+    _fields_ = [("q", c_void_p), ("ldq", c_int64), ("k", c_void_p), ("v", c_void_p), ("ldk", c_int64), ("y", c_void_p),
+                ("ldy", c_int64), ("pos", c_void_p)] + \
+               [(n, c_int32) for n in ("B", "S", "H", "dk", "dv", "window", "n_keys", "Smax", "dtype")] + \
+               [("scale", c_float)]
+
+
+def window_attention(q, kv, y, pos, B, S, H, dk, dv, window: int, n_keys: int, Smax: int, scale: float):
+    """Sliding-window attention of S queries per sequence; kv [B * n_keys, >= H dk + H dv] = k | v of the rows
+    latent_window hands out."""
+    _, qc, ldq = _rows_ld(q)
+    krows, kcols, ldk = _rows_ld(kv)
+    _, yc, ldy = _rows_ld(y)
+    assert qc >= H * dk and krows == B * n_keys and kcols >= H * (dk + dv) and yc >= H * dv
+    assert pos.dtype == torch.int32 and pos.numel() == S and q.dtype == kv.dtype == y.dtype
+    es = kv.element_size()
+    d = _WindowAttention(q=_dev(q, q.dtype), ldq=ldq, k=_dev(kv, q.dtype), v=kv.data_ptr() + H * dk * es, ldk=ldk,
+                         y=_dev(y, q.dtype), ldy=ldy, pos=pos.data_ptr(), B=B, S=S, H=H, dk=dk, dv=dv, window=int(window),
+                         n_keys=n_keys, Smax=Smax, dtype=_DTYPES[q.dtype], scale=scale)
+    _check(load().lr_window_attention(ctypes.byref(d), _stream()), "lr_window_attention")
+    return y
+
+
+class _LatentAttention(ctypes.Structure):   # lr_latent_attention_t
+    _fields_ = [("q", c_void_p), ("ldq", c_int64), ("uk", c_void_p), ("uv", c_void_p), ("cache", c_void_p),
+                ("y", c_void_p), ("ldy", c_int64), ("pos", c_void_p), ("scratch", c_void_p), ("scratch_bytes", c_size_t)] + \
+               [(n, c_int32) for n in ("B", "S", "H", "dk", "dv", "ldr", "window", "Smax", "dtype")] + \
+               [("scale", c_float)]
+
+
+def latent_attention_scratch_bytes(B, S, H, ldr, Smax) -> int:
+    return int(load().lr_latent_attention_scratch_bytes(B, S, H, ldr, Smax))
+
+
+def latent_attention(q, uk, uv, cache, y, pos, scratch, B, S, H, dk, dv, window: int, scale: float):
+    """Sliding-window attention of short portions straight on the latent cache [>= B, Smax, ldr]."""
+    rows, qc, ldq = _rows_ld(q)
+    _, yc, ldy = _rows_ld(y)
+    ldr = cache.shape[2]
+    assert rows == B * S and qc >= H * dk and yc >= H * dv and cache.is_contiguous() and cache.shape[0] >= B
+    assert uk.is_contiguous() and uv.is_contiguous() and tuple(uk.shape) == (H * dk, ldr) and tuple(uv.shape) == (H * dv, ldr)
+    assert pos.dtype == torch.int32 and pos.numel() == S
+    dt = q.dtype
+    d = _LatentAttention(q=_dev(q, dt), ldq=ldq, uk=_dev(uk, dt), uv=_dev(uv, dt), cache=_dev(cache, dt), y=_dev(y, dt),
+                         ldy=ldy, pos=pos.data_ptr(), scratch=scratch.data_ptr(),
+                         scratch_bytes=scratch.numel() * scratch.element_size(), B=B, S=S, H=H, dk=dk, dv=dv, ldr=ldr,
+                         window=int(window), Smax=cache.shape[1], dtype=_DTYPES[dt], scale=scale)
+    _check(load().lr_latent_attention(ctypes.byref(d), _stream()), "lr_latent_attention")
+    return y
 
 
 def _ladder_model_desc(model, attention_workgroups: int = 0):

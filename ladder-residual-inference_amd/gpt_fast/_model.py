@@ -89,13 +89,7 @@ class GPTBase(nn.Module):
     def setup_caches(self, max_batch_size, max_seq_length):
         if self.max_seq_length >= max_seq_length and self.max_batch_size >= max_batch_size:
             return
-        cfg = self.config
-        if cfg.head_dim not in (64, 128):
-            raise NotImplementedError(f"head_dim {cfg.head_dim}: the attention kernels are built for 64 and 128")
-        if max_seq_length > cfg.block_size:
-            # the RoPE table has block_size rows: the reference fails with an index error at the first position
-            # beyond it (gpt_ladder_TP.py:255); here the mistake is reported before anything is allocated
-            raise ValueError(f"max_seq_length {max_seq_length} exceeds the model's block_size {cfg.block_size}")
+        self._check_caches(max_seq_length)
         max_seq_length = find_multiple(max_seq_length, 8)
         self.max_seq_length = max_seq_length
         self.max_batch_size = max_batch_size
@@ -104,16 +98,38 @@ class GPTBase(nn.Module):
         if hasattr(self.output, "scales"):
             dtype = self.output.scales.dtype
         device = self.output.weight.device
-        if dtype != torch.bfloat16:
-            raise NotImplementedError(f"the HIP kernels compute in bfloat16 storage; model dtype is {dtype}")
+        if dtype not in self.supported_dtypes:
+            raise NotImplementedError(f"the HIP kernels of this family compute in {self.supported_dtypes}; model dtype is "
+                                      f"{dtype}")
+        self._build_caches(max_batch_size, max_seq_length, dtype, device)
+        self._ws.clear()
+        _hip.device_error_word(device)  # exists before any step is captured into a graph
+
+    supported_dtypes = (torch.bfloat16,)
+
+    def _check_caches(self, max_seq_length):
+        cfg = self.config
+        if cfg.head_dim not in (64, 128):
+            raise NotImplementedError(f"head_dim {cfg.head_dim}: the attention kernels are built for 64 and 128")
+        if max_seq_length > cfg.block_size:
+            # the RoPE table has block_size rows: the reference fails with an index error at the first position
+            # beyond it (gpt_ladder_TP.py:255); here the mistake is reported before anything is allocated
+            raise ValueError(f"max_seq_length {max_seq_length} exceeds the model's block_size {cfg.block_size}")
+
+    def _build_caches(self, max_batch_size, max_seq_length, dtype, device):
+        cfg = self.config
         for b in self.layers:
             b.attention.kv_cache = KVCache(max_batch_size, max_seq_length, cfg.n_kv_local, cfg.head_dim, dtype).to(device)
         self.freqs_cis = precompute_freqs_cis(cfg.block_size, cfg.head_dim, cfg.rope_base, dtype,
                                               cfg.rope_scaling).to(device)
         # kept for API compatibility (the kernels derive visibility from input_pos)
         self.causal_mask = torch.tril(torch.ones(max_seq_length, max_seq_length, dtype=torch.bool, device=device))
-        self._ws.clear()
-        _hip.device_error_word(device)  # exists before any step is captured into a graph
+
+    def recurrent_states(self):
+        """State tensors that a step changes in place, so that running it again does something else (none here: a KV
+        cache is written by position).  Whoever runs steps for their side effects on the allocator -- a graph's
+        warm-up -- puts these back."""
+        return []
 
     def check_device_errors(self):
         """Synchronises, then raises LadderHipError if a kernel of an earlier call reported a condition
@@ -130,26 +146,34 @@ class GPTBase(nn.Module):
         key = (B, S, self.last_logits_only)
         ws = self._ws.get(key)
         if ws is None:
-            w = self.output.weight
-            ws = Workspace(self.config, B, S, self._fused_width(), w.device, self.norm.weight.dtype, self.max_seq_length,
-                           not self.last_logits_only)
+            ws = self._new_workspace(B, S)
             if S > 1:  # keep at most one prefill-sized workspace alive
                 for k in [k for k in self._ws if k[1] > 1]:
                     del self._ws[k]
             self._ws[key] = ws
         return ws
 
+    def _new_workspace(self, B: int, S: int):
+        return Workspace(self.config, B, S, self._fused_width(), self.output.weight.device, self.norm.weight.dtype,
+                         self.max_seq_length, not self.last_logits_only)
+
     # -- forward --------------------------------------------------------------------------------
     def forward(self, idx: Tensor, input_pos: Optional[Tensor] = None) -> Tensor:
-        assert self.freqs_cis is not None, "Caches must be initialized first"
+        assert self.max_batch_size > 0, "Caches must be initialized first"
         B, S = idx.shape
         assert B <= self.max_batch_size and input_pos.shape[-1] == S
         pos = _pos_i32(input_pos)
         ws = self._workspace(B, S)
         ws.next_token_valid_for = None
+        self._embed(ws, idx)
+        return self._head(ws, *self._run_layers(ws, pos))
+
+    def _embed(self, ws: Workspace, idx: Tensor):
         _hip.embed(self.tok_embeddings.weight, idx.contiguous(), ws.x)
-        final_d1, final_d2 = self._run_layers(ws, pos)
-        cfg = self.config
+
+    def _head(self, ws: Workspace, final_d1, final_d2) -> Tensor:
+        """Final norm and lm_head on ws.x plus what _run_layers left to be added."""
+        cfg, B, S = self.config, ws.B, ws.S
         if self.last_logits_only and S > 1:
             # only row S-1 of each sequence feeds the head: gather those B rows, then norm + lm_head
             last = lambda t, out: None if t is None else _hip.embed(t.view(B * S, -1), ws.last_rows, out)

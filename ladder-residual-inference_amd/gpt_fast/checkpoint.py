@@ -18,6 +18,10 @@ Three steps, each usable on its own (all on plain state dicts, CPU tensors are f
                           Separate wq / wk / wv (utils.py:178-185) are accepted and fused.
   load_checkpoint         convert if needed, shard, cast, and load into a GPT* module.
 
+  convert_lasivik_state_dict  a Lasivik checkpoint's names (`embed`, `l<i>.mix.*`, `l<i>.mlp.*`, `head`, ...) ->
+                          GPTLasivik's, projections of the same input fused, padded columns and rows zero.
+  load_pretrained         a folder with config.json and weights -> the model it describes, loaded.
+
 `model_args_from_hf_config` turns the fields of an HF config.json (hf_modeling_utils/configs/*.json)
 into ModelArgs keywords, `ladder_layers` included (configuration_llama_ladder.py:32-45)."""
 import json
@@ -26,6 +30,8 @@ from typing import Dict, List, Optional, Union
 
 import torch
 from torch import Tensor
+
+from .mixers import pad8
 
 StateDict = Dict[str, Tensor]
 
@@ -110,6 +116,79 @@ def model_args_from_hf_config(cfg: Union[str, dict], **overrides) -> dict:
 
 
 # ------------------------------------------------------------------------------------------------
+# Lasivik names -> GPTLasivik names
+# ------------------------------------------------------------------------------------------------
+
+def is_lasivik_state_dict(sd: StateDict) -> bool:
+    return "embed" in sd and "final.norm" in sd
+
+
+def lasivik_decay_ranks(sd: StateDict) -> Dict[int, int]:
+    """Layer -> rank of its decay projection."""
+    return {int(k[1:].split(".")[0]): w.shape[0] for k, w in sd.items() if k.endswith(".mix.a1")}
+
+
+def _padded(w: Tensor, *shape: int) -> Tensor:
+    """w with zeros behind it up to `shape`."""
+    if tuple(w.shape) == shape:
+        return w
+    out = w.new_zeros(shape)
+    out[tuple(slice(0, n) for n in w.shape)] = w
+    return out
+
+
+def convert_lasivik_state_dict(sd: StateDict, args) -> StateDict:
+    """Checkpoint names -> GPTLasivik parameter names for LasivikArgs `args`.  Raises on tensors the configuration does
+    not account for and on missing ones."""
+    left = dict(sd)
+    out: StateDict = {}
+    D = args.dim
+    W = args.width
+
+    def take(name: str, *shape: int) -> Tensor:
+        if name not in left:
+            raise KeyError(f"checkpoint has no tensor {name!r}")
+        w = left.pop(name)
+        if tuple(w.shape) != shape:
+            raise ValueError(f"{name}: checkpoint {tuple(w.shape)}, configuration {shape}")
+        return w
+
+    wide = lambda w: _padded(w, w.shape[0], D)          # a projection of the residual stream
+    out["tok_embeddings.weight"] = wide(take("embed", args.vocab_size, W))
+    for i, layer in enumerate(args.layers):
+        m, src, dst = layer.mixer, f"l{i}.mix.", f"layers.{i}.mixer."
+        nq, nv = m.heads * m.dim, m.heads * m.vdim
+        rows = {"q": nq}
+        if m.kind == "latent_attention":
+            rows["dkv"] = m.kv_rank
+        else:
+            rows.update(k=nq, v=nv, g=nv)
+            if m.kind == "gla":
+                rows["a1"] = m.decay_rank
+        out[dst + "in_proj.weight"] = torch.cat([wide(take(src + n, r, W)) for n, r in rows.items()])
+        out[dst + "out_proj.weight"] = _padded(take(src + "o", W, nv), D, pad8(nv))
+        if m.kind == "gla":
+            out[dst + "decay_up.weight"] = take(src + "a2", nq, m.decay_rank)
+            out[dst + "decay_up.bias"] = take(src + "a2.b", nq)
+            out[dst + "norm.weight"] = take(src + "norm", m.vdim)
+        elif m.kind == "latent_attention":
+            out[dst + "norm.weight"] = take(src + "dkv.norm", m.kv_rank)
+            up = torch.cat([take(src + "uk", nq, m.kv_rank), take(src + "uv", nv, m.kv_rank)])
+            out[dst + "kv_up.weight"] = _padded(up, nq + nv, pad8(m.kv_rank))
+        out[f"layers.{i}.mixer_norm.weight"] = _padded(take(f"l{i}.norm1", W), D)
+        if layer.ffn is not None:
+            I, Ip, src, dst = layer.ffn, pad8(layer.ffn), f"l{i}.mlp.", f"layers.{i}.feed_forward."
+            out[dst + "w1.weight"] = torch.cat([_padded(take(src + n, I, W), Ip, D) for n in ("up", "gate")])
+            out[dst + "w2.weight"] = _padded(take(src + "down", W, I), D, Ip)
+            out[f"layers.{i}.ffn_norm.weight"] = _padded(take(f"l{i}.norm2", W), D)
+    out["norm.weight"] = _padded(take("final.norm", W), D)
+    out["output.weight"] = wide(take("head", args.vocab_size, W))
+    if left:
+        raise KeyError(f"tensors the configuration does not account for: {sorted(left)[:6]}")
+    return out
+
+
+# ------------------------------------------------------------------------------------------------
 # one rank's slice of an un-sharded gpt_fast state dict
 # ------------------------------------------------------------------------------------------------
 
@@ -189,12 +268,15 @@ def read_state_dict(path: str) -> StateDict:
 
 
 def load_checkpoint(model: torch.nn.Module, checkpoint: Union[str, StateDict], already_sharded: bool = False) -> List[str]:
-    """Load an un-sharded checkpoint (HF or gpt_fast names; a path or a state dict) into `model`,
+    """Load an un-sharded checkpoint (HF, Lasivik or gpt_fast names; a path or a state dict) into `model`,
     which was built for one tensor-parallel rank (model.config.tp_world_size / tp_rank).
     Returns the names of the tensors that were loaded.  Raises on missing or unexpected
     parameters; buffers the checkpoint does not carry (KV caches, masks) are left alone."""
     cfg = model.config
     sd = read_state_dict(checkpoint) if isinstance(checkpoint, (str, os.PathLike)) else dict(checkpoint)
+    if is_lasivik_state_dict(sd):
+        sd = convert_lasivik_state_dict(sd, cfg)
+        already_sharded = True   # one rank holds all of it
     if is_hf_state_dict(sd):
         # an already sharded checkpoint holds this rank's heads only
         heads = (cfg.n_head_local, cfg.n_kv_local) if already_sharded else (cfg.n_head, cfg.n_local_heads)
@@ -222,3 +304,39 @@ def load_checkpoint(model: torch.nn.Module, checkpoint: Union[str, StateDict], a
                 raise ValueError(f"{name}: checkpoint slice {tuple(w.shape)} vs parameter {tuple(p.shape)}")
             p.copy_(w.to(dtype=p.dtype))
     return sorted(params)
+
+
+def _folder_config(folder: str) -> dict:
+    with open(os.path.join(folder, "config.json")) as f:
+        return json.load(f)
+
+
+def pretrained_class(folder: str):
+    """The model class a checkpoint folder's config.json asks for: `architecture` "Lasivik" -> GPTLasivik; a Hugging Face
+    Llama or Llama-Ladder configuration -> GPTLadder (whose layers outside `ladder_layers` are dense)."""
+    from .gpt_ladder_TP import GPTLadder
+    from .gpt_lasivik import GPTLasivik
+
+    cfg = _folder_config(folder)
+    if cfg.get("architecture") == "Lasivik":
+        return GPTLasivik
+    if "hidden_size" in cfg:
+        return GPTLadder
+    raise ValueError(f"{folder}/config.json describes no model this package has")
+
+
+def load_pretrained(folder: str, device="cuda", dtype: torch.dtype = torch.bfloat16) -> torch.nn.Module:
+    """The model a checkpoint folder (config.json and weights) describes, on `device` in `dtype`."""
+    from .config import LasivikArgs, ModelArgs
+
+    cls = pretrained_class(folder)
+    if dtype not in cls.supported_dtypes:
+        raise NotImplementedError(f"{cls.__name__} does not run in {dtype}")
+    cfg, sd = _folder_config(folder), read_state_dict(folder)
+    args = LasivikArgs.from_config(cfg, lasivik_decay_ranks(sd)) if cls.family == "lasivik" else \
+        ModelArgs(**model_args_from_hf_config(cfg))
+    with torch.device("meta"):
+        model = cls(args)
+    model = model.to(dtype=dtype).to_empty(device=device)
+    load_checkpoint(model, sd)
+    return model.eval()

@@ -11,6 +11,7 @@ from dataclasses import dataclass
 from typing import Dict, List, Optional
 
 from . import tp as _tp
+from .mixers import MixerArgs, pad8
 
 
 def find_multiple(n: int, k: int) -> int:
@@ -190,12 +191,96 @@ def _build_family(family: str) -> Dict[str, dict]:
     return reg
 
 
+# ------------------------------------------------------------------------------------------------
+# Lasivik: a hybrid whose configuration lists every layer's mixer and feed-forward
+# ------------------------------------------------------------------------------------------------
+
+@dataclass
+class LayerArgs:
+    mixer: MixerArgs
+    ffn: Optional[int]              # feed-forward width, None: the layer has none
+
+
+@dataclass
+class LasivikArgs:
+    vocab_size: int
+    width: int                      # `dim`, the padded width, is what buffers and weights have
+    layers: List[LayerArgs]
+    norm_eps: float
+    residual_scale: float           # alpha of norm(alpha x + sublayer(x))
+    embedding_scale: float
+    logit_scale: float
+    logit_softcap: float
+    block_size: int = 1 << 30       # no table limits the positions: the caches' length does
+    tp_world_size: int = 1
+
+    def __post_init__(self):
+        if _tp.get_tp_world_size() != 1:
+            raise NotImplementedError("Lasivik models run whole on one GPU: their mixers are not sharded over ranks")
+
+    @property
+    def dim(self) -> int:
+        return pad8(self.width)
+
+    @property
+    def n_layer(self) -> int:
+        return len(self.layers)
+
+    @property
+    def output_rows(self) -> int:
+        return self.vocab_size
+
+    @classmethod
+    def from_config(cls, cfg: dict, decay_ranks: Optional[Dict[int, int]] = None) -> "LasivikArgs":
+        """From a parsed config.json.  The rank of a gated linear attention's decay projection is no entry of it; a
+        checkpoint's tensors tell it (decay_ranks: layer -> rank), 16 otherwise."""
+        layers = []
+        for i, layer in enumerate(cfg["layers"]):
+            kind, m, mlp = layer["type"], layer["mixer"], layer.get("mlp")
+            kw = dict(kind=kind, heads=m["heads"], dim=m["dim"], vdim=m["vdim"])
+            if kind == "gla":
+                kw.update(tau=float(m["tau"]), decay_rank=(decay_ranks or {}).get(i, m.get("decay_rank", 16)))
+            elif kind == "retention":
+                assert len(m["decay"]) == m["heads"], "one decay per head"
+                kw.update(decay=[float(d) for d in m["decay"]], rot_dims=m["rot"]["dims"],
+                          rot_base=float(m["rot"]["base"]))
+            elif kind == "latent_attention":
+                kw.update(kv_rank=m["kv_rank"], window=m["mask"]["size"], scale=float(m["scale"]))
+            else:
+                raise ValueError(f"layer {i}: unknown mixer {kind!r}")
+            if mlp is not None and mlp["kind"] != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
+            layers.append(LayerArgs(MixerArgs(**kw), None if mlp is None else mlp["ff"]))
+        return cls(vocab_size=cfg["vocab"], width=cfg["width"], layers=layers, norm_eps=float(cfg["norm"]["eps"]),
+                   residual_scale=float(cfg["postln_alpha"]), embedding_scale=float(cfg["embedding"]["scale"]),
+                   logit_scale=float(cfg["logit_scale"]), logit_softcap=float(cfg["logit_softcap"]))
+
+
+def _lasivik_config(width: int, ff: int, vocab: int, periods: int, heads: int, window: int) -> dict:
+    """A config.json of the design: (latent attention, gla, retention, gla) `periods` times, 128 dimensions per head."""
+    latent = dict(heads=heads, dim=128, vdim=128, kv_rank=512, mask=dict(size=window), scale=128 ** -0.5)
+    gla = dict(heads=heads // 2, dim=128, vdim=256, tau=16.0)
+    retention = dict(heads=heads // 2, dim=128, vdim=256, rot=dict(dims=128, base=500000.0),
+                     decay=[1 - 2.0 ** -(5 + 4 * i / max(heads // 2 - 1, 1)) for i in range(heads // 2)])
+    order = [("latent_attention", latent), ("gla", gla), ("retention", retention), ("gla", gla)]
+    return dict(architecture="Lasivik", vocab=vocab, width=width, norm=dict(eps=1e-5), postln_alpha=(2 * 4 * periods) ** 0.25,
+                embedding=dict(scale=width ** 0.5), logit_scale=1.0, logit_softcap=30.0,
+                layers=[dict(type=t, mixer=m, mlp=dict(kind="dense", ff=ff)) for _ in range(periods) for t, m in order])
+
+
+# benchmark shapes: layers of the size of the dense "llama-3.2-1b" / "llama-3-8b"
+_LASIVIK = {
+    "lasivik-1b": _lasivik_config(2048, 8192, 128256, 4, 16, 1024),
+    "lasivik-8b": _lasivik_config(4096, 14336, 128256, 8, 32, 1024),
+}
+
 REGISTRIES = {f: _build_family(f) for f in ("ladder", "dense", "desync", "parallel")}
+REGISTRIES["lasivik"] = _LASIVIK
 
 
-def args_from_name(family: str, name: str) -> ModelArgs:
+def args_from_name(family: str, name: str):
     reg = REGISTRIES[family]
     if name not in reg:
         # the reference returns None here and fails later with an AttributeError (gpt_ladder_TP.py:59-62)
         raise KeyError(f"unknown {family} config '{name}'; known: {sorted(reg)}")
-    return ModelArgs(**reg[name])
+    return LasivikArgs.from_config(reg[name]) if family == "lasivik" else ModelArgs(**reg[name])
