@@ -258,11 +258,19 @@ __device__ __forceinline__ u32 cvt_pk_bf2(float lo, float hi) {
 }
 constexpr float PREFILL_TAU2 = 8.0f;  // log2 of the largest softmax weight before the reference point moves
 
-template <int HD, int NWH>
+struct WindowKeys {
+  int window, n_keys, ld, dk, dv;
+  float scale;
+};
+
+// WIN (lr_window_attention): a sliding window, the score scale as an argument, and keys and values of one head per query
+// head as rows of a matrix, in the order lr_latent_window gives them; head sizes up to HD.
+template <int HD, int NWH, bool WIN = false>
 __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict__ q, int64_t ldq,
                                                            const u16* __restrict__ kc, const u16* __restrict__ vc,
                                                            const int32_t* __restrict__ pos, u16* __restrict__ y,
-                                                           int64_t ldy, int S, int Hq, int Hkv, int Smax) {
+                                                           int64_t ldy, int S, int Hq, int Hkv, int Smax,
+                                                           const WindowKeys w = {}) {
   constexpr int NWQ = 4 / NWH;            // query tiles per workgroup
   constexpr int KS = HD / 16;             // k-steps of the score product
   constexpr int DT = HD / 32;             // 32-row tiles of O^T
@@ -292,7 +300,12 @@ __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict
   const int s = (bx * NWQ + wave / NWH) * 32 + col;  // this lane's query
   const bool valid = s < S;
   int p = valid ? pos[s] : -1;
-  p = p >= Smax ? Smax - 1 : p;
+  if constexpr (WIN) {
+    if (valid) p -= lr_window_base(pos[0], w.window, w.n_keys, Smax);   // this query's row among the keys
+    p = p >= w.n_keys ? w.n_keys - 1 : p;
+  } else {
+    p = p >= Smax ? Smax - 1 : p;
+  }
   // keys needed by anybody in the workgroup
   int kmax = p;
 #pragma unroll
@@ -305,14 +318,28 @@ __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict
   __syncthreads();
   kmax = max(max(s_kmax[0], s_kmax[1]), max(s_kmax[2], s_kmax[3]));
   const int nkeys = kmax + 1;
+  // (WIN) the last key of this wave's queries, and the first tile anybody in the workgroup sees
+  int pmax = 0, t_first = 0;
+  if constexpr (WIN) {
+    pmax = __builtin_amdgcn_readfirstlane(s_kmax[wave]);
+    int lo = 0x7fffffff;
+#pragma unroll
+    for (int t = 0; t < NWQ; ++t) {
+      const int s_lo = (bx * NWQ + t) * 32;   // positions are consecutive: a query tile's first query is its smallest
+      if (s_lo < S) lo = min(lo, pos[s_lo] - lr_window_base(pos[0], w.window, w.n_keys, Smax));
+    }
+    lo = lo - w.window + 1;
+    t_first = lo > 0 ? lo & ~31 : 0;
+  }
 
   // Q as B operands: k-step ks_ holds elements 16 ks_ + 8 half .. + 8 of this lane's query
   u32x4_t qb[KS];
   {
-    const u16* qrow = q + ((int64_t)b * S + (valid ? s : 0)) * ldq + head * HD;
+    const int dq = WIN ? w.dk : HD;
+    const u16* qrow = q + ((int64_t)b * S + (valid ? s : 0)) * ldq + head * dq;
 #pragma unroll
     for (int i = 0; i < KS; ++i) {
-      const uint4 t = valid ? ld16(qrow + 16 * i + 8 * half) : make_uint4(0, 0, 0, 0);
+      const uint4 t = valid && 16 * i + 8 * half < dq ? ld16(qrow + 16 * i + 8 * half) : make_uint4(0, 0, 0, 0);
       qb[i] = u32x4_t{t.x, t.y, t.z, t.w};
     }
   }
@@ -322,7 +349,7 @@ __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict
 #pragma unroll
     for (int v = 0; v < 16; ++v) o[d][v] = 0.0f;
   float m = -INFINITY, l = 0.0f;  // m: reference point in raw score units; l: this lane's half of the row sum
-  const float c2 = rsqrtf((float)HD) * 1.4426950408889634f;  // e^(x / sqrt(HD)) = 2^(x c2)
+  const float c2 = (WIN ? w.scale : rsqrtf((float)HD)) * 1.4426950408889634f;  // e^(x / sqrt(HD)) = 2^(x c2)
   const float tau_raw = PREFILL_TAU2 / c2;
   // the smallest position among the wave's queries (lanes without a query do not count)
   int pmin = valid ? p : 0x7fffffff;
@@ -332,8 +359,9 @@ __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict
     pmin = t < pmin ? t : pmin;
   }
   pmin = __builtin_amdgcn_readfirstlane(pmin);
-  const u16* kbase = kc + ((int64_t)b * Hkv + kvh) * Smax * HD;
-  const u16* vbase = vc + ((int64_t)b * Hkv + kvh) * Smax * HD;
+  const int krow = WIN ? w.ld : HD;   // elements from key to key
+  const u16* kbase = WIN ? kc + (int64_t)b * w.n_keys * w.ld + kvh * w.dk : kc + ((int64_t)b * Hkv + kvh) * Smax * HD;
+  const u16* vbase = WIN ? vc + (int64_t)b * w.n_keys * w.ld + kvh * w.dv : vc + ((int64_t)b * Hkv + kvh) * Smax * HD;
 
   // Staging: a thread owns one 8-element slice of TWO neighbouring keys (key pair kp, slice dch), so
   // that V^T can be written as whole dwords (two keys of one dimension).  The pair index is XOR-ed
@@ -347,18 +375,19 @@ __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict
   u32x4_t gk[2], gv[2];
   const __amdgpu_buffer_rsrc_t kres = __builtin_amdgcn_make_buffer_rsrc(const_cast<u16*>(kbase), 0, 0x7fffffff, 0x00020000);
   const __amdgpu_buffer_rsrc_t vres = __builtin_amdgcn_make_buffer_rsrc(const_cast<u16*>(vbase), 0, 0x7fffffff, 0x00020000);
-  const int stage_off = stager ? (2 * kp * HD + dch * 8) * 2 : (int)0x80000000;  // bytes, first key of the pair
+  const int stage_off = stager ? (2 * kp * krow + dch * 8) * 2 : (int)0x80000000;  // bytes, first key of the pair
+  const bool k_has = !WIN || dch * 8 < w.dk, v_has = !WIN || dch * 8 < w.dv;
   auto stage_load = [&](int t0) {
 #pragma unroll
     for (int e = 0; e < 2; ++e) {
-      const int off = (stager && t0 + 2 * kp + e < nkeys) ? stage_off + (t0 + e) * HD * 2 : (int)0x80000000;
-      gk[e] = __builtin_amdgcn_raw_buffer_load_b128(kres, off, 0, 0);
-      gv[e] = __builtin_amdgcn_raw_buffer_load_b128(vres, off, 0, 0);
+      const int off = (stager && t0 + 2 * kp + e < nkeys) ? stage_off + (t0 + e) * krow * 2 : (int)0x80000000;
+      gk[e] = __builtin_amdgcn_raw_buffer_load_b128(kres, k_has ? off : (int)0x80000000, 0, 0);
+      gv[e] = __builtin_amdgcn_raw_buffer_load_b128(vres, v_has ? off : (int)0x80000000, 0, 0);
     }
   };
-  stage_load(0);
+  stage_load(t_first);
   u32* vt32 = reinterpret_cast<u32*>(vt);
-  for (int t0 = 0; t0 < nkeys; t0 += 32) {
+  for (int t0 = t_first; t0 < nkeys; t0 += 32) {
     __syncthreads();
     // ---- 32 keys into LDS: K row-major, V transposed ([d][key], two keys per dword)
     if (stager) {
@@ -373,6 +402,7 @@ __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict
     }
     __syncthreads();
     stage_load(t0 + 32);
+    if (WIN && (t0 > pmax || t0 + 31 <= pmin - w.window)) continue;   // nothing here for this wave's queries
     // ---- S^T tile: rows = keys, columns = queries
     f32x16_t sacc;
 #pragma unroll
@@ -386,11 +416,11 @@ __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict
     }
     // element v is key t0 + (v / 4) * 8 + half * 4 + v % 4 for query `col`; only a tile that reaches past the
     // smallest position of the wave's queries has anything to mask
-    if (t0 + 31 > pmin) {
+    if (t0 + 31 > pmin || (WIN && t0 <= pmax - w.window)) {
 #pragma unroll
       for (int v = 0; v < 16; ++v) {
         const int key = t0 + (v / 4) * 8 + half * 4 + (v % 4);
-        sacc[v] = key <= p ? sacc[v] : -INFINITY;
+        sacc[v] = key <= p && (!WIN || key > p - w.window) ? sacc[v] : -INFINITY;
       }
     }
     float tmax = max_med3(sacc[0], sacc[1]);
@@ -453,7 +483,8 @@ __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict
   l += __shfl_xor(l, 32, LR_WAVE);
   if (valid) {
     const float inv = l > 0.0f ? 1.0f / l : 0.0f;
-    u16* yrow = y + ((int64_t)b * S + s) * ldy + head * HD;
+    const int dy = WIN ? w.dv : HD;
+    u16* yrow = y + ((int64_t)b * S + s) * ldy + head * dy;
     // element v of tile d: dimension d * 32 + (v / 4) * 8 + half * 4 + v % 4
 #pragma unroll
     for (int d = 0; d < DT; ++d)
@@ -462,7 +493,7 @@ __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict
         uint2 w2;
         w2.x = pack_bf2(o[d][4 * g4] * inv, o[d][4 * g4 + 1] * inv);
         w2.y = pack_bf2(o[d][4 * g4 + 2] * inv, o[d][4 * g4 + 3] * inv);
-        *reinterpret_cast<uint2*>(yrow + d * 32 + g4 * 8 + half * 4) = w2;
+        if (!WIN || d * 32 + g4 * 8 < dy) *reinterpret_cast<uint2*>(yrow + d * 32 + g4 * 8 + half * 4) = w2;
       }
   }
 }
@@ -519,3 +550,26 @@ extern "C" int lr_attn_prefill(const void* q, int64_t ldq, const void* k_cache, 
     return LR_E_UNSUPPORTED;
   return lr_launch_status();
 }
+
+// lr_window_attention on the matrix cores (bf16; head sizes up to 128 and multiples of 8, all strides multiples of 8).
+namespace lr_detail {
+int window_attention_mfma(const lr_window_attention_t* d, lr_stream_t stream) {
+  const int hd = d->dk > d->dv ? d->dk : d->dv;
+  if (d->dtype != LR_BF16 || hd > 128 || d->dk % 8 || d->dv % 8 || d->ldq % 8 || d->ldk % 8 || d->ldy % 8 ||
+      lr_misaligned(d->q) || lr_misaligned(d->k) || lr_misaligned(d->v) || lr_misaligned(d->y) || !(d->scale > 0.0f))
+    return LR_E_UNSUPPORTED;
+  if ((int64_t)(d->n_keys + 64) * d->ldk * 2 >= 0x7fffffff || (int64_t)((d->S + 127) / 128) * d->H * d->B >= (1 << 24))
+    return LR_E_UNSUPPORTED;
+  const WindowKeys w = {d->window, d->n_keys, (int)d->ldk, d->dk, d->dv, d->scale};
+  const dim3 grid((unsigned)((int64_t)((d->S + 127) / 128) * d->H * d->B));
+  hipStream_t s = (hipStream_t)stream;
+#define LR_WIN(HD)                                                                                                     \
+  k_attn_prefill_mfma<HD, 1, true><<<grid, dim3(256), 0, s>>>((const u16*)d->q, d->ldq, (const u16*)d->k,             \
+                                                              (const u16*)d->v, d->pos, (u16*)d->y, d->ldy, d->S, d->H, \
+                                                              d->H, d->Smax, w)
+  if (hd <= 64) LR_WIN(64);
+  else LR_WIN(128);
+#undef LR_WIN
+  return lr_launch_status();
+}
+}  // namespace lr_detail

@@ -8,6 +8,10 @@
 // latents, and the result goes through W_uv (lr_latent_attention).  Scores, softmax and sums are fp32.
 #include "mixer_common.h"
 
+namespace lr_detail {
+int window_attention_mfma(const lr_window_attention_t* d, lr_stream_t stream);   // attention.hip
+}
+
 namespace {
 
 // one wave per row: the latent's norm, into the cache at the row's position
@@ -35,20 +39,13 @@ __global__ __launch_bounds__(256) void k_latent_update(const T* __restrict__ c, 
   for (int r = lane; r < ldc; r += 64) stf(dst + r, r < rank ? ldf(src + r) * inv * ldf(gain + r) : 0.0f);
 }
 
-// First position of the n rows lr_latent_window hands out: the portion's window, or the whole cache where it is shorter.
-__device__ __forceinline__ int window_base(int pos0, int window, int n, int Smax) {
-  if (n >= Smax) return 0;
-  const int b = pos0 - window + 1;
-  return b > 0 ? b : 0;
-}
-
 __global__ __launch_bounds__(256) void k_latent_window(const uint4* __restrict__ cache, const int32_t* __restrict__ pos,
                                                        uint4* __restrict__ out, int n, int window, int q16, int Smax) {
   const int b = blockIdx.y;
   const int i = blockIdx.x * 256 + threadIdx.x;   // 16-byte piece of this sequence's n rows
   if (i >= n * q16) return;
   const int row = i / q16;
-  const int p = window_base(pos[0], window, n, Smax) + row;
+  const int p = lr_window_base(pos[0], window, n, Smax) + row;
   out[(int64_t)b * n * q16 + i] = p >= 0 && p < Smax ? cache[((int64_t)b * Smax + p) * q16 + (i - row * q16)]
                                                      : make_uint4(0, 0, 0, 0);
 }
@@ -74,7 +71,7 @@ __global__ __launch_bounds__(64) void k_window_attention(const WinAttn a) {
   const int h = blockIdx.x, s = blockIdx.y, b = blockIdx.z, lane = threadIdx.x;
   const int64_t row = (int64_t)b * a.S + s;
   const int p = a.pos[s];
-  const int base = a.windowed_rows ? window_base(a.pos[0], a.window, a.n_keys, a.Smax) : 0;
+  const int base = a.windowed_rows ? lr_window_base(a.pos[0], a.window, a.n_keys, a.Smax) : 0;
   const TQ* q = reinterpret_cast<const TQ*>(a.q) + row * a.ldq + h * a.hq;
   for (int d = lane; d < a.dk; d += 64) qs[d] = ldf(q + d);
   __syncthreads();
@@ -231,7 +228,12 @@ extern "C" int lr_window_attention(const lr_window_attention_t* d, lr_stream_t s
   if (d->ldq < (int64_t)d->H * d->dk || d->ldy < (int64_t)d->H * d->dv || d->ldk < (int64_t)d->H * d->dk ||
       d->ldk < (int64_t)d->H * d->dv)
     return LR_E_SHAPE;
-  if (d->B > 65535 || d->S > 65535) return LR_E_UNSUPPORTED;
+  if (d->B > 65535) return LR_E_UNSUPPORTED;
+  {
+    const int rc = lr_detail::window_attention_mfma(d, stream);
+    if (rc != LR_E_UNSUPPORTED) return rc;
+  }
+  if (d->S > 65535) return LR_E_UNSUPPORTED;
   if (d->dv > 1024 || d->dk > 8192) return LR_E_UNSUPPORTED;
   WinAttn a = {};
   a.q = d->q; a.ldq = d->ldq; a.hq = d->dk;

@@ -10,7 +10,7 @@
 // b_t the running sum of log-decays inside the chunk,
 //     Q_t = q_t e^{b_t},  K_s = k_s e^{-b_s},  A = tril(Q K^T)
 //     O   = Q S + A V,    S <- diag(e^{b_last}) (S + K^T V).
-// A wave owns 16 value columns of S in its accumulators: registers i of a 16-row tile are rows 4 (lane / 16) + i, which
+// A wave owns 32 value columns of S in its accumulators: registers i of a 16-row tile are rows 4 (lane / 16) + i, which
 // is exactly the operand a k-step over those four channels wants, so S is multiplied where it lies.  Where a chunk's
 // decay is so steep that e^{-b} would leave the safe range, the chunk is walked in runs of 4 or 1 tokens instead.
 // Few (sequence, head) pairs: the tokens are cut into segments that run side by side -- first the state each segment
@@ -23,14 +23,14 @@
 namespace {
 
 constexpr int CH = 16;              // tokens per chunk
-constexpr float STEEP = -24.0f;     // a run of tokens whose log-decay sums below this is cut into shorter runs
+constexpr float STEEP = -34.0f;     // a run of tokens whose log2-decay sums below this is cut into shorter runs
 constexpr int AS = 20;              // row stride of the score partials in LDS
 
 struct LinAttn {
   const void *q, *k, *v, *g;
   int64_t ld;
-  const float* log_decay;   // [B * S, H * dk], or NULL
-  const float* head_decay;  // [H] log-decays, used when log_decay is NULL
+  const float* log_decay;   // [B * S, H * dk] base-2 logarithms, or NULL
+  const float* head_decay;  // [H] natural logarithms, used when log_decay is NULL
   const float* rope;        // [rope_len, rot / 2, 2], or NULL
   const int32_t* pos;
   float* state;             // [B, H, dk, dv]
@@ -55,9 +55,39 @@ __device__ __forceinline__ float rotated(float own, float partner, float c, floa
 }
 
 // ---------------------------------------------------------------------------------------------- prefill
+// Eight consecutive channels as stored.
+template <typename T> struct Oct;
+template <> struct Oct<u16> {
+  uint4 r;
+  __device__ __forceinline__ void load(rsrc_t p, int off) {
+    const u32x4_t t = __builtin_amdgcn_raw_buffer_load_b128(p, off, 0, 0);
+    r = make_uint4(t.x, t.y, t.z, t.w);
+  }
+  __device__ __forceinline__ void get(float* f) const { unpack8(r, f); }
+};
+template <> struct Oct<float> {
+  u32x4_t a, b;
+  __device__ __forceinline__ void load(rsrc_t p, int off) {
+    a = __builtin_amdgcn_raw_buffer_load_b128(p, off, 0, 0);
+    b = __builtin_amdgcn_raw_buffer_load_b128(p, off + 16, 0, 0);
+  }
+  __device__ __forceinline__ void get(float* f) const {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) { f[j] = __uint_as_float(a[j]); f[4 + j] = __uint_as_float(b[j]); }
+  }
+};
+
+__device__ __forceinline__ void lds_st8(float* p, const float* f) {
+  *reinterpret_cast<float4*>(p) = make_float4(f[0], f[1], f[2], f[3]);
+  *reinterpret_cast<float4*>(p + 4) = make_float4(f[4], f[5], f[6], f[7]);
+}
+
+constexpr int MAX_NW = 8;   // waves per workgroup, 32 value columns each
+
 // state_only: no outputs, the segment starts from zero and leaves its state and its total log-decay in scratch.
-template <typename T, int DKT>
-__global__ __launch_bounds__(1024) void k_linear_attention(const LinAttn a, const int state_only) {
+// VEC: dk is a multiple of 8, rotation pairs lie a multiple of 8 apart and rows are 16-byte aligned.
+template <typename T, int DKT, bool VEC>
+__global__ __launch_bounds__(64 * MAX_NW) void k_linear_attention(const LinAttn a, const int state_only) {
   constexpr int DKP = 16 * DKT, QS = DKP + 4;
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const int NW = blockDim.x >> 6;
@@ -73,283 +103,345 @@ __global__ __launch_bounds__(1024) void k_linear_attention(const LinAttn a, cons
   const int bh = blockIdx.x, seg = blockIdx.y;
   const int b = bh / a.H, h = bh - b * a.H;
   const int dk = a.dk, dv = a.dv;
-  const int s0 = seg * a.seg_len, s1 = min(a.S, s0 + a.seg_len);
+  const int s0 = seg * a.seg_len, len = min(a.S - s0, a.seg_len);
   const int pos0 = a.pos[0];
   if (pos0 < 0 || (a.rope && pos0 + a.S > a.rope_len)) {
     if (a.err && tid == 0) *a.err = LR_DEV_POS_RANGE;
     return;
   }
-  const T* q = reinterpret_cast<const T*>(a.q) + (int64_t)b * a.S * a.ld + h * dk;
-  const T* k = reinterpret_cast<const T*>(a.k) + (int64_t)b * a.S * a.ld + h * dk;
-  const T* v = reinterpret_cast<const T*>(a.v) + (int64_t)b * a.S * a.ld + h * dv;
-  const T* g = reinterpret_cast<const T*>(a.g) + (int64_t)b * a.S * a.ld + h * dv;
-  const float* ld_ = a.log_decay ? a.log_decay + (int64_t)b * a.S * a.H * dk + h * dk : nullptr;
-  const float hd_ = a.log_decay ? 0.0f : fmaxf(a.head_decay[h], LOG_DECAY_FLOOR);
-  const int col = wave * 16 + l16;      // this lane's value column
-  const bool live = wave * 16 < dv, colv = col < dv;
-  const bool vec = (dk & 3) == 0;
+  // (uniform pointers to the current chunk's first row, per-lane offsets that stay the same from chunk to chunk)
+  const int64_t row0 = (int64_t)b * a.S + s0;
+  const T* q = reinterpret_cast<const T*>(a.q) + row0 * a.ld + h * dk;
+  const T* k = reinterpret_cast<const T*>(a.k) + row0 * a.ld + h * dk;
+  const T* v = reinterpret_cast<const T*>(a.v) + row0 * a.ld + h * dv;
+  const T* g = reinterpret_cast<const T*>(a.g) + row0 * a.ld + h * dv;
+  T* y = reinterpret_cast<T*>(a.y) + row0 * a.ldy + h * dv;
+  const int lstr = a.H * dk;
+  const float* lg = a.log_decay ? a.log_decay + row0 * lstr + h * dk : nullptr;
+  const float lh = a.log_decay ? 0.0f : fmaxf(a.head_decay[h] * LOG2E, LOG_DECAY_FLOOR);
   const int half = a.rot >> 1;
-  const bool vrot = vec && (half & 3) == 0;
-  const float gain = (a.norm && colv) ? ldf(reinterpret_cast<const T*>(a.norm) + col) : 1.0f;
+  const float* tab = a.rope ? a.rope + (int64_t)(pos0 + s0) * half * 2 : nullptr;
+  const int c0w = wave * 32;            // the wave's value columns: c0w + l16 and c0w + 16 + l16
+  const bool live = c0w < dv;
+  const bool cv[2] = {c0w + l16 < dv, c0w + 16 + l16 < dv};
+  float gain[2] = {1.0f, 1.0f};
+  if (a.norm) {
+#pragma unroll
+    for (int n = 0; n < 2; ++n)
+      if (cv[n]) gain[n] = ldf(reinterpret_cast<const T*>(a.norm) + c0w + 16 * n + l16);
+  }
 
-  // ---- the state: tile m, register i is row 16 m + 4 g4 + i of this lane's column
-  f32x4_t S[DKT];
+  const int col[2] = {cv[0] ? c0w + l16 : 0, cv[1] ? c0w + 16 + l16 : 0};   // (loads never branch: they go to a valid
+                                                                            // place and the value is dropped)
+  // ---- the state: tile (m, n), register i is row 16 m + 4 g4 + i of column c0w + 16 n + l16
+  f32x4_t S[DKT][2];
   {
-    const float* src = nullptr;
-    if (!state_only) {
-      if (a.nseg > 1) src = a.seg_state + ((int64_t)bh * a.nseg + seg) * dk * dv;
-      else if (pos0 > 0) src = a.state + (int64_t)bh * dk * dv;
-    }
+    const bool have = !state_only && (a.nseg > 1 || pos0 > 0);
+    const float* src = a.nseg > 1 ? a.seg_state + ((int64_t)bh * a.nseg + seg) * dk * dv : a.state + (int64_t)bh * dk * dv;
 #pragma unroll
     for (int m = 0; m < DKT; ++m)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int c = 16 * m + 4 * g4 + i;
-        S[m][i] = (src && colv && c < dk) ? src[(int64_t)c * dv + col] : 0.0f;
-      }
+      for (int n = 0; n < 2; ++n) S[m][n] = f32x4_t{0, 0, 0, 0};
+    if (have) {
+#pragma unroll
+      for (int m = 0; m < DKT; ++m)
+#pragma unroll
+        for (int n = 0; n < 2; ++n)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int c = 16 * m + 4 * g4 + i;
+            const float t = src[(c < dk ? c : 0) * dv + col[n]];
+            S[m][n][i] = (cv[n] && c < dk) ? t : 0.0f;
+          }
+    }
   }
 
-  // ---- what one chunk needs from memory, fetched one chunk ahead
-  const int it = tid / (DKP / 4), ic = (tid % (DKP / 4)) * 4;   // item: token it, channels ic .. ic + 3
-  const bool item = tid < CH * (DKP / 4);
-  Quad<T> rq, rk, pq, pk;
-  float la[CH], vr[4], gr[4], cs[8];
-  rq.zero(); rk.zero(); pq.zero(); pk.zero();
-  auto fetch = [&](int c0) {
-    if (tid < dk) {
+  // ---- what one chunk needs from memory, fetched while the chunk before is worked on
+  constexpr int SZ = (int)sizeof(T);
+  const int ldb = (int)a.ld * SZ;       // bytes from token to token
+  const int it = tid / (DKP / 8), ic = (tid % (DKP / 8)) * 8;   // item: token it, channels ic .. ic + 7
+  const bool item = tid < CH * (DKP / 8) && ic < dk;
+  const bool turns = a.rope && ic < a.rot;
+  const int pc = ic < half ? ic + half : ic - half, fi = ic < half ? ic : ic - half;
+  const int o_item = item ? it * ldb + ic * SZ : NOWHERE;
+  const int o_pair = item && turns ? it * ldb + pc * SZ : NOWHERE;
+  const int o_cs = item && turns ? (it * half + fi) * 8 : NOWHERE;
+  const int o_la = tid < dk ? tid * 4 : NOWHERE;
+  const int o_col[2] = {cv[0] ? 4 * g4 * ldb + (c0w + l16) * SZ : NOWHERE,
+                        cv[1] ? 4 * g4 * ldb + (c0w + 16 + l16) * SZ : NOWHERE};
+  const int ldyb = (int)a.ldy * SZ;
+  const int o_y[2] = {cv[0] ? 4 * g4 * ldyb + (c0w + l16) * SZ : NOWHERE,
+                      cv[1] ? 4 * g4 * ldyb + (c0w + 16 + l16) * SZ : NOWHERE};
+  Oct<T> rq, rk, pq, pk;
+  float la[CH], cs[16];
+  T vr[2][4], gr[2][4];
+  // a chunk of nt tokens starting at row c0 of the segment: its rows of q / k / v / g as a buffer that ends with them
+  auto rows_of = [&](const T* base, int c0, int cols) {
+    const int nt = min(len - c0, CH);
+    return buffer_of(base + (int64_t)c0 * a.ld, (nt - 1) * ldb + cols * SZ);
+  };
+  auto fetch = [&](int c0) {            // c0: chunk start, from the segment's start
+    const int nt = min(len - c0, CH);
+    if (lg) {
+      const rsrc_t r = buffer_of(lg + (int64_t)c0 * lstr, ((nt - 1) * lstr + dk) * 4);
+      int off = fresh(o_la);
 #pragma unroll
-      for (int t = 0; t < CH; ++t) {
-        const int s = c0 + t;
-        la[t] = s < s1 ? (ld_ ? fmaxf(ld_[(int64_t)s * a.H * dk + tid], LOG_DECAY_FLOOR) : hd_) : 0.0f;
+      for (int t = 0; t < CH; ++t, off += lstr * 4) la[t] = buf_ld(r, off, 0.0f);
+    }
+    if constexpr (VEC) {
+      const rsrc_t rk_ = rows_of(k, c0, dk), rq_ = rows_of(q, c0, dk);
+      rk.load(rk_, o_item);
+      if (!state_only) rq.load(rq_, o_item);
+      if (a.rope) {
+        pk.load(rk_, o_pair);
+        if (!state_only) pq.load(rq_, o_pair);
+        const rsrc_t rt = buffer_of(tab + (int64_t)c0 * half * 2, nt * half * 8);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const u32x4_t t4 = __builtin_amdgcn_raw_buffer_load_b128(rt, o_cs + 16 * j, 0, 0);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) cs[4 * j + e] = __uint_as_float(t4[e]);
+        }
       }
     }
-    rq.zero(); rk.zero(); pq.zero(); pk.zero();
-    const int s = c0 + it;
-    if (item && s < s1 && ic < dk) {
-      const T* qr = q + (int64_t)s * a.ld;
-      const T* kr = k + (int64_t)s * a.ld;
-      if (vec) {
-        rk.load(kr + ic);
-        if (!state_only) rq.load(qr + ic);
-      } else {
+    const rsrc_t rv = rows_of(v, c0, dv);
+    int off[2] = {fresh(o_col[0]), fresh(o_col[1])};
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-          if (ic + j < dk) { rk.put(j, kr + ic + j); rq.put(j, qr + ic + j); }
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int n = 0; n < 2; ++n) vr[n][i] = buf_ld(rv, off[n] + i * ldb, T());
+  };
+  // (the gate values are needed at the end of the chunk only)
+  auto fetch_gate = [&](int c0) {
+    const rsrc_t rg = rows_of(g, c0, dv);
+    int off[2] = {fresh(o_col[0]), fresh(o_col[1])};
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int n = 0; n < 2; ++n) gr[n][i] = buf_ld(rg, off[n] + i * ldb, T());
+  };
+  // this thread's eight channels of q and k, rotated and scaled
+  auto item_values = [&](int c0, float* fq, float* fk) {
+    if constexpr (VEC) {
+      rq.get(fq);
+      rk.get(fk);
+      if (turns) {
+        float xq[8], xk[8];
+        pk.get(xk);
+        if (!state_only) pq.get(xq);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          const float sn = ic < half ? -cs[2 * j + 1] : cs[2 * j + 1];
+          fk[j] = fk[j] * cs[2 * j] + xk[j] * sn;
+          if (!state_only) fq[j] = fq[j] * cs[2 * j] + xq[j] * sn;
+        }
       }
-      if (a.rope && ic < a.rot) {
-        const float* tr = a.rope + (int64_t)(pos0 + s) * half * 2;
-        if (vrot) {
-          const int pc = ic < half ? ic + half : ic - half, fi = ic < half ? ic : ic - half;
-          pk.load(kr + pc);
-          if (!state_only) pq.load(qr + pc);
+    } else {
 #pragma unroll
-          for (int j = 0; j < 8; ++j) cs[j] = tr[2 * fi + j];
-        } else {
+      for (int j = 0; j < 8; ++j) fq[j] = fk[j] = 0.0f;
+      if (item && it < len - c0) {
+        const T* kr = k + (int64_t)(c0 + it) * a.ld;
+        const T* qr = q + (int64_t)(c0 + it) * a.ld;
 #pragma unroll
-          for (int j = 0; j < 4; ++j) {
-            const int c = ic + j;
-            if (c < a.rot && c < dk) {
-              const int pc = c < half ? c + half : c - half, fi = c < half ? c : c - half;
-              pk.put(j, kr + pc);
-              pq.put(j, qr + pc);
-              cs[2 * j] = tr[2 * fi];
-              cs[2 * j + 1] = tr[2 * fi + 1];
+        for (int j = 0; j < 8; ++j) {
+          const int c = ic + j;
+          if (c < dk) {
+            fq[j] = ldf(qr + c);
+            fk[j] = ldf(kr + c);
+            if (a.rope && c < a.rot) {
+              const int p = c < half ? c + half : c - half, f = c < half ? c : c - half;
+              const float* tr = tab + ((int64_t)(c0 + it) * half + f) * 2;
+              fq[j] = rotated(fq[j], ldf(qr + p), tr[0], tr[1], c < half);
+              fk[j] = rotated(fk[j], ldf(kr + p), tr[0], tr[1], c < half);
             }
           }
         }
       }
     }
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int sr = c0 + 4 * g4 + i;
-      const bool ok = colv && sr < s1;
-      vr[i] = ok ? ldf(v + (int64_t)sr * a.ld + col) : 0.0f;
-    }
-  };
-  // (the gate values are needed at the end of the chunk only)
-  auto fetch_gate = [&](int c0) {
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int sr = c0 + 4 * g4 + i;
-      gr[i] = (colv && sr < s1) ? ldf(g + (int64_t)sr * a.ld + col) : 0.0f;
-    }
+    for (int j = 0; j < 8; ++j) { fq[j] *= a.q_scale; fk[j] *= a.k_scale; }
   };
 
   // ---- the finished chunk's outputs: norm over the head, gain, gate (its row sums lie in ssq)
-  f32x4_t o;
+  f32x4_t o[2];
+  const float inv_dv = 1.0f / (float)dv;
   auto emit = [&](int c0) {
-    if (!colv) return;
+    if (!live) return;
     float ss[4] = {0, 0, 0, 0};
-    for (int w = 0; w * 16 < dv; ++w) {
+#pragma clang loop unroll(disable)
+    for (int w = 0; w * 32 < dv; ++w) {
       const float4 p = *reinterpret_cast<const float4*>(&ssq[w * CH + 4 * g4]);
       ss[0] += p.x; ss[1] += p.y; ss[2] += p.z; ss[3] += p.w;
     }
-    T* yr = reinterpret_cast<T*>(a.y) + (int64_t)b * a.S * a.ldy + h * dv + col;
+    const rsrc_t ry = buffer_of(y + (int64_t)c0 * a.ldy, (min(len - c0, CH) - 1) * ldyb + dv * SZ);
+    int off[2] = {fresh(o_y[0]), fresh(o_y[1])};
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int sr = c0 + 4 * g4 + i;
-      if (sr < s1) stf(yr + (int64_t)sr * a.ldy, o[i] * (1.0f / sqrtf(ss[i] / (float)dv + a.eps)) * gain * silu_f(gr[i]));
+      const float inv = rsq_f(ss[i] * inv_dv + a.eps);
+#pragma unroll
+      for (int n = 0; n < 2; ++n)
+        buf_st(ry, off[n] + i * ldyb, o[n][i] * inv * gain[n] * silu_f(ldf(&gr[n][i])), T());
     }
   };
 
-  float total = 0.0f;   // log-decay of the whole segment, for channel tid
+  float total = 0.0f;   // log2-decay of the whole segment, for channel tid
   if (tid < 4) steep[tid] = 0;
-  fetch(s0);
+  fetch(0);
   __syncthreads();
   int par = 0;
-  for (int c0 = s0; c0 < s1; c0 += CH, par ^= 1) {
+  for (int c0 = 0; c0 < len; c0 += CH, par ^= 1) {
     // ---- running log-decay of every channel
     if (tid < dk) {
       float acc = 0.0f, run4 = 0.0f;
-      bool s16 = false, s4 = false;
+      bool s4 = false;
 #pragma unroll
       for (int t = 0; t < CH; ++t) {
+        if (!lg) la[t] = t < len - c0 ? lh : 0.0f;
+        la[t] = fmaxf(la[t], LOG_DECAY_FLOOR);
         acc += la[t];
         run4 = (t & 3) ? run4 + la[t] : la[t];
         s4 = s4 || run4 < STEEP;
         Bs[t * DKP + tid] = acc;
       }
-      s16 = acc < STEEP;
       total += acc;
-      if (s16) steep[2 * par] = 1;
+      if (acc < STEEP) steep[2 * par] = 1;
       if (s4) steep[2 * par + 1] = 1;
-    } else if (tid < DKP) {
-#pragma unroll
-      for (int t = 0; t < CH; ++t) Bs[t * DKP + tid] = 0.0f;
     }
     if (tid < 2) steep[2 * (par ^ 1) + tid] = 0;
+    float fq[8], fk[8];
+    item_values(c0, fq, fk);
     __syncthreads();
-    if (!state_only && c0 > s0) emit(c0 - CH);
-    if (!state_only) fetch_gate(c0);
-    const int run = steep[2 * par + 1] ? 1 : (steep[2 * par] ? 4 : CH);   // uniform over the workgroup
+    if (!state_only) {
+      if (c0 > 0) emit(c0 - CH);
+      fetch_gate(c0);
+    }
+    const int run = __builtin_amdgcn_readfirstlane(steep[2 * par + 1] ? 1 : (steep[2 * par] ? 4 : CH));
     if (run < CH) {
       __syncthreads();
       if (tid < dk) {   // sums that start again with every run
         float acc = 0.0f;
 #pragma unroll
         for (int t = 0; t < CH; ++t) {
-          acc = (t % run) ? acc + la[t] : la[t];
+          acc = (t & (run - 1)) ? acc + la[t] : la[t];
           Bs[t * DKP + tid] = acc;
         }
       }
       __syncthreads();
     }
-    // ---- this thread's item, rotated and scaled
-    float fq[4], fk[4];
-    rq.get(fq);
-    rk.get(fk);
-    if (a.rope && item && ic < a.rot) {
-      float fpq[4], fpk[4];
-      pq.get(fpq);
-      pk.get(fpk);
+    float vv[2][4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (ic + j < a.rot) {
-          fq[j] = rotated(fq[j], fpq[j], cs[2 * j], cs[2 * j + 1], ic + j < half);
-          fk[j] = rotated(fk[j], fpk[j], cs[2 * j], cs[2 * j + 1], ic + j < half);
-        }
+    for (int n = 0; n < 2; ++n) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) vv[n][i] = ldf(&vr[n][i]);
+      o[n] = f32x4_t{0, 0, 0, 0};
     }
-#pragma unroll
-    for (int j = 0; j < 4; ++j) { fq[j] *= a.q_scale; fk[j] *= a.k_scale; }
-    float vv[4] = {vr[0], vr[1], vr[2], vr[3]};
-    o = f32x4_t{0, 0, 0, 0};
 
     for (int lo = 0; lo < CH; lo += run) {
       if (lo > 0) __syncthreads();
-      if (item) {
-        const float4 bb = *reinterpret_cast<const float4*>(&Bs[it * DKP + ic]);
-        const float e[4] = {expf(bb.x), expf(bb.y), expf(bb.z), expf(bb.w)};
+      if (tid < CH * (DKP / 8)) {
+        float e[8], wq[8], wk[8];
         const bool in = it >= lo && it < lo + run;
-        float4 wq, wk;
-        wq.x = in ? fq[0] * e[0] : 0.0f; wk.x = in ? fk[0] / e[0] : 0.0f;
-        wq.y = in ? fq[1] * e[1] : 0.0f; wk.y = in ? fk[1] / e[1] : 0.0f;
-        wq.z = in ? fq[2] * e[2] : 0.0f; wk.z = in ? fk[2] / e[2] : 0.0f;
-        wq.w = in ? fq[3] * e[3] : 0.0f; wk.w = in ? fk[3] / e[3] : 0.0f;
-        *reinterpret_cast<float4*>(&Qs[it * QS + ic]) = wq;
-        *reinterpret_cast<float4*>(&Ks[it * QS + ic]) = wk;
-        if (it == lo + run - 1) *reinterpret_cast<float4*>(&eC[ic]) = make_float4(e[0], e[1], e[2], e[3]);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          const float bb = ic + j < dk ? Bs[it * DKP + ic + j] : 0.0f;
+          e[j] = exp2_f(bb);
+          wq[j] = in ? fq[j] * e[j] : 0.0f;
+          wk[j] = in ? fk[j] * exp2_f(-bb) : 0.0f;
+        }
+        lds_st8(&Qs[it * QS + ic], wq);
+        lds_st8(&Ks[it * QS + ic], wk);
+        if (it == lo + run - 1) lds_st8(&eC[ic], e);
       }
       __syncthreads();
-      if (lo + run >= CH && c0 + CH < s1) fetch(c0 + CH);   // everything of this chunk is in registers or LDS
+      if (lo + run >= CH && c0 + CH < len) fetch(c0 + CH);   // everything of this chunk is in registers or LDS
       if (!state_only) {
         // scores, the channels shared out among the waves; then Q S while the partial scores settle
-        f32x4_t pa = {0, 0, 0, 0};
-        for (int m = wave; m < DKT; m += NW) {
-          const float4 x = *reinterpret_cast<const float4*>(&Qs[l16 * QS + 16 * m + 4 * g4]);
-          const float4 y = *reinterpret_cast<const float4*>(&Ks[l16 * QS + 16 * m + 4 * g4]);
-          pa = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, pa, 0, 0, 0);
-          pa = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, pa, 0, 0, 0);
-          pa = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, y.z, pa, 0, 0, 0);
-          pa = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, pa, 0, 0, 0);
-        }
         if (wave < DKT) {
+          f32x4_t pa = {0, 0, 0, 0};
+#pragma clang loop unroll(disable)
+          for (int m = wave; m < DKT; m += NW) {
+            const float4 x = *reinterpret_cast<const float4*>(&Qs[l16 * QS + 16 * m + 4 * g4]);
+            const float4 z = *reinterpret_cast<const float4*>(&Ks[l16 * QS + 16 * m + 4 * g4]);
+            pa = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, z.x, pa, 0, 0, 0);
+            pa = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, z.y, pa, 0, 0, 0);
+            pa = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, z.z, pa, 0, 0, 0);
+            pa = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, z.w, pa, 0, 0, 0);
+          }
 #pragma unroll
           for (int i = 0; i < 4; ++i) Ap[(wave * CH + 4 * g4 + i) * AS + l16] = pa[i];
         }
         if (live) {
-          f32x4_t o2 = {0, 0, 0, 0};
 #pragma unroll
           for (int m = 0; m < DKT; ++m) {
             const float4 x = *reinterpret_cast<const float4*>(&Qs[l16 * QS + 16 * m + 4 * g4]);
-            o = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, S[m][0], o, 0, 0, 0);
-            o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, S[m][1], o2, 0, 0, 0);
-            o = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, S[m][2], o, 0, 0, 0);
-            o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, S[m][3], o2, 0, 0, 0);
+            const float xe[4] = {x.x, x.y, x.z, x.w};
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+              o[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(xe[i], S[m][0][i], o[0], 0, 0, 0);
+              o[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(xe[i], S[m][1][i], o[1], 0, 0, 0);
+            }
           }
-          o += o2;
         }
         __syncthreads();
       }
       if (live) {
         if (!state_only) {
-          float4 as = make_float4(0, 0, 0, 0);
+          float as[4] = {0, 0, 0, 0};
           const int np = NW < DKT ? NW : DKT;
+#pragma clang loop unroll(disable)
           for (int w = 0; w < np; ++w) {
             const float4 p = *reinterpret_cast<const float4*>(&Ap[(w * CH + l16) * AS + 4 * g4]);
-            as.x += p.x; as.y += p.y; as.z += p.z; as.w += p.w;
+            as[0] += p.x; as[1] += p.y; as[2] += p.z; as[3] += p.w;
           }
-          const int sc = 4 * g4;   // key token of the first of the four values; the query token is l16
-          o = __builtin_amdgcn_mfma_f32_16x16x4f32(sc <= l16 ? as.x : 0.0f, vv[0], o, 0, 0, 0);
-          o = __builtin_amdgcn_mfma_f32_16x16x4f32(sc + 1 <= l16 ? as.y : 0.0f, vv[1], o, 0, 0, 0);
-          o = __builtin_amdgcn_mfma_f32_16x16x4f32(sc + 2 <= l16 ? as.z : 0.0f, vv[2], o, 0, 0, 0);
-          o = __builtin_amdgcn_mfma_f32_16x16x4f32(sc + 3 <= l16 ? as.w : 0.0f, vv[3], o, 0, 0, 0);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {   // key token 4 g4 + i, query token l16
+            const float w = 4 * g4 + i <= l16 ? as[i] : 0.0f;
+            o[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(w, vv[0][i], o[0], 0, 0, 0);
+            o[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(w, vv[1][i], o[1], 0, 0, 0);
+          }
         }
 #pragma unroll
         for (int m = 0; m < DKT; ++m) {
           const float4 e = *reinterpret_cast<const float4*>(&eC[16 * m + 4 * g4]);
-          f32x4_t s = S[m];
+          f32x4_t x0 = S[m][0], x1 = S[m][1];
 #pragma unroll
-          for (int i = 0; i < 4; ++i)
-            s = __builtin_amdgcn_mfma_f32_16x16x4f32(Ks[(4 * g4 + i) * QS + 16 * m + l16], vv[i], s, 0, 0, 0);
-          s[0] *= e.x; s[1] *= e.y; s[2] *= e.z; s[3] *= e.w;
-          S[m] = s;
+          for (int i = 0; i < 4; ++i) {
+            const float kx = Ks[(4 * g4 + i) * QS + 16 * m + l16];
+            x0 = __builtin_amdgcn_mfma_f32_16x16x4f32(kx, vv[0][i], x0, 0, 0, 0);
+            x1 = __builtin_amdgcn_mfma_f32_16x16x4f32(kx, vv[1][i], x1, 0, 0, 0);
+          }
+          const f32x4_t ev = {e.x, e.y, e.z, e.w};
+          S[m][0] = x0 * ev;
+          S[m][1] = x1 * ev;
         }
       }
     }
     if (!state_only && live) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const float s = row16_sum(colv ? o[i] * o[i] : 0.0f);
+        const float s = row16_sum(o[0][i] * o[0][i] + o[1][i] * o[1][i])   /* (columns beyond dv are zero) */;
         if (l16 == 0) ssq[wave * CH + 4 * g4 + i] = s;
       }
     }
   }
   if (!state_only) {
     __syncthreads();
-    emit(s0 + ((s1 - s0 - 1) / CH) * CH);
+    emit(((len - 1) / CH) * CH);
   }
   // ---- the state the segment leaves
   float* dst = nullptr;
   if (state_only) dst = a.seg_state + ((int64_t)bh * a.nseg + seg + 1) * dk * dv;
   else if (seg == a.nseg - 1) dst = a.state + (int64_t)bh * dk * dv;
-  if (dst && colv) {
+  if (dst) {
 #pragma unroll
     for (int m = 0; m < DKT; ++m)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int c = 16 * m + 4 * g4 + i;
-        if (c < dk) dst[(int64_t)c * dv + col] = S[m][i];
-      }
+      for (int n = 0; n < 2; ++n)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int c = 16 * m + 4 * g4 + i;
+          if (cv[n] && c < dk) dst[c * dv + c0w + 16 * n + l16] = S[m][n][i];
+        }
   }
   if (state_only && tid < dk) a.seg_decay[((int64_t)bh * a.nseg + seg) * dk + tid] = total;
 }
@@ -366,12 +458,12 @@ __global__ __launch_bounds__(256) void k_linear_attention_scan(const LinAttn a) 
   float acc = a.pos[0] > 0 ? a.state[(int64_t)bh * n + e] : 0.0f;
   slot[0] = acc;
   for (int j = 1; j < a.nseg; ++j) {
-    acc = acc * expf(dec[(int64_t)(j - 1) * a.dk]) + slot[(int64_t)j * n];
+    acc = acc * exp2_f(dec[(int64_t)(j - 1) * a.dk]) + slot[(int64_t)j * n];
     slot[(int64_t)j * n] = acc;
   }
 }
 
-// log-decays of a gated linear attention: out[row, c] = log sigmoid(a2[c, :] . lowrank[row, :] + bias[c]) / tau
+// log2-decays of a gated linear attention: out[row, c] = log2 sigmoid(a2[c, :] . lowrank[row, :] + bias[c]) / tau
 template <typename T>
 __global__ __launch_bounds__(256) void k_gla_log_decay(const T* __restrict__ lowrank, int64_t ld, const T* __restrict__ a2,
                                                        const T* __restrict__ bias, float* __restrict__ out, int rows,
@@ -397,7 +489,7 @@ __global__ __launch_bounds__(256) void k_gla_log_decay(const T* __restrict__ low
     }
 #pragma unroll
     for (int r = 0; r < R; ++r)
-      if (r < nr) out[(int64_t)(r0 + r) * n + c] = log_sigmoid_f(z[r]) * inv_tau;
+      if (r < nr) out[(int64_t)(r0 + r) * n + c] = log_sigmoid_f(z[r]) * (inv_tau * LOG2E);
   }
 }
 
@@ -455,13 +547,13 @@ __global__ __launch_bounds__(1024) void k_linear_attention_step(const LinAttn a)
       const T* w = reinterpret_cast<const T*>(a.a2) + (int64_t)(h * dk + c) * a.rank;
       float z = ldf(reinterpret_cast<const T*>(a.a_bias) + h * dk + c);
       for (int j = 0; j < a.rank; ++j) z = fmaf(ldf(w + j), ldf(t + j), z);
-      la = log_sigmoid_f(z) * a.inv_tau;
+      la = log_sigmoid_f(z) * a.inv_tau * LOG2E;
     } else {
-      la = a.head_decay[h];
+      la = a.head_decay[h] * LOG2E;
     }
     qs[c] = fq * a.q_scale;
     ks[c] = fk * a.k_scale;
-    es[c] = expf(la);
+    es[c] = exp2_f(la);
   }
   __syncthreads();
   float acc[V];
@@ -505,7 +597,7 @@ __global__ __launch_bounds__(1024) void k_linear_attention_step(const LinAttn a)
   __syncthreads();
   float tot = 0.0f;
   for (int w = 0; w < (nt >> 6); ++w) tot += wsum[w];
-  const float inv = 1.0f / sqrtf(tot / (float)dv + a.eps);
+  const float inv = rsq_f(tot / (float)dv + a.eps);
   (void)mine;
   for (int d = tid; d < dv; d += nt) {
     const float gain = a.norm ? ldf(reinterpret_cast<const T*>(a.norm) + d) : 1.0f;
@@ -527,6 +619,7 @@ int fill(const lr_linear_attention_t* d, LinAttn& a) {
   if (d->ld < (int64_t)d->H * d->dk || d->ld < (int64_t)d->H * d->dv || d->ldy < (int64_t)d->H * d->dv) return LR_E_SHAPE;
   if ((int64_t)d->B * d->H > 0x7fffffff || (int64_t)d->B * d->S > 0x7fffffff) return LR_E_SHAPE;
   if (d->ld % 8) return LR_E_ALIGN;
+  if (d->ld > (1 << 24) || d->ldy > (1 << 24) || (int64_t)d->H * d->dk > (1 << 24)) return LR_E_UNSUPPORTED;  // 32-bit offsets in a chunk
   if (d->dk > MAX_DIM || d->dv > MAX_DIM) return LR_E_UNSUPPORTED;
   const bool gated = d->lowrank != nullptr;
   if (gated && (d->a2 == nullptr || d->a_bias == nullptr)) return LR_E_NULL;
@@ -546,10 +639,10 @@ int fill(const lr_linear_attention_t* d, LinAttn& a) {
   return LR_OK;
 }
 
-// Segments: enough workgroups to fill the chip, none shorter than 64 tokens.
-int segments(int B, int S, int H) {
+// Segments: about as many workgroups as the chip holds at once, none shorter than 64 tokens.
+int segments(int B, int S, int H, int dv) {
   const int64_t wgs = (int64_t)B * H;
-  int64_t want = (512 + wgs - 1) / wgs;
+  int64_t want = ((dv <= 128 ? 512 : 256) + wgs - 1) / wgs;
   const int64_t most = S / 64;
   if (want > most) want = most;
   return want < 1 ? 1 : (int)want;
@@ -557,16 +650,23 @@ int segments(int B, int S, int H) {
 
 size_t align16(size_t n) { return (n + 15) & ~(size_t)15; }
 
-template <typename T, int DKT>
+template <typename T, int DKT, bool VEC>
 int launch(const LinAttn& a, int state_only, hipStream_t s) {
   constexpr int DKP = 16 * DKT;
-  int nw = (a.dv + 15) / 16;
-  if (nw < DKT) nw = DKT;             // one item of the chunk's preparation per thread
+  int nw = (a.dv + 31) / 32;
+  if (nw < 4) nw = 4;
+  if (64 * nw < CH * (DKP / 8)) nw = CH * (DKP / 8) / 64;   // one item of the chunk's preparation per thread
   const size_t lds = sizeof(float) * ((size_t)2 * CH * (DKP + 4) + CH * DKP + DKP + (size_t)nw * CH * AS + nw * CH + 4);
   static std::atomic<unsigned long long> raised{0};
-  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_linear_attention<T, DKT>), lds, raised)) return LR_E_LAUNCH;
-  k_linear_attention<T, DKT><<<dim3(a.B * a.H, state_only ? a.nseg - 1 : a.nseg), dim3(64 * nw), lds, s>>>(a, state_only);
+  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_linear_attention<T, DKT, VEC>), lds, raised)) return LR_E_LAUNCH;
+  k_linear_attention<T, DKT, VEC><<<dim3(a.B * a.H, state_only ? a.nseg - 1 : a.nseg), dim3(64 * nw), lds, s>>>(a, state_only);
   return lr_launch_status();
+}
+
+template <typename T, int DKT>
+int launch(const LinAttn& a, int state_only, hipStream_t s) {
+  const bool vec = a.dk % 8 == 0 && a.rot % 16 == 0 && !lr_misaligned(a.q) && !lr_misaligned(a.k) && !lr_misaligned(a.rope);
+  return vec ? launch<T, DKT, true>(a, state_only, s) : launch<T, DKT, false>(a, state_only, s);
 }
 
 template <typename T>
@@ -588,7 +688,7 @@ int prefill(LinAttn& a, const lr_linear_attention_t* d, hipStream_t s) {
         (const T*)a.lowrank, a.ld, (const T*)a.a2, (const T*)a.a_bias, const_cast<float*>(a.log_decay), rows, n, a.rank,
         a.inv_tau);
   }
-  a.nseg = segments(a.B, a.S, a.H);
+  a.nseg = segments(a.B, a.S, a.H, a.dv);
   if (a.nseg > 1) {
     a.seg_len = ((a.S + a.nseg - 1) / a.nseg + CH - 1) / CH * CH;
     a.nseg = (a.S + a.seg_len - 1) / a.seg_len;
@@ -626,7 +726,7 @@ int step(const LinAttn& a, hipStream_t s) {
 extern "C" size_t lr_linear_attention_scratch_bytes(int B, int S, int H, int dk, int dv, int gated) {
   if (B <= 0 || S <= 0 || H <= 0 || dk <= 0 || dv <= 0 || S == 1) return 0;
   size_t n = gated ? align16((size_t)B * S * H * dk * sizeof(float)) : 0;
-  const int ns = segments(B, S, H);
+  const int ns = segments(B, S, H, dv);
   if (ns > 1) n += align16((size_t)B * H * ns * dk * dv * sizeof(float)) + align16((size_t)B * H * ns * dk * sizeof(float));
   return n;
 }

@@ -111,6 +111,13 @@ __device__ __forceinline__ float wave_max(float v) {
   return fmaxf(fmaxf(lr_lane(v, 0), lr_lane(v, 16)), fmaxf(lr_lane(v, 32), lr_lane(v, 48)));
 }
 
+// First position of the n rows lr_latent_window hands out: the portion's window, or the whole cache where it is shorter.
+__device__ __forceinline__ int lr_window_base(int pos0, int window, int n, int Smax) {
+  if (n >= Smax) return 0;
+  const int b = pos0 - window + 1;
+  return b > 0 ? b : 0;
+}
+
 // silu in fp32 the way the eager reference evaluates it: x / (1 + exp(-x)), rounded to bf16, then
 // multiplied by u and rounded again.
 __device__ __forceinline__ float swiglu_bf(float u, float g) {
