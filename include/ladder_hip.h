@@ -489,21 +489,26 @@ int lr_window_attention(const lr_window_attention_t* desc, lr_stream_t stream);
 
 /* The same attention straight on the latent cache, for single tokens and short portions: with k = W_uk c and v = W_uv c
  * per head, scores are ((W_uk^T q) . c) * scale and the output W_uv (sum of weights times c).  uk [H*dk, ldr], uv
- * [H*dv, ldr], cache [Bmax, Smax, ldr] (columns beyond the rank zero in all three); the portion's own latents must be in
- * the cache.  ldr <= 1024. */
+ * [H*dv, ldr], cache [Bmax, Smax, ldr] (columns beyond the rank zero in all three).  latent != NULL: the portion's own
+ * latents [B*S, rank] (row stride ldl) are normed with gain `norm` and cached first, as lr_latent_update does; NULL: the
+ * cache holds them already.  ldr <= 1024. */
 typedef struct lr_latent_attention {
   const void* q;
   int64_t ldq;
-  const void *uk, *uv, *cache;
+  const void *uk, *uv;
+  void* cache;
   void* y;
   int64_t ldy;
   const int32_t* pos;
+  const void *latent, *norm;
+  int64_t ldl;
+  int32_t* err; /* may be NULL */
   void* scratch;
   size_t scratch_bytes;
-  int32_t B, S, H, dk, dv, ldr, window, Smax, dtype;
-  float scale;
+  int32_t B, S, H, dk, dv, ldr, rank, window, Smax, dtype;
+  float scale, eps;
 } lr_latent_attention_t;
-size_t lr_latent_attention_scratch_bytes(int B, int S, int H, int ldr, int Smax);
+size_t lr_latent_attention_scratch_bytes(int B, int S, int H, int ldr, int window, int Smax);
 int lr_latent_attention(const lr_latent_attention_t* desc, lr_stream_t stream);
 
 #ifdef __cplusplus

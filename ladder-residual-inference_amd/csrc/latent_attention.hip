@@ -5,7 +5,8 @@
 // caller's linear expands them) and attend there: on the matrix cores (attention.hip) where the head sizes allow it, one
 // wave per query otherwise.
 // Single tokens and the shortest portions never form k and v: q is taken through W_uk once, scores and sums run on the
-// latents, and the result goes through W_uv (lr_latent_attention).  Scores, softmax and sums are fp32.
+// latents -- on the matrix cores, the keys cut into ranges that run side by side --, and the merged result goes through
+// W_uv (lr_latent_attention: three launches, the cache write included).  Scores, softmax and sums are fp32.
 #include "mixer_common.h"
 
 namespace lr_detail {
@@ -14,13 +15,12 @@ int window_attention_mfma(const lr_window_attention_t* d, lr_stream_t stream);  
 
 namespace {
 
-// one wave per row: the latent's norm, into the cache at the row's position
+// a wave: the latent of one row, normed, into the cache at the row's position
 template <typename T>
-__global__ __launch_bounds__(256) void k_latent_update(const T* __restrict__ c, int64_t ld, const T* __restrict__ gain,
-                                                       const int32_t* __restrict__ pos, T* __restrict__ cache, int rows,
-                                                       int S, int rank, int ldc, int Smax, float eps, int32_t* err) {
-  const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (row >= rows) return;
+__device__ __forceinline__ void latent_row(const T* __restrict__ c, int64_t ld, const T* __restrict__ gain,
+                                           const int32_t* __restrict__ pos, T* __restrict__ cache, int row, int S, int rank,
+                                           int ldc, int Smax, float eps, int32_t* err) {
+  const int lane = threadIdx.x & 63;
   const int b = row / S, s = row - b * S;
   const int p = pos[s];
   if (p < 0 || p >= Smax) {
@@ -34,9 +34,24 @@ __global__ __launch_bounds__(256) void k_latent_update(const T* __restrict__ c, 
     ss += f * f;
   }
   ss = wave_sum(ss);
-  const float inv = 1.0f / sqrtf(ss / (float)rank + eps);
+  const float inv = rsq_f(ss / (float)rank + eps);
   T* dst = cache + ((int64_t)b * Smax + p) * ldc;
   for (int r = lane; r < ldc; r += 64) stf(dst + r, r < rank ? ldf(src + r) * inv * ldf(gain + r) : 0.0f);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void k_latent_update(const T* __restrict__ c, int64_t ld, const T* __restrict__ gain,
+                                                       const int32_t* __restrict__ pos, T* __restrict__ cache, int rows,
+                                                       int S, int rank, int ldc, int Smax, float eps, int32_t* err) {
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (row < rows) latent_row(c, ld, gain, pos, cache, row, S, rank, ldc, Smax, eps, err);
+}
+
+// eight consecutive values; the pointer is 16-byte aligned
+__device__ __forceinline__ void ld8(const u16* p, float* f) { unpack8(ld16(p), f); }
+__device__ __forceinline__ void ld8(const float* p, float* f) {
+  const float4 x = *reinterpret_cast<const float4*>(p), y = *reinterpret_cast<const float4*>(p + 4);
+  f[0] = x.x; f[1] = x.y; f[2] = x.z; f[3] = x.w; f[4] = y.x; f[5] = y.y; f[6] = y.z; f[7] = y.w;
 }
 
 __global__ __launch_bounds__(256) void k_latent_window(const uint4* __restrict__ cache, const int32_t* __restrict__ pos,
@@ -117,39 +132,358 @@ __global__ __launch_bounds__(64) void k_window_attention(const WinAttn a) {
     if (lane + 64 * i < a.dv) stf(y + lane + 64 * i, acc[i] * inv);
 }
 
-// q' [rows, H, ldr] fp32: q' = W_uk^T q per head
-template <typename T>
-__global__ __launch_bounds__(256) void k_latent_absorb(const T* __restrict__ q, int64_t ldq, const T* __restrict__ uk,
-                                                       float* __restrict__ out, int H, int dk, int ldr) {
-  extern __shared__ float qs[];
-  const int h = blockIdx.x;
-  const int64_t row = blockIdx.y;
-  for (int d = threadIdx.x; d < dk; d += 256) qs[d] = ldf(q + row * ldq + h * dk + d);
+// ---- q through W_uk.  Workgroup h < H: q'[row, h, :] = W_uk[h]^T q[row, h, :] in fp32 for RB rows and up to 128 latent
+// columns, eight per thread, the head's dk rows of W_uk shared out among the thread groups.  Workgroup H: the new
+// latents, normed, into the cache (a wave per row).  The result goes out in fp32, or multiplied by `mul` and in bf16 (as k
+// does where it is expanded).
+struct Absorb {
+  const void *q, *uk;
+  int64_t ldq;
+  float* out;
+  u16* out_bf;
+  float mul;
+  int H, dk, ldr, rows, S;
+  const void *c, *gain;      // latents to be cached, NULL: they already are
+  int64_t ldc;
+  const int32_t* pos;
+  void* cache;
+  int rank, Smax;
+  float eps;
+  int32_t* err;
+};
+
+template <typename T, int RB>
+__global__ __launch_bounds__(512) void k_latent_absorb(const Absorb a) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  const int h = blockIdx.x, tid = threadIdx.x, row0 = blockIdx.y * RB, col0 = blockIdx.z * 128;
+  if (h == a.H) {
+    if (blockIdx.z == 0)
+      for (int r = tid >> 6; r < RB && row0 + r < a.rows; r += 8)
+        latent_row(reinterpret_cast<const T*>(a.c), a.ldc, reinterpret_cast<const T*>(a.gain), a.pos,
+                   reinterpret_cast<T*>(a.cache), row0 + r, a.S, a.rank, a.ldr, a.Smax, a.eps, a.err);
+    return;
+  }
+  const int cols = min(128, a.ldr - col0);
+  float* qs = sm;                         // [RB][dk]
+  float* part = sm + RB * a.dk;           // [groups][RB][cols]
+  for (int i = tid; i < RB * a.dk; i += 512) {
+    const int r = i / a.dk, d = i - r * a.dk;
+    qs[i] = row0 + r < a.rows ? ldf(reinterpret_cast<const T*>(a.q) + (int64_t)(row0 + r) * a.ldq + h * a.dk + d) : 0.0f;
+  }
   __syncthreads();
-  for (int r = threadIdx.x; r < ldr; r += 256) {
-    float acc = 0.0f;
-    const T* w = uk + (int64_t)h * dk * ldr + r;
+  const int n8 = cols / 8, groups = 512 / n8, g = tid / n8, c8 = (tid - g * n8) * 8;
+  if (g < groups) {
+    float acc[RB][8];
+#pragma unroll
+    for (int r = 0; r < RB; ++r)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) acc[r][j] = 0.0f;
+    const T* w = reinterpret_cast<const T*>(a.uk) + (int64_t)h * a.dk * a.ldr + col0 + c8;
+#pragma unroll 4
+    for (int d = g; d < a.dk; d += groups) {
+      float f[8];
+      ld8(w + (int64_t)d * a.ldr, f);
+#pragma unroll
+      for (int r = 0; r < RB; ++r) {
+        const float qd = qs[r * a.dk + d];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) acc[r][j] = fmaf(qd, f[j], acc[r][j]);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < RB; ++r)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) part[(g * RB + r) * cols + c8 + j] = acc[r][j];
+  }
+  __syncthreads();
+  const int used = min(groups, a.dk);
+  for (int i = tid; i < RB * cols; i += 512) {
+    const int r = i / cols;
+    float t = 0.0f;
 #pragma unroll 8
-    for (int d = 0; d < dk; ++d) acc = fmaf(qs[d], ldf(w + (int64_t)d * ldr), acc);
-    out[(row * H + h) * ldr + r] = acc;
+    for (int gg = 0; gg < used; ++gg) t += part[gg * RB * cols + i];
+    const int64_t at = ((int64_t)(row0 + r) * a.H + h) * a.ldr + col0 + (i - r * cols);
+    if (row0 + r < a.rows) {
+      if (a.out) a.out[at] = t;
+      else a.out_bf[at] = f_to_bf(t * a.mul);
+    }
   }
 }
 
-// y[row, h dv + e] = W_uv[h dv + e, :] . o[row, h, :]
-template <typename T>
-__global__ __launch_bounds__(256) void k_latent_up(const float* __restrict__ o, const T* __restrict__ uv, T* __restrict__ y,
-                                                   int64_t ldy, int H, int dv, int ldr) {
-  extern __shared__ float os[];
-  const int h = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int64_t row = blockIdx.y;
-  for (int r = threadIdx.x; r < ldr; r += 256) os[r] = o[(row * H + h) * ldr + r];
+// ---- scores and sums on the latents, on the matrix cores.  One workgroup: one query row, 32 heads, a range of its
+// keys, 64 at a time.  The tile of latents lies in LDS twice: by key (operand of the scores) and by column (operand of
+// the weighted sums).  The fp32 softmax weights enter the bf16 products as hi + lo, which keeps them to about 2^-17.  The eight waves: (key quarter, head half) for the scores, an eighth of the latent columns for the sums.
+struct Partial {
+  const u16* q;              // q' [rows, H, ldr], in base-2 exponents
+  const u16* cache;
+  const int32_t* pos;
+  float *o, *ml;             // [rows, H, nsplit, ldr], [rows, H, nsplit, 2]
+  int S, H, ldr, window, Smax, nsplit;
+};
+
+constexpr int KT = 64;       // keys per tile
+
+template <int R>
+__global__ __launch_bounds__(512) void k_latent_partial(const Partial a) {
+  constexpr int KS = R / 32, CROW = R + 8, VROW = KT + 8, RT = R >= 128 ? R / 128 : 1, ITEMS = R >= 128 ? R / 128 : 1;
+  constexpr int SL = R >= 128 ? 16 : R / 8, PB = 64 / SL;   // a wave stages SL column slices of PB key pairs at once
+  extern __shared__ __attribute__((aligned(16))) u16 su[];
+  u16* Cs = su;                           // [KT][CROW]
+  u16* Vt = Cs + KT * CROW;               // [R][VROW], groups of 8 keys permuted (see vgroup)
+  u16* Ph = Vt + R * VROW;                // [32 heads][VROW] weights, hi and lo
+  u16* Pl = Ph + 32 * VROW;
+  float* mx = reinterpret_cast<float*>(Pl + 32 * VROW);   // [4][32] tile maxima of the key quarters
+  float* corr = mx + 128;                 // [32]
+  float* ls = corr + 32;                  // [4][32]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g4 = lane >> 4, l16 = lane & 15;
+  const int sp = blockIdx.x, hb = blockIdx.y * 32, row = blockIdx.z;
+  const int b = row / a.S, s = row - b * a.S;
+  const int p = min(a.pos[s], a.Smax - 1);
+  const int lo = max(0, p - a.window + 1), n = p - lo + 1;
+  const int per = ((n + a.nsplit - 1) / a.nsplit + KT - 1) / KT * KT;
+  const int k0 = lo + sp * per, k1 = min(p + 1, k0 + per);
+  const int nh = min(32, a.H - hb);
+  float* mlp = a.ml + (((int64_t)row * a.H + hb) * a.nsplit + sp) * 2;
+  if (k0 >= k1) {
+    if (tid < nh) {
+      mlp[(int64_t)tid * a.nsplit * 2] = -INFINITY;
+      mlp[(int64_t)tid * a.nsplit * 2 + 1] = 0.0f;
+    }
+    return;
+  }
+  const int kq = wave & 3, hg = wave >> 2;
+  // Staging: an item is eight columns of two neighbouring keys, stored by column as dwords of two keys.  Column slices
+  // that a wave writes together would meet in two LDS banks (their rows lie 8 * 36 dwords apart): the groups of eight
+  // keys of a row are permuted by its slice, which spreads them over all banks and leaves a group whole for the reader.
+  const rsrc_t res = buffer_of(a.cache + (int64_t)b * a.Smax * a.ldr, a.Smax * a.ldr * 2);
+  u32x4_t st[ITEMS][2];
+  auto slot = [&](int i, int& kp, int& c) {
+    const int blk = i * 8 + wave;                   // PB key pairs x SL slices
+    constexpr int NP = (KT / 2) / PB;
+    kp = (blk % NP) * PB + lane / SL;
+    c = ((blk / NP) * SL + lane % SL) * 8;
+  };
+  auto stage_load = [&](int t0) {
+#pragma unroll
+    for (int i = 0; i < ITEMS; ++i) {
+      int kp, c;
+      slot(i, kp, c);
+#pragma unroll
+      for (int e = 0; e < 2; ++e) {
+        const int key = t0 + 2 * kp + e;
+        st[i][e] = __builtin_amdgcn_raw_buffer_load_b128(res, (c < a.ldr && key < k1) ? (key * a.ldr + c) * 2 : NOWHERE, 0, 0);
+      }
+    }
+  };
+  auto vgroup = [](int group, int r) { return group ^ ((r >> 4) & 7); };
+  stage_load(k0);
+  // ---- q' of the wave's 16 heads
+  u32x4_t qh[KS];
+  {
+    const int head = hb + hg * 16 + l16;
+    const int64_t at = ((int64_t)row * a.H + head) * a.ldr;
+#pragma unroll
+    for (int j = 0; j < KS; ++j) {
+      const int c = 32 * j + 8 * g4;
+      qh[j] = u32x4_t{0, 0, 0, 0};
+      if (head < a.H && c < a.ldr) qh[j] = *reinterpret_cast<const u32x4_t*>(a.q + at + c);
+    }
+  }
+  f32x4_t o[2][RT];
+#pragma unroll
+  for (int g = 0; g < 2; ++g)
+#pragma unroll
+    for (int t = 0; t < RT; ++t) o[g][t] = f32x4_t{0, 0, 0, 0};
+  float m[4] = {-INFINITY, -INFINITY, -INFINITY, -INFINITY}, l[4] = {0, 0, 0, 0};
+  u32* vt32 = reinterpret_cast<u32*>(Vt);
+  const int cw = wave * 16 * RT;          // this wave's first column in the sums
+  for (int t0 = k0; t0 < k1; t0 += KT) {
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < ITEMS; ++i) {
+      int kp, c;
+      slot(i, kp, c);
+      if (c < R) {
+#pragma unroll
+        for (int e = 0; e < 2; ++e) *reinterpret_cast<u32x4_t*>(&Cs[(2 * kp + e) * CROW + c]) = st[i][e];
+        const int at = vgroup(kp >> 2, c) * 4 + (kp & 3);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          vt32[(c + 2 * j) * (VROW / 2) + at] = (st[i][0][j] & 0xffffu) | (st[i][1][j] << 16);
+          vt32[(c + 2 * j + 1) * (VROW / 2) + at] = (st[i][0][j] >> 16) | (st[i][1][j] & 0xffff0000u);
+        }
+      }
+    }
+    __syncthreads();
+    if (t0 + KT < k1) stage_load(t0 + KT);
+    // ---- scores: rows are heads, columns keys
+    f32x4_t sa = {0, 0, 0, 0}, sb = {0, 0, 0, 0};
+#pragma unroll
+    for (int j = 0; j < KS; ++j) {
+      const u32x4_t kc = *reinterpret_cast<const u32x4_t*>(&Cs[(kq * 16 + l16) * CROW + 32 * j + 8 * g4]);
+      f32x4_t& acc = j & 1 ? sb : sa;
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, qh[j]), __builtin_bit_cast(bf16x8_t, kc), acc, 0, 0, 0);
+    }
+    sa += sb;
+    const bool seen = t0 + kq * 16 + l16 < k1;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      sa[i] = seen ? sa[i] : -INFINITY;
+      const float t = row16_max(sa[i]);
+      if (l16 == 0) mx[kq * 32 + hg * 16 + 4 * g4 + i] = t;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int hh = hg * 16 + 4 * g4 + i;
+      const float mt = fmaxf(fmaxf(mx[hh], mx[32 + hh]), fmaxf(mx[64 + hh], mx[96 + hh]));
+      const float mn = fmaxf(m[i], mt);   // finite: the tile's first key is seen
+      const float cr = exp2_f(m[i] - mn), w = exp2_f(sa[i] - mn);
+      m[i] = mn;
+      l[i] = l[i] * cr + w;
+      Ph[hh * VROW + kq * 16 + l16] = f_to_bf(w);
+      Pl[hh * VROW + kq * 16 + l16] = f_to_bf(w - round_bf(w));
+      if (kq == 0 && l16 == 0) corr[hh] = cr;
+    }
+    __syncthreads();
+    // ---- sums: this wave's columns, keys 32 at a time
+    if (cw < R) {
+      bf16x8_t ph[2][2], pl[2][2];
+#pragma unroll
+      for (int g = 0; g < 2; ++g)
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {
+          ph[g][k] = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4_t*>(&Ph[(16 * g + l16) * VROW + 32 * k + 8 * g4]));
+          pl[g][k] = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4_t*>(&Pl[(16 * g + l16) * VROW + 32 * k + 8 * g4]));
+        }
+      f32x4_t cv[2];
+#pragma unroll
+      for (int g = 0; g < 2; ++g) {
+        const float4 c = *reinterpret_cast<const float4*>(&corr[16 * g + 4 * g4]);
+        cv[g] = f32x4_t{c.x, c.y, c.z, c.w};
+      }
+#pragma unroll
+      for (int t = 0; t < RT; ++t) {
+        const int r = cw + 16 * t + l16;
+        o[0][t] *= cv[0];
+        o[1][t] *= cv[1];
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {
+          const bf16x8_t vt = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4_t*>(&Vt[r * VROW + 8 * vgroup(4 * k + g4, r)]));
+          o[0][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph[0][k], vt, o[0][t], 0, 0, 0);
+          o[1][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph[1][k], vt, o[1][t], 0, 0, 0);
+          o[0][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl[0][k], vt, o[0][t], 0, 0, 0);
+          o[1][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl[1][k], vt, o[1][t], 0, 0, 0);
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const float t = row16_sum(l[i]);
+    const int hh = hg * 16 + 4 * g4 + i;
+    if (l16 == 0) {
+      ls[kq * 32 + hh] = t;
+      if (kq == 0) mx[hh] = m[i];   // (nobody reads the last tile's maxima any more: a barrier lies between)
+    }
+  }
   __syncthreads();
-  for (int e = wave; e < dv; e += 4) {
-    const T* w = uv + ((int64_t)h * dv + e) * ldr;
-    float acc = 0.0f;
-    for (int r = lane; r < ldr; r += 64) acc = fmaf(ldf(w + r), os[r], acc);
-    acc = wave_sum(acc);
-    if (lane == 0) stf(y + row * ldy + h * dv + e, acc);
+  if (tid < nh) {
+    mlp[(int64_t)tid * a.nsplit * 2] = mx[tid];
+    mlp[(int64_t)tid * a.nsplit * 2 + 1] = (ls[tid] + ls[32 + tid]) + (ls[64 + tid] + ls[96 + tid]);
+  }
+  if (cw >= R) return;
+#pragma unroll
+  for (int g = 0; g < 2; ++g)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int hh = g * 16 + 4 * g4 + i;
+      if (hh < nh) {
+        float* op = a.o + (((int64_t)row * a.H + hb + hh) * a.nsplit + sp) * a.ldr;
+#pragma unroll
+        for (int t = 0; t < RT; ++t) {
+          const int c = cw + 16 * t + l16;
+          if (c < a.ldr) op[c] = o[g][t][i];
+        }
+      }
+    }
+}
+
+// ---- the ranges' results merged, then through W_uv: y[row, h dv + e] = W_uv[h dv + e, :] . o[row, h, :].  One workgroup
+// per head, RB rows and `per` value dimensions; a wave multiplies four rows of W_uv at a time.
+template <typename T, int RB>
+__global__ __launch_bounds__(512) void k_latent_up(const float* __restrict__ o, const float* __restrict__ ml,
+                                                   const T* __restrict__ uv, T* __restrict__ y, int64_t ldy, int H, int dv,
+                                                   int ldr, int nsplit, int rows, int per) {
+  extern __shared__ __attribute__((aligned(16))) float os[];   // [RB][ldr] and [RB][nsplit]
+  float* ws = os + RB * ldr;
+  const int h = blockIdx.x, row0 = blockIdx.y * RB, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  if (ml) {
+    // weight of every range: 2^(m - M) / sum of 2^(m - M) l
+    if (wave < RB) {
+      const int row = min(row0 + wave, rows - 1);
+      const float* p = ml + ((int64_t)row * H + h) * nsplit * 2;
+      float M = -INFINITY;
+      for (int s = lane; s < nsplit; s += 64) M = fmaxf(M, p[2 * s]);
+      M = wave_max(M);
+      float t = 0.0f;
+      for (int s = lane; s < nsplit; s += 64) {
+        const float w = exp2_f(p[2 * s] - M);
+        ws[wave * nsplit + s] = w;
+        t += w * p[2 * s + 1];
+      }
+      t = 1.0f / wave_sum(t);
+      for (int s = lane; s < nsplit; s += 64) ws[wave * nsplit + s] *= t;
+    }
+    __syncthreads();
+  }
+  for (int i = tid; i < RB * ldr; i += 512) {
+    const int r = i / ldr, c = i - r * ldr;
+    const int row = min(row0 + r, rows - 1);
+    float t = 0.0f;
+    if (ml) {
+      const float* p = o + ((int64_t)row * H + h) * nsplit * ldr + c;
+#pragma unroll 8
+      for (int s = 0; s < nsplit; ++s) {
+        const float w = ws[r * nsplit + s];   // 0: nothing was written there
+        const float x = p[(int64_t)s * ldr];
+        t += w > 0.0f ? w * x : 0.0f;
+      }
+    } else {
+      t = o[((int64_t)row * H + h) * ldr + c];
+    }
+    os[i] = t;
+  }
+  __syncthreads();
+  constexpr int E = 4;
+  const int e1 = min(dv, ((int)blockIdx.z + 1) * per);
+  for (int e0 = blockIdx.z * per + wave * E; e0 < e1; e0 += 8 * E) {
+    float acc[E][RB];
+#pragma unroll
+    for (int e = 0; e < E; ++e)
+#pragma unroll
+      for (int r = 0; r < RB; ++r) acc[e][r] = 0.0f;
+    for (int c = lane * 8; c < ldr; c += 512) {
+      float w[E][8];
+#pragma unroll
+      for (int e = 0; e < E; ++e) ld8(uv + ((int64_t)h * dv + min(e0 + e, e1 - 1)) * ldr + c, w[e]);
+#pragma unroll
+      for (int r = 0; r < RB; ++r) {
+        float x[8];
+        ld8(os + r * ldr + c, x);
+#pragma unroll
+        for (int e = 0; e < E; ++e)
+#pragma unroll
+          for (int j = 0; j < 8; ++j) acc[e][r] = fmaf(w[e][j], x[j], acc[e][r]);
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < E; ++e)
+#pragma unroll
+      for (int r = 0; r < RB; ++r) {
+        const float t = wave_sum(acc[e][r]);
+        if (lane == e * RB + r && e0 + e < e1 && row0 + r < rows) stf(y + (int64_t)(row0 + r) * ldy + h * dv + e0 + e, t);
+      }
   }
 }
 
@@ -160,24 +494,72 @@ int launch_window(const WinAttn& a, int B, hipStream_t s) {
   return lr_launch_status();
 }
 
+// Key ranges per query row of the matrix-core kernel: about a workgroup per CU, no range shorter than a tile.
+int splits(int rows, int H, int window, int Smax) {
+  const int keys = window < Smax ? window : Smax;
+  const int64_t wgs = (int64_t)rows * ((H + 31) / 32);
+  int64_t n = (256 + wgs - 1) / wgs;
+  const int most = (keys + KT - 1) / KT;
+  if (n > most) n = most;
+  return n > 64 ? 64 : (int)n;
+}
+
+template <int R>
+int launch_partial(const Partial& a, int rows, hipStream_t s) {
+  const size_t lds = sizeof(u16) * ((size_t)KT * (R + 8) + (R + 2 * 32) * (KT + 8)) + sizeof(float) * 288;
+  static std::atomic<unsigned long long> raised{0};
+  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_latent_partial<R>), lds, raised)) return LR_E_LAUNCH;
+  k_latent_partial<R><<<dim3(a.nsplit, (a.H + 31) / 32, rows), dim3(512), lds, s>>>(a);
+  return lr_launch_status();
+}
+
+template <typename T, int RB>
+int absorb(const Absorb& a, hipStream_t s) {
+  const size_t lds = sizeof(float) * ((size_t)RB * a.dk + (size_t)RB * 512 * 8);
+  static std::atomic<unsigned long long> raised{0};
+  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_latent_absorb<T, RB>), lds, raised)) return LR_E_LAUNCH;
+  k_latent_absorb<T, RB><<<dim3(a.H + (a.c ? 1 : 0), (a.rows + RB - 1) / RB, (a.ldr + 127) / 128), dim3(512), lds, s>>>(a);
+  return lr_launch_status();
+}
+
 template <typename T>
 int latent_attention(const lr_latent_attention_t* d, hipStream_t s) {
   float* qa = reinterpret_cast<float*>(d->scratch);
   const int rows = d->B * d->S;
   float* ol = qa + (size_t)rows * d->H * d->ldr;
-  k_latent_absorb<T><<<dim3(d->H, rows), dim3(256), d->dk * sizeof(float), s>>>((const T*)d->q, d->ldq, (const T*)d->uk, qa,
-                                                                               d->H, d->dk, d->ldr);
-  WinAttn a = {};
-  a.q = qa; a.ldq = (int64_t)d->H * d->ldr; a.hq = d->ldr;
-  a.k = a.v = d->cache;
-  a.kb = a.vb = (int64_t)d->Smax * d->ldr; a.kr = a.vr = d->ldr; a.kh = a.vh = 0;
-  a.y = ol; a.ldy = a.ldq; a.hy = d->ldr; a.pos = d->pos;
-  a.S = d->S; a.H = d->H; a.dk = a.dv = d->ldr; a.window = d->window; a.n_keys = d->Smax; a.Smax = d->Smax;
-  a.scale = d->scale;
-  const int rc = launch_window<float, T, float>(a, d->B, s);
+  // bf16: q' scaled to base-2 exponents, for the matrix-core kernel
+  const bool split = d->dtype == LR_BF16 && d->ldr <= 512 && d->scale > 0.0f && (int64_t)d->Smax * d->ldr * 2 < 0x7fffffff;
+  u16* qb = reinterpret_cast<u16*>(qa);
+  Absorb ab = {d->q, d->uk, d->ldq, split ? nullptr : qa, qb, d->scale * LOG2E, d->H, d->dk, d->ldr, rows, d->S,
+               d->latent, d->norm, d->ldl, d->pos, d->cache, d->rank, d->Smax, d->eps, d->err};
+  int rc = rows >= 8 ? absorb<T, 4>(ab, s) : absorb<T, 1>(ab, s);
   if (rc != LR_OK) return rc;
-  k_latent_up<T><<<dim3(d->H, rows), dim3(256), d->ldr * sizeof(float), s>>>(ol, (const T*)d->uv, (T*)d->y, d->ldy, d->H,
-                                                                            d->dv, d->ldr);
+  float* ml = nullptr;
+  int ns = 1;
+  if (split) {
+    ns = splits(rows, d->H, d->window, d->Smax);
+    ml = ol + (size_t)rows * d->H * ns * d->ldr;
+    const Partial p = {qb, (const u16*)d->cache, d->pos, ol, ml, d->S, d->H, d->ldr, d->window, d->Smax, ns};
+    rc = d->ldr <= 64 ? launch_partial<64>(p, rows, s) : d->ldr <= 128 ? launch_partial<128>(p, rows, s)
+         : d->ldr <= 256 ? launch_partial<256>(p, rows, s) : launch_partial<512>(p, rows, s);
+  } else {
+    WinAttn a = {};
+    a.q = qa; a.ldq = (int64_t)d->H * d->ldr; a.hq = d->ldr;
+    a.k = a.v = d->cache;
+    a.kb = a.vb = (int64_t)d->Smax * d->ldr; a.kr = a.vr = d->ldr; a.kh = a.vh = 0;
+    a.y = ol; a.ldy = a.ldq; a.hy = d->ldr; a.pos = d->pos;
+    a.S = d->S; a.H = d->H; a.dk = a.dv = d->ldr; a.window = d->window; a.n_keys = d->Smax; a.Smax = d->Smax;
+    a.scale = d->scale;
+    rc = launch_window<float, T, float>(a, d->B, s);
+  }
+  if (rc != LR_OK) return rc;
+  const size_t per_row = sizeof(float) * ((size_t)d->ldr + ns);
+  if (rows >= 8)
+    k_latent_up<T, 4><<<dim3(d->H, (rows + 3) / 4, 1), dim3(512), 4 * per_row, s>>>(
+        ol, ml, (const T*)d->uv, (T*)d->y, d->ldy, d->H, d->dv, d->ldr, ns, rows, d->dv);
+  else
+    k_latent_up<T, 1><<<dim3(d->H, rows, (d->dv + 31) / 32), dim3(512), per_row, s>>>(
+        ol, ml, (const T*)d->uv, (T*)d->y, d->ldy, d->H, d->dv, d->ldr, ns, rows, 32);
   return lr_launch_status();
 }
 
@@ -248,9 +630,10 @@ extern "C" int lr_window_attention(const lr_window_attention_t* d, lr_stream_t s
   return LR_E_UNSUPPORTED;
 }
 
-extern "C" size_t lr_latent_attention_scratch_bytes(int B, int S, int H, int ldr, int Smax) {
-  if (B <= 0 || S <= 0 || H <= 0 || ldr <= 0 || Smax <= 0) return 0;
-  return (size_t)2 * B * S * H * ldr * sizeof(float);
+extern "C" size_t lr_latent_attention_scratch_bytes(int B, int S, int H, int ldr, int window, int Smax) {
+  if (B <= 0 || S <= 0 || H <= 0 || ldr <= 0 || window <= 0 || Smax <= 0) return 0;
+  const size_t ns = splits(B * S, H, window, Smax);
+  return (size_t)B * S * H * (ldr + ns * (ldr + 2)) * sizeof(float);
 }
 
 extern "C" int lr_latent_attention(const lr_latent_attention_t* d, lr_stream_t stream) {
@@ -262,9 +645,13 @@ extern "C" int lr_latent_attention(const lr_latent_attention_t* d, lr_stream_t s
   if (d->B <= 0 || d->S <= 0 || d->H <= 0 || d->dk <= 0 || d->dv <= 0 || d->ldr <= 0 || d->window <= 0 || d->Smax <= 0)
     return LR_E_SHAPE;
   if (d->ldq < (int64_t)d->H * d->dk || d->ldy < (int64_t)d->H * d->dv) return LR_E_SHAPE;
-  if (d->scratch_bytes < lr_latent_attention_scratch_bytes(d->B, d->S, d->H, d->ldr, d->Smax)) return LR_E_SHAPE;
+  if (d->scratch_bytes < lr_latent_attention_scratch_bytes(d->B, d->S, d->H, d->ldr, d->window, d->Smax)) return LR_E_SHAPE;
+  if (d->latent) {
+    LR_REQUIRE_PTR(d->norm);
+    if (d->rank <= 0 || d->rank > d->ldr || d->ldl < d->rank) return LR_E_SHAPE;
+  }
   if (d->ldr % 8) return LR_E_ALIGN;
-  if (d->ldr > 1024 || (int64_t)d->B * d->S > 65535) return LR_E_UNSUPPORTED;
+  if (d->ldr > 1024 || (int64_t)d->B * d->S > 65535 || d->dk > 2048) return LR_E_UNSUPPORTED;
   if (d->dtype == LR_BF16) return latent_attention<u16>(d, (hipStream_t)stream);
   if (d->dtype == LR_F32) return latent_attention<float>(d, (hipStream_t)stream);
   return LR_E_UNSUPPORTED;

@@ -61,6 +61,12 @@ __device__ __forceinline__ float row16_sum(float v) {
   v += lr_dpp<0xb1>(v);   // quad_perm [1,0,3,2]
   return v;
 }
+__device__ __forceinline__ float row16_max(float v) {
+  v = fmaxf(v, lr_dpp<0x128>(v));
+  v = fmaxf(v, lr_dpp<0x124>(v));
+  v = fmaxf(v, lr_dpp<0x4e>(v));
+  return fmaxf(v, lr_dpp<0xb1>(v));
+}
 
 // ---- buffer access: a uniform base and size, per-lane 32-bit byte offsets; beyond the size loads give zero and stores
 //      are dropped, so a ragged edge needs no branch

@@ -77,7 +77,7 @@ _PROTOS = {
                                  c_float, c_int, c_void_p, c_void_p]),
     "lr_latent_window": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p]),
     "lr_window_attention": (c_int, [c_void_p, c_void_p]),
-    "lr_latent_attention_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int]),
+    "lr_latent_attention_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
     "lr_latent_attention": (c_int, [c_void_p, c_void_p]),
 }
 
@@ -734,17 +734,19 @@ def window_attention(q, kv, y, pos, B, S, H, dk, dv, window: int, n_keys: int, S
 
 class _LatentAttention(ctypes.Structure):   # lr_latent_attention_t
     _fields_ = [("q", c_void_p), ("ldq", c_int64), ("uk", c_void_p), ("uv", c_void_p), ("cache", c_void_p),
-                ("y", c_void_p), ("ldy", c_int64), ("pos", c_void_p), ("scratch", c_void_p), ("scratch_bytes", c_size_t)] + \
-               [(n, c_int32) for n in ("B", "S", "H", "dk", "dv", "ldr", "window", "Smax", "dtype")] + \
-               [("scale", c_float)]
+                ("y", c_void_p), ("ldy", c_int64), ("pos", c_void_p), ("latent", c_void_p), ("norm", c_void_p),
+                ("ldl", c_int64), ("err", c_void_p), ("scratch", c_void_p), ("scratch_bytes", c_size_t)] + \
+               [(n, c_int32) for n in ("B", "S", "H", "dk", "dv", "ldr", "rank", "window", "Smax", "dtype")] + \
+               [("scale", c_float), ("eps", c_float)]
 
 
-def latent_attention_scratch_bytes(B, S, H, ldr, Smax) -> int:
-    return int(load().lr_latent_attention_scratch_bytes(B, S, H, ldr, Smax))
+def latent_attention_scratch_bytes(B, S, H, ldr, window, Smax) -> int:
+    return int(load().lr_latent_attention_scratch_bytes(B, S, H, ldr, window, Smax))
 
 
-def latent_attention(q, uk, uv, cache, y, pos, scratch, B, S, H, dk, dv, window: int, scale: float):
-    """Sliding-window attention of short portions straight on the latent cache [>= B, Smax, ldr]."""
+def latent_attention(q, uk, uv, cache, y, pos, scratch, B, S, H, dk, dv, window: int, scale: float, new=None):
+    """Sliding-window attention of short portions straight on the latent cache [>= B, Smax, ldr].  new = (latents
+    [B * S, >= rank], gain, rank, eps): they are normed and cached on the way, as latent_update would."""
     rows, qc, ldq = _rows_ld(q)
     _, yc, ldy = _rows_ld(y)
     ldr = cache.shape[2]
@@ -752,10 +754,17 @@ def latent_attention(q, uk, uv, cache, y, pos, scratch, B, S, H, dk, dv, window:
     assert uk.is_contiguous() and uv.is_contiguous() and tuple(uk.shape) == (H * dk, ldr) and tuple(uv.shape) == (H * dv, ldr)
     assert pos.dtype == torch.int32 and pos.numel() == S
     dt = q.dtype
+    latent, gain, ldl, rank, eps = None, None, 0, 0, 0.0
+    if new is not None:
+        c, g, rank, eps = new
+        crows, ccols, ldl = _rows_ld(c)
+        assert crows == rows and ccols >= rank and g.numel() >= rank and c.dtype == dt
+        latent, gain = c.data_ptr(), _dev(g, dt)
     d = _LatentAttention(q=_dev(q, dt), ldq=ldq, uk=_dev(uk, dt), uv=_dev(uv, dt), cache=_dev(cache, dt), y=_dev(y, dt),
-                         ldy=ldy, pos=pos.data_ptr(), scratch=scratch.data_ptr(),
+                         ldy=ldy, pos=pos.data_ptr(), latent=latent, norm=gain, ldl=ldl,
+                         err=device_error_word(q.device).data_ptr(), scratch=scratch.data_ptr(),
                          scratch_bytes=scratch.numel() * scratch.element_size(), B=B, S=S, H=H, dk=dk, dv=dv, ldr=ldr,
-                         window=int(window), Smax=cache.shape[1], dtype=_DTYPES[dt], scale=scale)
+                         rank=rank, window=int(window), Smax=cache.shape[1], dtype=_DTYPES[dt], scale=scale, eps=eps)
     _check(load().lr_latent_attention(ctypes.byref(d), _stream()), "lr_latent_attention")
     return y
 

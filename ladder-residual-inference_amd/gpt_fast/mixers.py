@@ -182,7 +182,8 @@ class LatentAttention(Mixer):
     def scratch_bytes(self, B, S):
         if not self._absorbs(S):
             return 0
-        return _hip.latent_attention_scratch_bytes(B, S, self.args.heads, self.rank_p, self.latents.shape[1])
+        return _hip.latent_attention_scratch_bytes(B, S, self.args.heads, self.rank_p, self.args.window,
+                                                   self.latents.shape[1])
 
     def window_rows(self, B, S):
         a = self.args
@@ -195,13 +196,13 @@ class LatentAttention(Mixer):
         a = self.args
         nq, cache = a.heads * a.dim, self.latents
         proj = self._project_in(ws)
-        _hip.latent_update(proj[:, nq:], self.norm.weight, pos, cache, ws.B, ws.S, a.kv_rank, self.eps)
         y = self._y(ws)
         if self._absorbs(ws.S):
             w = self.kv_up.weight
             _hip.latent_attention(proj[:, :nq], w[:nq], w[nq:], cache, y, pos, ws.scratch, ws.B, ws.S, a.heads, a.dim,
-                                  a.vdim, a.window, a.scale)
+                                  a.vdim, a.window, a.scale, new=(proj[:, nq:], self.norm.weight, a.kv_rank, self.eps))
         else:
+            _hip.latent_update(proj[:, nq:], self.norm.weight, pos, cache, ws.B, ws.S, a.kv_rank, self.eps)
             n = self._n_keys(ws.S)
             rows, kv = ws.window_buffers(ws.B * n, self.rank_p, a.heads * (a.dim + a.vdim))
             if n == cache.shape[1]:      # the window reaches over the whole cache: its rows as they lie
