@@ -28,15 +28,40 @@ __device__ __forceinline__ void latent_row(const T* __restrict__ c, int64_t ld, 
     return;
   }
   const T* src = c + (int64_t)row * ld;
+  T* dst = cache + ((int64_t)b * Smax + p) * ldc;
+  // 1024 columns at a time, all of a lane's loads in flight together
   float ss = 0.0f;
-  for (int r = lane; r < rank; r += 64) {
-    const float f = ldf(src + r);
-    ss += f * f;
+  constexpr int N = 16;
+  T x[N], g[N];
+  auto load = [&](int c0) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const int j = c0 + i * 64 + lane;
+      x[i] = src[j < rank ? j : 0];
+      g[i] = gain[j < rank ? j : 0];
+    }
+  };
+  auto store = [&](int c0, float inv) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const int j = c0 + i * 64 + lane;
+      if (j < ldc) stf(dst + j, j < rank ? ldf(&x[i]) * inv * ldf(&g[i]) : 0.0f);
+    }
+  };
+  for (int c0 = 0; c0 < rank; c0 += 64 * N) {
+    load(c0);
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const float f = c0 + i * 64 + lane < rank ? ldf(&x[i]) : 0.0f;
+      ss = fmaf(f, f, ss);
+    }
   }
   ss = wave_sum(ss);
   const float inv = rsq_f(ss / (float)rank + eps);
-  T* dst = cache + ((int64_t)b * Smax + p) * ldc;
-  for (int r = lane; r < ldc; r += 64) stf(dst + r, r < rank ? ldf(src + r) * inv * ldf(gain + r) : 0.0f);
+  for (int c0 = 0; c0 < ldc; c0 += 64 * N) {
+    if (rank > 64 * N) load(c0);
+    store(c0, inv);
+  }
 }
 
 template <typename T>
@@ -132,10 +157,11 @@ __global__ __launch_bounds__(64) void k_window_attention(const WinAttn a) {
     if (lane + 64 * i < a.dv) stf(y + lane + 64 * i, acc[i] * inv);
 }
 
-// ---- q through W_uk.  Workgroup h < H: q'[row, h, :] = W_uk[h]^T q[row, h, :] in fp32 for RB rows and up to 128 latent
-// columns, eight per thread, the head's dk rows of W_uk shared out among the thread groups.  Workgroup H: the new
-// latents, normed, into the cache (a wave per row).  The result goes out in fp32, or multiplied by `mul` and in bf16 (as k
-// does where it is expanded).
+// ---- q through W_uk: q'[row, h, :] = W_uk[h]^T q[row, h, :], 16 rows and 128 latent columns of a head per workgroup, the
+// head's dk rows of W_uk shared out among its four waves.  fp32 products (v_mfma_f32_16x16x4_f32) on W_uk as it lies: a lane
+// reads eight consecutive columns of one row of W_uk, and column j of everybody's eight is one 16 x 16 product.  Workgroup
+// h = H: the new latents, normed, into the cache (a wave per row).  The result goes out in fp32, or multiplied by `mul`
+// and in bf16 (as k does where it is expanded).
 struct Absorb {
   const void *q, *uk;
   int64_t ldq;
@@ -152,60 +178,76 @@ struct Absorb {
   int32_t* err;
 };
 
-template <typename T, int RB>
-__global__ __launch_bounds__(512) void k_latent_absorb(const Absorb a) {
+constexpr int AW = 4;        // waves of the two projections' workgroups
+
+template <typename T>
+__global__ __launch_bounds__(64 * AW) void k_latent_absorb(const Absorb a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  const int h = blockIdx.x, tid = threadIdx.x, row0 = blockIdx.y * RB, col0 = blockIdx.z * 128;
+  const int h = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g4 = lane >> 4, l16 = lane & 15;
+  const int row0 = blockIdx.y * 16, col0 = blockIdx.z * 128;
   if (h == a.H) {
-    if (blockIdx.z == 0)
-      for (int r = tid >> 6; r < RB && row0 + r < a.rows; r += 8)
-        latent_row(reinterpret_cast<const T*>(a.c), a.ldc, reinterpret_cast<const T*>(a.gain), a.pos,
-                   reinterpret_cast<T*>(a.cache), row0 + r, a.S, a.rank, a.ldr, a.Smax, a.eps, a.err);
+    for (int r = blockIdx.z * AW + wave; r < 16 && row0 + r < a.rows; r += gridDim.z * AW)
+      latent_row(reinterpret_cast<const T*>(a.c), a.ldc, reinterpret_cast<const T*>(a.gain), a.pos,
+                 reinterpret_cast<T*>(a.cache), row0 + r, a.S, a.rank, a.ldr, a.Smax, a.eps, a.err);
     return;
   }
-  const int cols = min(128, a.ldr - col0);
-  float* qs = sm;                         // [RB][dk]
-  float* part = sm + RB * a.dk;           // [groups][RB][cols]
-  for (int i = tid; i < RB * a.dk; i += 512) {
-    const int r = i / a.dk, d = i - r * a.dk;
-    qs[i] = row0 + r < a.rows ? ldf(reinterpret_cast<const T*>(a.q) + (int64_t)(row0 + r) * a.ldq + h * a.dk + d) : 0.0f;
-  }
-  __syncthreads();
-  const int n8 = cols / 8, groups = 512 / n8, g = tid / n8, c8 = (tid - g * n8) * 8;
-  if (g < groups) {
-    float acc[RB][8];
+  const int per = ((a.dk + 4 * AW - 1) / (4 * AW)) * 4;    // rows of W_uk per wave
+  float* part = sm;                                        // [AW - 1][8][4][64]
+  const T* q = reinterpret_cast<const T*>(a.q) + (int64_t)min(row0 + l16, a.rows - 1) * a.ldq + h * a.dk;
+  const int c = min(col0 + 8 * l16, a.ldr - 8);            // (lanes beyond the row read its last columns, for nobody)
+  const T* w = reinterpret_cast<const T*>(a.uk) + (int64_t)h * a.dk * a.ldr + c;
+  f32x4_t acc[8];
 #pragma unroll
-    for (int r = 0; r < RB; ++r)
+  for (int j = 0; j < 8; ++j) acc[j] = f32x4_t{0, 0, 0, 0};
+  constexpr int U = 4;   // steps whose loads are in flight together
+  for (int d0 = 0; d0 < per; d0 += 4 * U) {
+    float f[U][8], x[U];
+    T xr[U];
 #pragma unroll
-      for (int j = 0; j < 8; ++j) acc[r][j] = 0.0f;
-    const T* w = reinterpret_cast<const T*>(a.uk) + (int64_t)h * a.dk * a.ldr + col0 + c8;
-#pragma unroll 4
-    for (int d = g; d < a.dk; d += groups) {
-      float f[8];
-      ld8(w + (int64_t)d * a.ldr, f);
-#pragma unroll
-      for (int r = 0; r < RB; ++r) {
-        const float qd = qs[r * a.dk + d];
-#pragma unroll
-        for (int j = 0; j < 8; ++j) acc[r][j] = fmaf(qd, f[j], acc[r][j]);
-      }
+    for (int u = 0; u < U; ++u) {
+      const int d = min(wave * per + d0 + 4 * u + g4, a.dk - 1);
+      ld8(w + (int64_t)d * a.ldr, f[u]);
+      xr[u] = q[d];
     }
 #pragma unroll
-    for (int r = 0; r < RB; ++r)
+    for (int u = 0; u < U; ++u)
+      x[u] = d0 + 4 * u < per && wave * per + d0 + 4 * u + g4 < a.dk ? ldf(&xr[u]) : 0.0f;
 #pragma unroll
-      for (int j = 0; j < 8; ++j) part[(g * RB + r) * cols + c8 + j] = acc[r][j];
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(f[u][j], x[u], acc[j], 0, 0, 0);
+  }
+  if (wave > 0) {
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) part[(((wave - 1) * 8 + j) * 4 + i) * 64 + lane] = acc[j][i];
   }
   __syncthreads();
-  const int used = min(groups, a.dk);
-  for (int i = tid; i < RB * cols; i += 512) {
-    const int r = i / cols;
-    float t = 0.0f;
-#pragma unroll 8
-    for (int gg = 0; gg < used; ++gg) t += part[gg * RB * cols + i];
-    const int64_t at = ((int64_t)(row0 + r) * a.H + h) * a.ldr + col0 + (i - r * cols);
-    if (row0 + r < a.rows) {
-      if (a.out) a.out[at] = t;
-      else a.out_bf[at] = f_to_bf(t * a.mul);
+  if (wave > 0) return;
+#pragma unroll
+  for (int v = 0; v < AW - 1; ++v)
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[j][i] += part[((v * 8 + j) * 4 + i) * 64 + lane];
+  // register i of product j: column col0 + 8 (4 g4 + i) + j of row row0 + l16
+  if (row0 + l16 >= a.rows) return;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int cc = col0 + 8 * (4 * g4 + i);
+    if (cc >= a.ldr) continue;
+    const int64_t at = ((int64_t)(row0 + l16) * a.H + h) * a.ldr + cc;
+    float f[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) f[j] = acc[j][i];
+    if (a.out) {
+      st4(a.out + at, f);
+      st4(a.out + at + 4, f + 4);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) f[j] *= a.mul;
+      st16(a.out_bf + at, pack8(f));
     }
   }
 }
@@ -409,81 +451,108 @@ __global__ __launch_bounds__(512) void k_latent_partial(const Partial a) {
     }
 }
 
-// ---- the ranges' results merged, then through W_uv: y[row, h dv + e] = W_uv[h dv + e, :] . o[row, h, :].  One workgroup
-// per head, RB rows and `per` value dimensions; a wave multiplies four rows of W_uv at a time.
-template <typename T, int RB>
-__global__ __launch_bounds__(512) void k_latent_up(const float* __restrict__ o, const float* __restrict__ ml,
-                                                   const T* __restrict__ uv, T* __restrict__ y, int64_t ldy, int H, int dv,
-                                                   int ldr, int nsplit, int rows, int per) {
-  extern __shared__ __attribute__((aligned(16))) float os[];   // [RB][ldr] and [RB][nsplit]
-  float* ws = os + RB * ldr;
-  const int h = blockIdx.x, row0 = blockIdx.y * RB, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+// ---- the ranges' results merged, then through W_uv: y[row, h dv + e] = W_uv[h dv + e, :] . o[row, h, :], 16 rows and 64 value
+// dimensions of a head per workgroup, 16 of them per wave; fp32 products.
+template <typename T>
+__global__ __launch_bounds__(64 * AW) void k_latent_up(const float* __restrict__ o, const float* __restrict__ ml,
+                                                       const T* __restrict__ uv, T* __restrict__ y, int64_t ldy, int H,
+                                                       int dv, int ldr, int nsplit, int rows) {
+  extern __shared__ __attribute__((aligned(16))) float os[];   // [16][orow] and [16][nsplit]
+  const int orow = (ldr + 127) / 128 * 128 + 4;
+  float* ws = os + 16 * orow;
+  const int h = blockIdx.x, row0 = blockIdx.y * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int g4 = lane >> 4, l16 = lane & 15;
+  const int nr = min(16, rows - row0);
+  // this wave's rows of W_uv, 32 columns a step: lane (g4, l16) has eight columns of row l16.  The first steps' loads are
+  // out before the merge begins.
+  const int e0 = blockIdx.z * 16 * AW + wave * 16;
+  constexpr int U = 8;
+  const T* w = uv + ((int64_t)h * dv + min(e0 + l16, dv - 1)) * ldr;
+  T wx[U][8];
+  auto load = [&](int c0) {
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      __builtin_memcpy(wx[u], __builtin_assume_aligned(w + min(c0 + 32 * u + 8 * g4, ldr - 8), 16), sizeof(wx[u]));
+  };
+  load(0);
   if (ml) {
     // weight of every range: 2^(m - M) / sum of 2^(m - M) l
-    if (wave < RB) {
-      const int row = min(row0 + wave, rows - 1);
-      const float* p = ml + ((int64_t)row * H + h) * nsplit * 2;
-      float M = -INFINITY;
-      for (int s = lane; s < nsplit; s += 64) M = fmaxf(M, p[2 * s]);
-      M = wave_max(M);
-      float t = 0.0f;
-      for (int s = lane; s < nsplit; s += 64) {
-        const float w = exp2_f(p[2 * s] - M);
-        ws[wave * nsplit + s] = w;
-        t += w * p[2 * s + 1];
-      }
-      t = 1.0f / wave_sum(t);
-      for (int s = lane; s < nsplit; s += 64) ws[wave * nsplit + s] *= t;
+    for (int r = wave; r < nr; r += AW) {
+      const float* p = ml + ((int64_t)(row0 + r) * H + h) * nsplit * 2;
+      const float m = lane < nsplit ? p[2 * lane] : -INFINITY, l = lane < nsplit ? p[2 * lane + 1] : 0.0f;
+      const float w = exp2_f(m - wave_max(m));
+      const float t = wave_sum(w * l);
+      if (lane < nsplit) ws[r * nsplit + lane] = w / t;
     }
     __syncthreads();
   }
-  for (int i = tid; i < RB * ldr; i += 512) {
-    const int r = i / ldr, c = i - r * ldr;
-    const int row = min(row0 + r, rows - 1);
-    float t = 0.0f;
-    if (ml) {
-      const float* p = o + ((int64_t)row * H + h) * nsplit * ldr + c;
-#pragma unroll 8
-      for (int s = 0; s < nsplit; ++s) {
-        const float w = ws[r * nsplit + s];   // 0: nothing was written there
-        const float x = p[(int64_t)s * ldr];
-        t += w > 0.0f ? w * x : 0.0f;
+  // Items of four columns, two per thread and eight ranges at a time in flight.  A row beyond the last repeats the last
+  // one's place with weight 0, as does a range beyond the last.
+  const int q4 = orow / 4 - 1, items = 16 * q4;
+  for (int i0 = tid; i0 < items; i0 += 2 * 64 * AW) {
+    float4 t[2] = {make_float4(0, 0, 0, 0), make_float4(0, 0, 0, 0)};
+    const float* p[2];
+    const float* wr[2];
+    bool on[2];
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const int i = i0 + k * 64 * AW, r = i / q4, c = (i - r * q4) * 4;
+      on[k] = i < items && r < nr && c < ldr;
+      p[k] = o + ((int64_t)(row0 + (on[k] ? r : 0)) * H + h) * nsplit * ldr + (on[k] ? c : 0);
+      wr[k] = ws + (on[k] ? r : 0) * nsplit;
+    }
+    if (!on[0] && !on[1]) {
+      // (rows and columns that are nobody's: zero)
+    } else if (ml) {
+      for (int s0 = 0; s0 < nsplit; s0 += 8) {
+        float4 x[2][8];
+#pragma unroll
+        for (int k = 0; k < 2; ++k)
+#pragma unroll
+          for (int s = 0; s < 8; ++s) x[k][s] = *reinterpret_cast<const float4*>(p[k] + (int64_t)min(s0 + s, nsplit - 1) * ldr);
+#pragma unroll
+        for (int k = 0; k < 2; ++k)
+#pragma unroll
+          for (int s = 0; s < 8; ++s) {
+            const float w = s0 + s < nsplit && on[k] ? wr[k][s0 + s] : 0.0f;   // 0: nothing was written there
+            t[k].x += w > 0.0f ? w * x[k][s].x : 0.0f;
+            t[k].y += w > 0.0f ? w * x[k][s].y : 0.0f;
+            t[k].z += w > 0.0f ? w * x[k][s].z : 0.0f;
+            t[k].w += w > 0.0f ? w * x[k][s].w : 0.0f;
+          }
       }
     } else {
-      t = o[((int64_t)row * H + h) * ldr + c];
+#pragma unroll
+      for (int k = 0; k < 2; ++k)
+        if (on[k]) t[k] = *reinterpret_cast<const float4*>(p[k]);
     }
-    os[i] = t;
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const int i = i0 + k * 64 * AW, r = i / q4, c = (i - r * q4) * 4;
+      if (i < items) *reinterpret_cast<float4*>(&os[r * orow + c]) = t[k];
+    }
   }
   __syncthreads();
-  constexpr int E = 4;
-  const int e1 = min(dv, ((int)blockIdx.z + 1) * per);
-  for (int e0 = blockIdx.z * per + wave * E; e0 < e1; e0 += 8 * E) {
-    float acc[E][RB];
+  if (e0 >= dv) return;
+  f32x4_t acc[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
+  for (int c0 = 0; c0 < orow - 4; c0 += 32 * U) {
+    if (c0 > 0) load(c0);
 #pragma unroll
-    for (int e = 0; e < E; ++e)
+    for (int u = 0; u < U; ++u) {
+      const int c = c0 + 32 * u;
+      if (c >= orow - 4) break;             // uniform
+      float z[8];                           // (zero beyond the latent)
+      ld8(&os[l16 * orow + c + 8 * g4], z);
 #pragma unroll
-      for (int r = 0; r < RB; ++r) acc[e][r] = 0.0f;
-    for (int c = lane * 8; c < ldr; c += 512) {
-      float w[E][8];
-#pragma unroll
-      for (int e = 0; e < E; ++e) ld8(uv + ((int64_t)h * dv + min(e0 + e, e1 - 1)) * ldr + c, w[e]);
-#pragma unroll
-      for (int r = 0; r < RB; ++r) {
-        float x[8];
-        ld8(os + r * ldr + c, x);
-#pragma unroll
-        for (int e = 0; e < E; ++e)
-#pragma unroll
-          for (int j = 0; j < 8; ++j) acc[e][r] = fmaf(w[e][j], x[j], acc[e][r]);
-      }
+      for (int i = 0; i < 8; ++i)
+        acc[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(ldf(&wx[u][i]), z[i], acc[i & 1], 0, 0, 0);
     }
+  }
+  if (l16 >= nr) return;
 #pragma unroll
-    for (int e = 0; e < E; ++e)
-#pragma unroll
-      for (int r = 0; r < RB; ++r) {
-        const float t = wave_sum(acc[e][r]);
-        if (lane == e * RB + r && e0 + e < e1 && row0 + r < rows) stf(y + (int64_t)(row0 + r) * ldy + h * dv + e0 + e, t);
-      }
+  for (int i = 0; i < 4; ++i) {
+    const int e = e0 + 4 * g4 + i;
+    if (e < dv) stf(y + (int64_t)(row0 + l16) * ldy + h * dv + e, acc[0][i] + acc[1][i]);
   }
 }
 
@@ -513,12 +582,20 @@ int launch_partial(const Partial& a, int rows, hipStream_t s) {
   return lr_launch_status();
 }
 
-template <typename T, int RB>
+template <typename T>
 int absorb(const Absorb& a, hipStream_t s) {
-  const size_t lds = sizeof(float) * ((size_t)RB * a.dk + (size_t)RB * 512 * 8);
+  const size_t lds = sizeof(float) * (AW - 1) * 8 * 4 * 64;
+  k_latent_absorb<T><<<dim3(a.H + (a.c ? 1 : 0), (a.rows + 15) / 16, (a.ldr + 127) / 128), dim3(64 * AW), lds, s>>>(a);
+  return lr_launch_status();
+}
+
+template <typename T>
+int up(const float* o, const float* ml, const lr_latent_attention_t* d, int rows, int nsplit, hipStream_t s) {
+  const size_t lds = sizeof(float) * 16 * ((size_t)(d->ldr + 127) / 128 * 128 + 4 + nsplit);
   static std::atomic<unsigned long long> raised{0};
-  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_latent_absorb<T, RB>), lds, raised)) return LR_E_LAUNCH;
-  k_latent_absorb<T, RB><<<dim3(a.H + (a.c ? 1 : 0), (a.rows + RB - 1) / RB, (a.ldr + 127) / 128), dim3(512), lds, s>>>(a);
+  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_latent_up<T>), lds, raised)) return LR_E_LAUNCH;
+  k_latent_up<T><<<dim3(d->H, (rows + 15) / 16, (d->dv + 16 * AW - 1) / (16 * AW)), dim3(64 * AW), lds, s>>>(
+      o, ml, (const T*)d->uv, (T*)d->y, d->ldy, d->H, d->dv, d->ldr, nsplit, rows);
   return lr_launch_status();
 }
 
@@ -532,7 +609,7 @@ int latent_attention(const lr_latent_attention_t* d, hipStream_t s) {
   u16* qb = reinterpret_cast<u16*>(qa);
   Absorb ab = {d->q, d->uk, d->ldq, split ? nullptr : qa, qb, d->scale * LOG2E, d->H, d->dk, d->ldr, rows, d->S,
                d->latent, d->norm, d->ldl, d->pos, d->cache, d->rank, d->Smax, d->eps, d->err};
-  int rc = rows >= 8 ? absorb<T, 4>(ab, s) : absorb<T, 1>(ab, s);
+  int rc = absorb<T>(ab, s);
   if (rc != LR_OK) return rc;
   float* ml = nullptr;
   int ns = 1;
@@ -553,14 +630,7 @@ int latent_attention(const lr_latent_attention_t* d, hipStream_t s) {
     rc = launch_window<float, T, float>(a, d->B, s);
   }
   if (rc != LR_OK) return rc;
-  const size_t per_row = sizeof(float) * ((size_t)d->ldr + ns);
-  if (rows >= 8)
-    k_latent_up<T, 4><<<dim3(d->H, (rows + 3) / 4, 1), dim3(512), 4 * per_row, s>>>(
-        ol, ml, (const T*)d->uv, (T*)d->y, d->ldy, d->H, d->dv, d->ldr, ns, rows, d->dv);
-  else
-    k_latent_up<T, 1><<<dim3(d->H, rows, (d->dv + 31) / 32), dim3(512), per_row, s>>>(
-        ol, ml, (const T*)d->uv, (T*)d->y, d->ldy, d->H, d->dv, d->ldr, ns, rows, 32);
-  return lr_launch_status();
+  return up<T>(ol, ml, d, rows, ns, s);
 }
 
 }  // namespace

@@ -503,36 +503,42 @@ __global__ __launch_bounds__(1024) void k_linear_attention_step(const LinAttn a)
   float* ks = qs + dk;
   float* es = ks + dk;
   float* red = es + dk;               // [rows][dv]
-  const int p = a.pos[0];
-  if (p < 0 || (a.rope && p >= a.rope_len)) {
-    if (a.err && tid == 0) *a.err = LR_DEV_POS_RANGE;
-    return;
-  }
   const int nq = dv / V, nrow = nt / nq;      // threads along dv, state rows side by side
   const int vq = tid % nq, r0 = tid / nq;
   const bool on = r0 < nrow;
   float* st = a.state + (int64_t)bh * dk * dv + vq * V;
-  constexpr int U = 4;
+  constexpr int U = V == 4 ? 8 : 4;
   float s[U][V];
+  // (loads never branch or wait for the position: a row outside goes to row 0 and is not used)
   auto load = [&](int r) {
 #pragma unroll
     for (int u = 0; u < U; ++u) {
       const int c = r + u * nrow;
-      const bool ok = on && c < dk && p > 0;
+      const float* src = st + (on && c < dk ? c * dv : 0);
       if constexpr (V == 4) {
-        const float4 t = ok ? *reinterpret_cast<const float4*>(st + (int64_t)c * dv) : make_float4(0, 0, 0, 0);
+        const float4 t = *reinterpret_cast<const float4*>(src);
         s[u][0] = t.x; s[u][1] = t.y; s[u][2] = t.z; s[u][3] = t.w;
       } else {
-        s[u][0] = ok ? st[(int64_t)c * dv] : 0.0f;
+        s[u][0] = *src;
       }
     }
   };
   load(r0);
   const T* q = reinterpret_cast<const T*>(a.q) + (int64_t)b * a.ld + h * dk;
   const T* k = reinterpret_cast<const T*>(a.k) + (int64_t)b * a.ld + h * dk;
-  float vv[V];
+  T vraw[V];
 #pragma unroll
-  for (int j = 0; j < V; ++j) vv[j] = ldf(reinterpret_cast<const T*>(a.v) + (int64_t)b * a.ld + h * dv + vq * V + j);
+  for (int j = 0; j < V; ++j) vraw[j] = (reinterpret_cast<const T*>(a.v) + (int64_t)b * a.ld + h * dv)[vq * V + j];
+  // (what the last lines need, for the dimension this thread finishes)
+  const int dl = tid < dv ? tid : 0;
+  const T graw = (reinterpret_cast<const T*>(a.g) + (int64_t)b * a.ld + h * dv)[dl];
+  const T nraw = a.norm ? reinterpret_cast<const T*>(a.norm)[dl] : graw;
+  const int p = a.pos[0];
+  if (p < 0 || (a.rope && p >= a.rope_len)) {
+    if (a.err && tid == 0) *a.err = LR_DEV_POS_RANGE;
+    return;
+  }
+  const bool have = p > 0;     // the first token starts from a zero state
   for (int c = tid; c < dk; c += nt) {
     float fq = ldf(q + c), fk = ldf(k + c);
     if (a.rope && c < a.rot) {
@@ -546,7 +552,16 @@ __global__ __launch_bounds__(1024) void k_linear_attention_step(const LinAttn a)
       const T* t = reinterpret_cast<const T*>(a.lowrank) + (int64_t)b * a.ld;
       const T* w = reinterpret_cast<const T*>(a.a2) + (int64_t)(h * dk + c) * a.rank;
       float z = ldf(reinterpret_cast<const T*>(a.a_bias) + h * dk + c);
-      for (int j = 0; j < a.rank; ++j) z = fmaf(ldf(w + j), ldf(t + j), z);
+      if ((a.rank & 7) == 0) {
+        for (int j = 0; j < a.rank; j += 8) {
+          T x[8];
+          __builtin_memcpy(x, __builtin_assume_aligned(w + j, 16), sizeof(x));
+#pragma unroll
+          for (int e = 0; e < 8; ++e) z = fmaf(ldf(&x[e]), ldf(t + j + e), z);
+        }
+      } else {
+        for (int j = 0; j < a.rank; ++j) z = fmaf(ldf(w + j), ldf(t + j), z);
+      }
       la = log_sigmoid_f(z) * a.inv_tau * LOG2E;
     } else {
       la = a.head_decay[h] * LOG2E;
@@ -555,6 +570,9 @@ __global__ __launch_bounds__(1024) void k_linear_attention_step(const LinAttn a)
     ks[c] = fk * a.k_scale;
     es[c] = exp2_f(la);
   }
+  float vv[V];
+#pragma unroll
+  for (int j = 0; j < V; ++j) vv[j] = ldf(&vraw[j]);
   __syncthreads();
   float acc[V];
 #pragma unroll
@@ -569,7 +587,7 @@ __global__ __launch_bounds__(1024) void k_linear_attention_step(const LinAttn a)
         float n[V];
 #pragma unroll
         for (int j = 0; j < V; ++j) {
-          n[j] = fmaf(e, s[u][j], kk * vv[j]);
+          n[j] = fmaf(e, have ? s[u][j] : 0.0f, kk * vv[j]);
           acc[j] = fmaf(n[j], qq, acc[j]);
         }
         if constexpr (V == 4) *reinterpret_cast<float4*>(st + (int64_t)c * dv) = make_float4(n[0], n[1], n[2], n[3]);
@@ -582,28 +600,20 @@ __global__ __launch_bounds__(1024) void k_linear_attention_step(const LinAttn a)
     for (int j = 0; j < V; ++j) red[r0 * dv + vq * V + j] = acc[j];
   }
   __syncthreads();
-  // the head's output, its mean square, gain and gate
-  float mine = 0.0f, ss = 0.0f;
+  // the head's output, its mean square, gain and gate (at least dv threads: one dimension each)
+  float t = 0.0f;
   __shared__ float wsum[16];
-  for (int d = tid; d < dv; d += nt) {
-    float t = 0.0f;
-    for (int r = 0; r < nrow; ++r) t += red[r * dv + d];
-    red[d] = t;        // (row 0 of column d is read by this thread only)
-    ss += t * t;
-    mine = t;
-  }
-  ss = wave_sum(ss);
+  if (tid < dv)
+    for (int r = 0; r < nrow; ++r) t += red[r * dv + tid];
+  const float ss = wave_sum(t * t);
   if ((tid & 63) == 0) wsum[tid >> 6] = ss;
   __syncthreads();
   float tot = 0.0f;
-  for (int w = 0; w < (nt >> 6); ++w) tot += wsum[w];
+  for (int w = 0; w * 64 < dv; ++w) tot += wsum[w];
   const float inv = rsq_f(tot / (float)dv + a.eps);
-  (void)mine;
-  for (int d = tid; d < dv; d += nt) {
-    const float gain = a.norm ? ldf(reinterpret_cast<const T*>(a.norm) + d) : 1.0f;
-    const float gate = silu_f(ldf(reinterpret_cast<const T*>(a.g) + (int64_t)b * a.ld + h * dv + d));
-    stf(reinterpret_cast<T*>(a.y) + (int64_t)b * a.ldy + h * dv + d, red[d] * inv * gain * gate);
-  }
+  if (tid < dv)
+    stf(reinterpret_cast<T*>(a.y) + (int64_t)b * a.ldy + h * dv + tid,
+        t * inv * (a.norm ? ldf(&nraw) : 1.0f) * silu_f(ldf(&graw)));
 }
 
 // ---------------------------------------------------------------------------------------------- host
@@ -622,6 +632,7 @@ int fill(const lr_linear_attention_t* d, LinAttn& a) {
   if (d->ld > (1 << 24) || d->ldy > (1 << 24) || (int64_t)d->H * d->dk > (1 << 24)) return LR_E_UNSUPPORTED;  // 32-bit offsets in a chunk
   if (d->dk > MAX_DIM || d->dv > MAX_DIM) return LR_E_UNSUPPORTED;
   const bool gated = d->lowrank != nullptr;
+  LR_OPTIONAL_PTR(d->a2);
   if (gated && (d->a2 == nullptr || d->a_bias == nullptr)) return LR_E_NULL;
   if (gated && (d->rank <= 0 || !(d->tau > 0.0f))) return LR_E_SHAPE;
   if (gated && d->rank > 1024) return LR_E_UNSUPPORTED;
@@ -708,9 +719,9 @@ template <typename T>
 int step(const LinAttn& a, hipStream_t s) {
   const int v = a.dv % 4 == 0 ? 4 : 1;
   const int nq = a.dv / v;
-  // about 16 state values per thread, at least one state row side by side
+  // about 16 state values per thread, at least a thread per value dimension
   int nt = (int)(((int64_t)a.dk * a.dv / 16 + 63) / 64 * 64);
-  if (nt < nq) nt = (nq + 63) / 64 * 64;
+  if (nt < a.dv) nt = (a.dv + 63) / 64 * 64;
   nt = nt < 64 ? 64 : (nt > 1024 ? 1024 : nt);
   const size_t lds = sizeof(float) * ((size_t)3 * a.dk + (size_t)(nt / nq) * a.dv + 4);
   if (v == 4) {
