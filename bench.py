@@ -1,6 +1,7 @@
 """Headline benchmark: batch-1 greedy decode of one TP=8 rank shard of Ladder-70B on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--no-cpu-baseline]
+    python bench.py --lasivik [SIZE ...]     # another workload, see below
 
 A "step" is one decode step (one new token per sequence) of the whole per-rank forward pass,
 replayed as a captured hipGraph: embedding -> 80 ladder blocks -> final add/norm -> vocab-shard
@@ -36,6 +37,10 @@ Measured in the same run and reported as extra keys (not the headline; --no-extr
 `fp8`         : the same shard with weight-only e4m3 projections at batch 1 (the one-kernel step on e4m3 weights)
                and batch 8 (per-op kernels): ms per step and the fraction of 8 TB/s on ITS algorithmic bytes
                (one byte per weight + scales).
+`--lasivik`   : instead of the above, the Lasivik hybrid beside the dense family at equal layer sizes (lasivik-1b /
+               gpt_dense:ladder-1b, lasivik-8b / gpt_dense:ladder-8b; random weights): prefill and decode throughput at
+               several batch sizes, and the kernels only one of the two has, each timed alone over data that does not
+               fit the caches, with the fraction of its roofline.  One JSON line of its own.
 `prefill`     : Ladder-8B, batch 32 x 2048 prompt tokens, causal prefill with last-position logits:
                seconds, algorithmic TFLOP/s and the fraction of 2.5 PFLOP/s (dense bf16 MFMA peak)."""
 import argparse
@@ -108,10 +113,13 @@ def decode_run(bm, model, prompt, B, T, K, W):
     rows = prompt.view(1, -1).repeat(B, 1)
     first = bm.prefill(model, rows, torch.arange(T, device=prompt.device, dtype=torch.int32), greedy=True).clone()
     dg = bm.get_cuda_graphs_for_decode(model, prompt, B, new, first, greedy=True)
+    states = [(s, s.clone()) for s in model.recurrent_states()]
     dg.reset(first)
     for _ in range(W):
         dg.replay()
     dg.reset(first)
+    for s, kept in states:               # the timed steps start where the prompt ended, here too
+        s.copy_(kept)
     torch.cuda.synchronize()
     t0 = time.perf_counter()
     for _ in range(K):
@@ -222,6 +230,176 @@ def extra_prefill(bm, B=32, T=2048, reps=2):
             "prompt_tok_per_s": round(B * T / sec, 1)}
 
 
+FP32_MATRIX_PEAK_TFLOPS = 157.3   # v_mfma_f32, the recurrences' products
+
+
+def _graph_us(calls, reps=5):
+    """Mean microseconds per call of a list of launches, captured into one hipGraph and replayed."""
+    import torch
+
+    for c in calls[:2]:
+        c()
+    torch.cuda.synchronize()
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        for c in calls:
+            c()
+    g.replay()
+    torch.cuda.synchronize()
+    ev0, ev1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+    ev0.record()
+    for _ in range(reps):
+        g.replay()
+    ev1.record()
+    torch.cuda.synchronize()
+    return 1e3 * ev0.elapsed_time(ev1) / (reps * len(calls))
+
+
+def _kernel_row(name, us, bound, work):
+    """`work`: bytes (bound hbm) or FLOP (bound mfma: bf16, mfma_f32)."""
+    peak = {"hbm": HBM_PEAK_GBPS * 1e9, "mfma": MFMA_PEAK_TFLOPS * 1e12, "mfma_f32": FP32_MATRIX_PEAK_TFLOPS * 1e12}[bound]
+    return {"kernel": name, "us": round(us, 2), "bound": bound, "work": int(work), "frac": round(work / (us * 1e-6) / peak, 4)}
+
+
+def mixer_kernels(hybrid, dense, B, T, decode):
+    """The kernels the hybrid and the dense model do not share, at `B` sequences of `T` tokens (decode: one more token on
+    top of them), on tensors of those models' shapes.  Inputs are rotated through copies that together exceed the caches."""
+    import torch
+
+    from gpt_fast import _hip
+    from gpt_fast.mixers import rotate_half_table
+
+    dev, BF = "cuda", torch.bfloat16
+    S = 1 if decode else T
+    rows = B * S
+    pos = torch.arange(T, T + 1, dtype=torch.int32, device=dev) if decode else torch.arange(T, dtype=torch.int32, device=dev)
+    rnd = lambda *s, dt=BF: torch.randn(*s, device=dev, dtype=torch.float32).to(dt)
+    copies = lambda nbytes: max(2, min(64, (600 << 20) // max(int(nbytes), 1))) if decode else 2
+    out = []
+    mixers = {blk.mixer.args.kind: blk.mixer for blk in hybrid.layers}
+    for kind in ("gla", "retention"):
+        m = mixers[kind]
+        a = m.args
+        carried = 2 * B * a.heads * a.dim * a.vdim * 4
+        n = copies(carried)
+        states = [torch.zeros(B, a.heads, a.dim, a.vdim, device=dev) for _ in range(n)]
+        proj, y = rnd(rows, (m.proj_cols + 7) // 8 * 8), torch.empty(rows, m.y_cols, dtype=BF, device=dev)
+        need = _hip.linear_attention_scratch_bytes(B, S, a.heads, a.dim, a.vdim, kind == "gla")
+        scratch = torch.empty(need, dtype=torch.uint8, device=dev) if need else None
+        if kind == "gla":
+            kw = dict(q_scale=a.dim ** -0.5, norm=rnd(a.vdim), gate=(rnd(a.heads * a.dim, a.decay_rank), rnd(a.heads * a.dim), a.tau))
+        else:
+            kw = dict(k_scale=a.dim ** -0.5, rope=rotate_half_table(T + 8, a.rot_dims, a.rot_base).to(dev),
+                      head_decay=torch.tensor(a.decay, device=dev).log())
+        us = _graph_us([lambda s=s: _hip.linear_attention(proj, y, s, pos, B, S, a.heads, a.dim, a.vdim, 1e-5, scratch=scratch, **kw)
+                        for s in states])
+        # per token and head: the state is multiplied by q and added k v^T to; inside a chunk of 16 the scores and their sums
+        flop = rows * a.heads * (4 * a.dim * a.vdim + 2 * 16 * (a.dim + a.vdim) // 2)
+        out.append(_kernel_row(f"lr_linear_attention ({kind}, {a.heads} heads of {a.dim} x {a.vdim})", us,
+                               "hbm" if decode else "mfma_f32", carried + 2 * rows * (m.proj_cols + m.y_cols) if decode else flop))
+        del states, proj, y, scratch
+    m = mixers["latent_attention"]
+    a = m.args
+    L = T + 8
+    nq, nv = a.heads * a.dim, a.heads * a.vdim
+    seen = min(T + 1, a.window)
+    if decode:
+        nbytes = B * seen * m.rank_p * 2 + (nq + nv) * m.rank_p * 2
+        n = copies(nbytes)
+        caches, ups = [rnd(B, L, m.rank_p) for _ in range(n)], [rnd(nq + nv, m.rank_p) for _ in range(n)]
+        q, c, gain = rnd(rows, nq), rnd(rows, m.rank_p), rnd(m.rank_p)
+        y = torch.empty(rows, nv, dtype=BF, device=dev)
+        scratch = torch.empty(_hip.latent_attention_scratch_bytes(B, 1, a.heads, m.rank_p, a.window, L), dtype=torch.uint8, device=dev)
+        us = _graph_us([lambda i=i: _hip.latent_attention(q, ups[i][:nq], ups[i][nq:], caches[i], y, pos, scratch, B, 1, a.heads, a.dim,
+                                                          a.vdim, a.window, a.scale, new=(c, gain, a.kv_rank, 1e-5)) for i in range(n)])
+        out.append(_kernel_row(f"lr_latent_attention ({a.heads} heads, rank {a.kv_rank}, window {a.window}; three launches)", us, "hbm", nbytes))
+        del caches, ups
+    else:
+        nk = min(T + a.window - 1, L)
+        q, kv, y = rnd(rows, nq), rnd(B * nk, nq + nv), torch.empty(rows, nv, dtype=BF, device=dev)
+        us = _graph_us([lambda: _hip.window_attention(q, kv, y, pos, B, T, a.heads, a.dim, a.vdim, a.window, nk, L, a.scale)] * 2)
+        keys = sum(min(i + 1, a.window) for i in range(T))
+        out.append(_kernel_row(f"lr_window_attention ({a.heads} heads of {a.dim}, window {a.window})", us, "mfma",
+                               B * a.heads * keys * 2 * (a.dim + a.vdim)))
+    # the dense model's counterpart
+    d = dense.config
+    Hq, Hkv, hd = d.n_head_local, d.n_kv_local, d.head_dim
+    nbytes = 2 * B * (T + 1) * Hkv * hd * 2
+    n = copies(nbytes)
+    kcs, vcs = [rnd(B, Hkv, L, hd) for _ in range(n)], [rnd(B, Hkv, L, hd) for _ in range(n)]
+    q, y = rnd(rows, Hq * hd), torch.empty(rows, Hq * hd, dtype=BF, device=dev)
+    if decode:
+        scratch = torch.empty(_hip.attn_decode_scratch_bytes(B, Hq, hd, L) // 4, device=dev)
+        us = _graph_us([lambda i=i: _hip.attn_decode(q, kcs[i], vcs[i], pos, y, scratch, B, Hq, Hkv, hd) for i in range(n)])
+        out.append(_kernel_row(f"dense: lr_attn_decode ({Hq} / {Hkv} heads of {hd}; two launches)", us, "hbm", nbytes))
+    else:
+        us = _graph_us([lambda: _hip.attn_prefill(q, kcs[0], vcs[0], pos, y, B, T, Hq, Hkv, hd)] * 2)
+        out.append(_kernel_row(f"dense: lr_attn_prefill ({Hq} / {Hkv} heads of {hd})", us, "mfma", B * Hq * (T * (T + 1) // 2) * 4 * hd))
+    del kcs, vcs
+    # the norms, a launch per sublayer in both
+    D = hybrid.config.dim
+    n = copies(rows * D * 12)
+    xs, ds = [rnd(rows, D, dt=torch.float32) for _ in range(n)], [rnd(rows, D) for _ in range(n)]
+    xc, gain = torch.empty(rows, D, dtype=BF, device=dev), rnd(D)
+    us = _graph_us([lambda i=i: _hip.residual_rmsnorm(xs[i], 2.0, ds[i], gain, xs[i], xc, 1e-5, gain_offset=1.0) for i in range(n)])
+    out.append(_kernel_row("lr_residual_rmsnorm (fp32 residual)", us, "hbm", rows * D * (4 + 2 + 4 + 2)))
+    bs = [rnd(rows, D) for _ in range(n)]
+    us = _graph_us([lambda i=i: _hip.add_rmsnorm(bs[i], ds[i], None, gain, bs[i], xc, 1e-5) for i in range(n)])
+    out.append(_kernel_row("dense: lr_add_rmsnorm", us, "hbm", rows * D * 8))
+    torch.cuda.empty_cache()
+    return out
+
+
+LASIVIK_PAIRS = {"1b": ("gpt_lasivik:lasivik-1b", "gpt_dense:ladder-1b"), "8b": ("gpt_lasivik:lasivik-8b", "gpt_dense:ladder-8b")}
+
+
+def lasivik_compare(sizes, T=1792, K=32, W=5):
+    import torch
+
+    import benchmark as bm
+    from gpt_fast import _hip
+
+    _hip.load()
+    out = {"workload": "lasivik beside dense", "prompt_len": T, "data": "synthetic", "dtype": "bf16", "models": [], "kernels": []}
+    for size in sizes:
+        models = [bm._load_model(name, "cuda", torch.bfloat16, seed=0, verbose=False) for name in LASIVIK_PAIRS[size]]
+        g = torch.Generator(device="cuda")
+        g.manual_seed(1)
+        prompt = torch.randint(0, 100000, (T,), device="cuda", generator=g)
+        for name, model in zip(LASIVIK_PAIRS[size], models):
+            model.last_logits_only = True
+            row = {"model": name, "parameters": sum(p.numel() for p in model.parameters()), "prefill": [], "decode": []}
+            count = sum(p.numel() for n, p in model.named_parameters() if p.dim() == 2 and not n.startswith(("tok_emb", "output")))
+            for B in (1, 8):
+                model.max_seq_length = -1
+                model.setup_caches(B, T + 8)
+                rows, pos = prompt.view(1, -1).repeat(B, 1), torch.arange(T, device="cuda", dtype=torch.int32)
+                bm.prefill(model, rows, pos, greedy=True)
+                torch.cuda.synchronize()
+                t0 = time.perf_counter()
+                for _ in range(3):
+                    bm.prefill(model, rows, pos, greedy=True)
+                torch.cuda.synchronize()
+                sec = (time.perf_counter() - t0) / 3
+                row["prefill"].append({"batch": B, "ms": round(1e3 * sec, 3), "tok_per_s": round(B * T / sec, 1),
+                                       "projection_TFLOPs": round(2 * count * B * T / sec / 1e12, 1)})
+            for B in (1, 8, 32):
+                ms, _, dg = decode_run(bm, model, prompt, B, T, K, W)
+                nbytes = bm.decode_bytes_per_step(model if hasattr(model, "decode_bytes") else model.config, B, T + K // 2)
+                row["decode"].append({"batch": B, "ms_per_step": round(ms, 4), "tok_per_s": round(B * 1e3 / ms, 1),
+                                      "bytes_per_step": int(nbytes), "frac": round(nbytes / (ms * 1e-3) / 1e9 / HBM_PEAK_GBPS, 4)})
+                del dg
+            model.check_device_errors()
+            model.release_workspace()
+            out["models"].append(row)
+        for B, decode in ((1, False), (8, False), (1, True), (8, True), (32, True)):
+            out["kernels"].append({"size": size, "batch": B, "phase": "decode" if decode else "prefill",
+                                   "rows": mixer_kernels(models[0], models[1], B, T, decode)})
+        del models, model
+        torch.cuda.empty_cache()
+    print(json.dumps(out), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -238,6 +416,8 @@ def main():
                          "one-kernel step: the comparison point, not the headline")
     ap.add_argument("--fp8", action="store_true",
                     help="weight-only e4m3 projections (gpt_fast.quantize): a profiling aid, not the headline")
+    ap.add_argument("--lasivik", nargs="*", choices=sorted(LASIVIK_PAIRS), metavar="SIZE",
+                    help="the Lasivik family beside the dense one instead of the headline (sizes 1b and 8b; default both)")
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="also run a plain 1 GiB device copy (reads 1 GiB, writes 1 GiB) a few times: under "
                          "rocprofv3 --pmc its FETCH_SIZE / WRITE_SIZE readings calibrate the counters' unit")
@@ -253,6 +433,8 @@ def main():
     from gpt_fast import _hip
 
     assert torch.cuda.is_available(), "bench.py needs the MI355X"
+    if args.lasivik is not None:
+        return lasivik_compare(args.lasivik or sorted(LASIVIK_PAIRS))
     _hip.load()
     dev = "cuda"
     B, T, K, W = args.batch, args.prompt, args.steps, args.warmup
