@@ -280,6 +280,19 @@ __global__ __launch_bounds__(512) void k_latent_partial(const Partial a) {
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g4 = lane >> 4, l16 = lane & 15;
   const int sp = blockIdx.x, hb = blockIdx.y * 32, row = blockIdx.z;
   const int b = row / a.S, s = row - b * a.S;
+  const int kq = wave & 3, hg = wave >> 2;
+  // ---- q' of the wave's 16 heads (asked for before the position is known)
+  u32x4_t qh[KS];
+  {
+    const int head = hb + hg * 16 + l16;
+    const int64_t at = ((int64_t)row * a.H + head) * a.ldr;
+#pragma unroll
+    for (int j = 0; j < KS; ++j) {
+      const int c = 32 * j + 8 * g4;
+      qh[j] = u32x4_t{0, 0, 0, 0};
+      if (head < a.H && c < a.ldr) qh[j] = *reinterpret_cast<const u32x4_t*>(a.q + at + c);
+    }
+  }
   const int p = min(a.pos[s], a.Smax - 1);
   const int lo = max(0, p - a.window + 1), n = p - lo + 1;
   const int per = ((n + a.nsplit - 1) / a.nsplit + KT - 1) / KT * KT;
@@ -293,7 +306,6 @@ __global__ __launch_bounds__(512) void k_latent_partial(const Partial a) {
     }
     return;
   }
-  const int kq = wave & 3, hg = wave >> 2;
   // Staging: an item is eight columns of two neighbouring keys, stored by column as dwords of two keys.  Column slices
   // that a wave writes together would meet in two LDS banks (their rows lie 8 * 36 dwords apart): the groups of eight
   // keys of a row are permuted by its slice, which spreads them over all banks and leaves a group whole for the reader.
@@ -319,18 +331,6 @@ __global__ __launch_bounds__(512) void k_latent_partial(const Partial a) {
   };
   auto vgroup = [](int group, int r) { return group ^ ((r >> 4) & 7); };
   stage_load(k0);
-  // ---- q' of the wave's 16 heads
-  u32x4_t qh[KS];
-  {
-    const int head = hb + hg * 16 + l16;
-    const int64_t at = ((int64_t)row * a.H + head) * a.ldr;
-#pragma unroll
-    for (int j = 0; j < KS; ++j) {
-      const int c = 32 * j + 8 * g4;
-      qh[j] = u32x4_t{0, 0, 0, 0};
-      if (head < a.H && c < a.ldr) qh[j] = *reinterpret_cast<const u32x4_t*>(a.q + at + c);
-    }
-  }
   f32x4_t o[2][RT];
 #pragma unroll
   for (int g = 0; g < 2; ++g)
@@ -451,21 +451,27 @@ __global__ __launch_bounds__(512) void k_latent_partial(const Partial a) {
     }
 }
 
-// ---- the ranges' results merged, then through W_uv: y[row, h dv + e] = W_uv[h dv + e, :] . o[row, h, :], 16 rows and 64 value
-// dimensions of a head per workgroup, 16 of them per wave; fp32 products.
-template <typename T>
-__global__ __launch_bounds__(64 * AW) void k_latent_up(const float* __restrict__ o, const float* __restrict__ ml,
-                                                       const T* __restrict__ uv, T* __restrict__ y, int64_t ldy, int H,
-                                                       int dv, int ldr, int nsplit, int rows) {
-  extern __shared__ __attribute__((aligned(16))) float os[];   // [16][orow] and [16][nsplit]
-  const int orow = (ldr + 127) / 128 * 128 + 4;
-  float* ws = os + 16 * orow;
-  const int h = blockIdx.x, row0 = blockIdx.y * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+// ---- the ranges' results merged, then through W_uv: y[row, h dv + e] = W_uv[h dv + e, :] . o[row, h, :], UR rows and 64
+// value dimensions of a head per workgroup.  Eight waves: (16 value dimensions, half of the latent columns).  bf16: the
+// fp32 o enters the products as hi + lo; fp32: fp32 products.
+constexpr int UR = 4, UT = 512;
+
+template <typename T, int SB>
+__global__ __launch_bounds__(UT) void k_latent_up(const float* __restrict__ o, const float* __restrict__ ml,
+                                                  const T* __restrict__ uv, T* __restrict__ y, int64_t ldy, int H, int dv,
+                                                  int ldr, int nsplit, int rows) {
+  constexpr bool BF = sizeof(T) == 2;
+  extern __shared__ __attribute__((aligned(16))) float os[];   // fp32: [16][orow]; bf16: hi [16][orow], lo [16][orow]
+  __shared__ float ws[UR][64];
+  __shared__ float part[4][64][4];
+  const int kp = (ldr + 63) / 64 * 64, orow = kp + 8;
+  u16 *oh = reinterpret_cast<u16*>(os), *ol = oh + 16 * orow;
+  const int h = blockIdx.x, row0 = blockIdx.y * UR, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int g4 = lane >> 4, l16 = lane & 15;
-  const int nr = min(16, rows - row0);
+  const int nr = min(UR, rows - row0);
   // this wave's rows of W_uv, 32 columns a step: lane (g4, l16) has eight columns of row l16.  The first steps' loads are
   // out before the merge begins.
-  const int e0 = blockIdx.z * 16 * AW + wave * 16;
+  const int e0 = blockIdx.z * 64 + (wave & 3) * 16, cb = (wave >> 2) * (kp / 2), ce = cb + kp / 2;
   constexpr int U = 8;
   const T* w = uv + ((int64_t)h * dv + min(e0 + l16, dv - 1)) * ldr;
   T wx[U][8];
@@ -474,85 +480,99 @@ __global__ __launch_bounds__(64 * AW) void k_latent_up(const float* __restrict__
     for (int u = 0; u < U; ++u)
       __builtin_memcpy(wx[u], __builtin_assume_aligned(w + min(c0 + 32 * u + 8 * g4, ldr - 8), 16), sizeof(wx[u]));
   };
-  load(0);
-  if (ml) {
+  load(cb);
+  // ---- an item is four columns of a row; its ranges' values, SB at a time, do not wait for the ranges' weights.  A range
+  // beyond the last repeats the last one's place with weight 0.
+  const int q4 = kp / 4, items = UR * q4;
+  const int ns = ml ? nsplit : 1;
+  float4 x[SB];
+  auto fetch = [&](int i, int s0) {
+    const int r = i / q4, c = (i - r * q4) * 4;
+    const float* p = o + ((int64_t)(row0 + min(r, nr - 1)) * H + h) * ns * ldr + min(c, ldr - 4);
+#pragma unroll
+    for (int s = 0; s < SB; ++s)
+      if (s0 + s < ns) x[s] = *reinterpret_cast<const float4*>(p + (int64_t)(s0 + s) * ldr);
+  };
+  fetch(min(tid, items - 1), 0);
+  if (wave < UR) {
     // weight of every range: 2^(m - M) / sum of 2^(m - M) l
-    for (int r = wave; r < nr; r += AW) {
-      const float* p = ml + ((int64_t)(row0 + r) * H + h) * nsplit * 2;
-      const float m = lane < nsplit ? p[2 * lane] : -INFINITY, l = lane < nsplit ? p[2 * lane + 1] : 0.0f;
-      const float w = exp2_f(m - wave_max(m));
-      const float t = wave_sum(w * l);
-      if (lane < nsplit) ws[r * nsplit + lane] = w / t;
+    const float* p = ml + ((int64_t)(row0 + min(wave, nr - 1)) * H + h) * nsplit * 2;
+    float m = lane == 0 ? 0.0f : -INFINITY, l = 1.0f;
+    if (ml) {
+      m = lane < nsplit ? p[2 * lane] : -INFINITY;
+      l = lane < nsplit ? p[2 * lane + 1] : 0.0f;
     }
-    __syncthreads();
+    const float f = exp2_f(m - wave_max(m));
+    ws[wave][lane] = f / wave_sum(f * l);
   }
-  // Items of four columns, two per thread and eight ranges at a time in flight.  A row beyond the last repeats the last
-  // one's place with weight 0, as does a range beyond the last.
-  const int q4 = orow / 4 - 1, items = 16 * q4;
-  for (int i0 = tid; i0 < items; i0 += 2 * 64 * AW) {
-    float4 t[2] = {make_float4(0, 0, 0, 0), make_float4(0, 0, 0, 0)};
-    const float* p[2];
-    const float* wr[2];
-    bool on[2];
+  // (rows of the products that are nobody's)
+  for (int i = tid; i < (16 - UR) * orow; i += UT) {
+    if constexpr (BF) oh[UR * orow + i] = ol[UR * orow + i] = 0;
+    else os[UR * orow + i] = 0.0f;
+  }
+  __syncthreads();
+  for (int i = tid; i < items; i += UT) {
+    const int r = i / q4, c = (i - r * q4) * 4;
+    float t[4] = {0, 0, 0, 0};
+    for (int s0 = 0; s0 < ns; s0 += SB) {
+      if (i != tid || s0 > 0) fetch(i, s0);
 #pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      const int i = i0 + k * 64 * AW, r = i / q4, c = (i - r * q4) * 4;
-      on[k] = i < items && r < nr && c < ldr;
-      p[k] = o + ((int64_t)(row0 + (on[k] ? r : 0)) * H + h) * nsplit * ldr + (on[k] ? c : 0);
-      wr[k] = ws + (on[k] ? r : 0) * nsplit;
+      for (int s = 0; s < SB; ++s)
+        if (s0 + s < ns) {
+          const float f = ws[r][s0 + s];   // 0: nothing was written there
+          t[0] += f > 0.0f ? f * x[s].x : 0.0f;
+          t[1] += f > 0.0f ? f * x[s].y : 0.0f;
+          t[2] += f > 0.0f ? f * x[s].z : 0.0f;
+          t[3] += f > 0.0f ? f * x[s].w : 0.0f;
+        }
     }
-    if (!on[0] && !on[1]) {
-      // (rows and columns that are nobody's: zero)
-    } else if (ml) {
-      for (int s0 = 0; s0 < nsplit; s0 += 8) {
-        float4 x[2][8];
+    const bool ok = r < nr && c < ldr;
 #pragma unroll
-        for (int k = 0; k < 2; ++k)
+    for (int j = 0; j < 4; ++j) t[j] = ok ? t[j] : 0.0f;
+    if constexpr (BF) {
+      st4(&oh[r * orow + c], t);
 #pragma unroll
-          for (int s = 0; s < 8; ++s) x[k][s] = *reinterpret_cast<const float4*>(p[k] + (int64_t)min(s0 + s, nsplit - 1) * ldr);
-#pragma unroll
-        for (int k = 0; k < 2; ++k)
-#pragma unroll
-          for (int s = 0; s < 8; ++s) {
-            const float w = s0 + s < nsplit && on[k] ? wr[k][s0 + s] : 0.0f;   // 0: nothing was written there
-            t[k].x += w > 0.0f ? w * x[k][s].x : 0.0f;
-            t[k].y += w > 0.0f ? w * x[k][s].y : 0.0f;
-            t[k].z += w > 0.0f ? w * x[k][s].z : 0.0f;
-            t[k].w += w > 0.0f ? w * x[k][s].w : 0.0f;
-          }
-      }
+      for (int j = 0; j < 4; ++j) t[j] -= round_bf(t[j]);
+      st4(&ol[r * orow + c], t);
     } else {
-#pragma unroll
-      for (int k = 0; k < 2; ++k)
-        if (on[k]) t[k] = *reinterpret_cast<const float4*>(p[k]);
-    }
-#pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      const int i = i0 + k * 64 * AW, r = i / q4, c = (i - r * q4) * 4;
-      if (i < items) *reinterpret_cast<float4*>(&os[r * orow + c]) = t[k];
+      st4(&os[r * orow + c], t);
     }
   }
   __syncthreads();
-  if (e0 >= dv) return;
   f32x4_t acc[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
-  for (int c0 = 0; c0 < orow - 4; c0 += 32 * U) {
-    if (c0 > 0) load(c0);
+  for (int c0 = cb; c0 < ce; c0 += 32 * U) {
+    if (c0 > cb) load(c0);
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      const int c = c0 + 32 * u;
-      if (c >= orow - 4) break;             // uniform
-      float z[8];                           // (zero beyond the latent)
-      ld8(&os[l16 * orow + c + 8 * g4], z);
+      const int c = c0 + 32 * u + 8 * g4;
+      if (c0 + 32 * u >= ce) break;         // uniform
+      if constexpr (BF) {
+        bf16x8_t a;
+        __builtin_memcpy(&a, wx[u], sizeof(a));
+        const u32x4_t zh = *reinterpret_cast<const u32x4_t*>(&oh[l16 * orow + c]);
+        const u32x4_t zl = *reinterpret_cast<const u32x4_t*>(&ol[l16 * orow + c]);
+        acc[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, __builtin_bit_cast(bf16x8_t, zh), acc[0], 0, 0, 0);
+        acc[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, __builtin_bit_cast(bf16x8_t, zl), acc[1], 0, 0, 0);
+      } else {
+        float z[8];
+        ld8(&os[l16 * orow + c], z);
 #pragma unroll
-      for (int i = 0; i < 8; ++i)
-        acc[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(ldf(&wx[u][i]), z[i], acc[i & 1], 0, 0, 0);
+        for (int i = 0; i < 8; ++i)
+          acc[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(ldf(&wx[u][i]), z[i], acc[i & 1], 0, 0, 0);
+      }
     }
   }
-  if (l16 >= nr) return;
+  acc[0] += acc[1];
+  if (wave >= 4) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) part[wave & 3][lane][i] = acc[0][i];
+  }
+  __syncthreads();
+  if (wave >= 4 || l16 >= nr) return;
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int e = e0 + 4 * g4 + i;
-    if (e < dv) stf(y + (int64_t)(row0 + l16) * ldy + h * dv + e, acc[0][i] + acc[1][i]);
+    if (e < dv) stf(y + (int64_t)(row0 + l16) * ldy + h * dv + e, acc[0][i] + part[wave][lane][i]);
   }
 }
 
@@ -589,14 +609,20 @@ int absorb(const Absorb& a, hipStream_t s) {
   return lr_launch_status();
 }
 
-template <typename T>
-int up(const float* o, const float* ml, const lr_latent_attention_t* d, int rows, int nsplit, hipStream_t s) {
-  const size_t lds = sizeof(float) * 16 * ((size_t)(d->ldr + 127) / 128 * 128 + 4 + nsplit);
+template <typename T, int SB>
+int up_as(const float* o, const float* ml, const lr_latent_attention_t* d, int rows, int nsplit, hipStream_t s) {
+  const size_t lds = (size_t)16 * ((d->ldr + 63) / 64 * 64 + 8) * sizeof(float);   // (hi and lo, or fp32)
   static std::atomic<unsigned long long> raised{0};
-  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_latent_up<T>), lds, raised)) return LR_E_LAUNCH;
-  k_latent_up<T><<<dim3(d->H, (rows + 15) / 16, (d->dv + 16 * AW - 1) / (16 * AW)), dim3(64 * AW), lds, s>>>(
+  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_latent_up<T, SB>), lds, raised)) return LR_E_LAUNCH;
+  k_latent_up<T, SB><<<dim3(d->H, (rows + UR - 1) / UR, (d->dv + 63) / 64), dim3(UT), lds, s>>>(
       o, ml, (const T*)d->uv, (T*)d->y, d->ldy, d->H, d->dv, d->ldr, nsplit, rows);
   return lr_launch_status();
+}
+
+// (the registers of eight ranges' values instead of sixteen's leave room for a second workgroup on a CU)
+template <typename T>
+int up(const float* o, const float* ml, const lr_latent_attention_t* d, int rows, int nsplit, hipStream_t s) {
+  return nsplit <= 8 ? up_as<T, 8>(o, ml, d, rows, nsplit, s) : up_as<T, 16>(o, ml, d, rows, nsplit, s);
 }
 
 template <typename T>
