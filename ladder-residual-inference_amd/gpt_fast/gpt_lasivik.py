@@ -83,6 +83,7 @@ class HybridBlock(nn.Module):
 
 class GPTLasivik(GPTBase):
     family = "lasivik"
+    supports_fp8 = False
 
     def _make_block(self, config, layer_idx):
         return HybridBlock(config, config.layers[layer_idx])

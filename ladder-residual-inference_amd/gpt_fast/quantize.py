@@ -57,6 +57,8 @@ class WeightOnlyFp8Linear(nn.Module):
 def quantize_model_fp8(model: nn.Module, include_output: bool = True) -> nn.Module:
     """Replace every projection of the blocks (wqkv / wqkv1, wo, w1, w2) and, optionally, the lm_head by its
     weight-only fp8 form, in place.  Norm gains and the embedding table keep the model dtype."""
+    if not getattr(model, "supports_fp8", True):
+        raise NotImplementedError(f"{type(model).__name__} has no weight-only e4m3 projections")
     for blk in model.layers:
         for parent in (getattr(blk, "attention", None), getattr(blk, "feed_forward", None)):
             if parent is None:

@@ -170,6 +170,16 @@ def test_rank_shards_are_refused(monkeypatch):
         args_from_name("lasivik", "lasivik-1b")
 
 
+def test_weight_only_quantisation_is_refused():
+    from gpt_fast import GPTLasivik
+    from gpt_fast.quantize import quantize_model_fp8
+
+    with torch.device("meta"):
+        model = GPTLasivik.from_name("lasivik-1b")
+    with pytest.raises(NotImplementedError):
+        quantize_model_fp8(model)
+
+
 def test_bytes_per_step_count_weights_states_and_caches():
     import benchmark as bm
     from gpt_fast import GPTLasivik
