@@ -398,7 +398,7 @@ int lr_sample_topk(const void* logits, int64_t ldl, const void* noise, int64_t l
                    int top_k, void* probs, int64_t ldp, int32_t* next_token, lr_stream_t stream);
 
 /* ---------------------------------------------------------------------------------------------
- * Models with an fp32 residual stream and token mixers of other kinds (the Lasivik family).  No
+ * Models with an fp32 residual stream and token mixers of other kinds (the Lasivik and Gepolix families).  No
  * counterpart in the reference.  `dtype` selects the storage of weights and activations: bf16 as
  * everywhere above, or fp32 for running such a model in true 32-bit throughout; the arithmetic
  * named fp32 below is fp32 in both. */
@@ -423,7 +423,7 @@ int lr_logit_cap(void* logits, int64_t ldl, int rows, int V, float scale, float 
 /* lr_linear / lr_swiglu / lr_argmax on fp32 tensors (fp32 matrix-core products, no reduced-precision mode; any sizes). */
 int lr_linear_f32(const float* x, int64_t ldx, const float* w, float* y, int64_t ldy, int M, int N, int K,
                   lr_stream_t stream);
-int lr_swiglu_f32(const float* h, int64_t ldh, float* out, int rows, int I, lr_stream_t stream);
+int lr_swiglu_f32(const float* h, int64_t ldh, float* out, int64_t ldo, int rows, int I, lr_stream_t stream);
 int lr_argmax_f32(const float* logits, int64_t ldl, int32_t* out, int B, int V, lr_stream_t stream);
 
 /* Linear attention with decay over S consecutive tokens per sequence, the state carried from call to call:
@@ -470,9 +470,10 @@ int lr_latent_update(const void* c, int64_t ld, const void* gain, const int32_t*
 int lr_latent_window(const void* cache, const int32_t* pos, void* rows, int B, int n, int window, int ldc, int Smax,
                      int dtype, lr_stream_t stream);
 
-/* Sliding-window softmax attention of S queries per sequence over keys and values expanded from such rows: position i
- * sees positions i - window + 1 .. i.  q [B*S, H*dk] (row stride ldq), k and v: column ranges [B * n_keys, H*dk] and
- * [B * n_keys, H*dv] of buffers with row stride ldk, rows as lr_latent_window orders them; y [B*S, H*dv].
+/* Sliding-window softmax attention of S queries per sequence over keys and values expanded from such rows, or over the rows
+ * of a cache (n_keys == Smax): position i sees positions i - window + 1 .. i.  q [B*S, H*dk] (row stride ldq), k and v:
+ * column ranges [B * n_keys, G*dk] and [B * n_keys, G*dv] of buffers with row stride ldk, rows as lr_latent_window orders
+ * them; y [B*S, H*dv].  G = kv_heads (0: H); query head h reads head h / (H / G).
  * score = (q . k) * scale; scores, softmax and sums in fp32. */
 typedef struct lr_window_attention {
   const void* q;
@@ -482,7 +483,7 @@ typedef struct lr_window_attention {
   void* y;
   int64_t ldy;
   const int32_t* pos;
-  int32_t B, S, H, dk, dv, window, n_keys, Smax, dtype;
+  int32_t B, S, H, dk, dv, window, n_keys, Smax, dtype, kv_heads;
   float scale;
 } lr_window_attention_t;
 int lr_window_attention(const lr_window_attention_t* desc, lr_stream_t stream);
@@ -510,6 +511,91 @@ typedef struct lr_latent_attention {
 } lr_latent_attention_t;
 size_t lr_latent_attention_scratch_bytes(int B, int S, int H, int ldr, int window, int Smax);
 int lr_latent_attention(const lr_latent_attention_t* desc, lr_stream_t stream);
+
+/* r = x + d + sum_k expert_weights[row, k] * expert_out[row * top + k, :]   (fp32; d and expert_out may be NULL), then
+ *     x_out = r    and    x_compute = tanh(alpha * r) * gain + bias
+ * (either may be NULL; x_out may alias x).  alpha: one value; gain, bias [dim]; d, expert_out, alpha, gain, bias and
+ * x_compute in the compute type.  Rows are dense, dim % 8 == 0. */
+int lr_residual_tanh(const float* x, const void* d, const void* expert_out, const float* expert_weights, int top,
+                     const void* alpha, const void* gain, const void* bias, float* x_out, void* x_compute, int rows, int dim,
+                     int dtype, lr_stream_t stream);
+
+/* Causal convolution per channel and silu over S consecutive tokens per sequence: out[t, c] =
+ * silu(bias[c] + sum_j w[c, j] u[t - (taps - 1) + j, c]).  u [B*S, C] (row stride ldu), w [C, taps] (the last column is the
+ * current token's), out [B*S, C] (row stride ldo; not u).  ring [Bmax, taps, C] holds a sequence's last inputs, a token's at
+ * position % taps: read for the portion's first tokens, filled for the next one's.  pos[0]: position of the first token;
+ * before position 0 the inputs are zero, whatever the ring holds.  C % 8 == 0, taps <= 8. */
+int lr_causal_conv(const void* u, int64_t ldu, const void* w, const void* bias, void* ring, const int32_t* pos, void* out,
+                   int64_t ldo, int B, int S, int C, int taps, int dtype, lr_stream_t stream);
+
+/* Selective state space with a scalar decay per head over S consecutive tokens per sequence, the state [B, H, N, P] (fp32)
+ * carried from call to call:
+ *     dt = softplus(dt_raw + dt_bias),   S_t = exp(-exp(a_log) dt) S_(t-1) + dt b_t x_t^T,   y_t = (S_t^T c_t + d x_t) * silu(z_t)
+ * x [B*S, H*P], b and c [B*S, G*N] (head h reads group h / (H / G)) are columns of a buffer with row stride ldu, z [B*S, H*P]
+ * and dt [B*S, H] columns of one with row stride ld; dt_bias, a_log, d [H]; y [B*S, H*P].  pos[0] as in lr_linear_attention:
+ * 0 starts from a zero state.  N, P multiples of 8, at most 256 (bf16: on the matrix cores when multiples of 16). */
+typedef struct lr_ssd {
+  const void *z, *x, *b, *c, *dt;
+  int64_t ld, ldu;
+  const void *dt_bias, *a_log, *d;
+  const int32_t* pos;
+  float* state;
+  void* y;
+  int64_t ldy;
+  int32_t* err; /* may be NULL */
+  void* scratch;
+  size_t scratch_bytes;
+  int32_t B, S, H, G, N, P, dtype;
+} lr_ssd_t;
+size_t lr_ssd_scratch_bytes(int B, int S, int H, int N, int P, int dtype);
+int lr_ssd(const lr_ssd_t* desc, lr_stream_t stream);
+/* One token per sequence, lr_causal_conv included: desc.x points at the convolution's input [B, C] with C = H P + 2 G N
+ * columns x | b | c (desc.b and desc.c are its later columns, desc.S == 1), ring as in lr_causal_conv. */
+int lr_ssd_step(const lr_ssd_t* desc, const void* conv_w, const void* conv_b, void* ring, int taps, lr_stream_t stream);
+
+/* In place: each of `parts` equal ranges of a row's `cols` columns divided by its root mean square (eps inside the root),
+ * times gain.  Column c lies at (c / P) * PP + c % P: heads of P columns padded to PP (gain is laid out the same way). */
+int lr_parts_norm(void* y, int64_t ld, const void* gain, int rows, int cols, int parts, int P, int PP, float eps, int dtype,
+                  lr_stream_t stream);
+
+/* What follows a projection [q | k | v] of B * S rows (H heads of dk; G of dk; G of dv; row b * S + s at position pos[s]):
+ * bias added (may be NULL), the pairs (i, i + rot / 2) of the first `rot` dimensions of q and k turned by the angles whose
+ * (cos, sin) is rope[position][i] (fp32 [rope_len, rot / 2, 2]), q left in place, k and v stored in
+ * cache[b, pos[s]] = [k of every head | v of every head], [Bmax, Smax, ldc].  cache NULL: the projection is q alone.
+ * A position outside the cache or the table sets *err = LR_DEV_POS_RANGE and leaves that row alone. */
+int lr_bias_rope_cache(void* proj, int64_t ld, const void* bias, const float* rope, const int32_t* pos, void* cache, int B, int S,
+                       int H, int G, int dk, int dv, int rot, int rope_len, int ldc, int Smax, int dtype, int32_t* err,
+                       lr_stream_t stream);
+
+/* lr_window_attention for one bf16 query per sequence over such a cache, the window cut into ranges that run side by side.
+ * dk, dv multiples of 8, at most 256. */
+size_t lr_window_decode_scratch_bytes(int B, int H, int G, int dv, int window, int Smax);
+int lr_window_decode(const void* q, int64_t ldq, const void* cache, const int32_t* pos, void* y, int64_t ldy, int B, int H, int G,
+                     int dk, int dv, int ldc, int Smax, int window, float scale, void* scratch, size_t scratch_bytes,
+                     lr_stream_t stream);
+
+/* Mixture of experts: router logits router[e, :] . x + router_bias[e] in fp32; experts[row, :] = the `top` largest (the lower
+ * index among equals), weights[row, :] = softmax over those; out[row * top + k, :] = w2[e] (silu(gate) * up) with
+ * [up; gate] = w1[e] x, e = experts[row, k].  x [rows, D] (row stride ldx), router [E (+ 1), D], w1 [E, 2 I, D],
+ * w2 [E, D, I], out [rows * top, D].  shared != NULL: router has one more row, without a bias, and shared [rows, shared_cols]
+ * (row stride ld_shared) is multiplied by the sigmoid of its product with x.  counts: [E] int32, zero before the first call
+ * and left zero.  E <= 512, top <= 64. */
+typedef struct lr_moe {
+  const void* x;
+  int64_t ldx;
+  const void *router, *router_bias, *w1, *w2;
+  void* out;
+  int32_t* experts;
+  float* weights;
+  int32_t* counts;
+  void* shared;
+  int64_t ld_shared;
+  void* scratch;
+  size_t scratch_bytes;
+  int32_t rows, D, I, E, top, shared_cols, dtype;
+} lr_moe_t;
+size_t lr_moe_scratch_bytes(int rows, int E, int top, int I, int shared, int dtype);
+int lr_moe(const lr_moe_t* desc, lr_stream_t stream);
 
 #ifdef __cplusplus
 }

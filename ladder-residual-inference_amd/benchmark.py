@@ -27,7 +27,7 @@ import torch
 
 sys.path.insert(0, str(Path(__file__).parent.resolve()))
 
-from gpt_fast import GPTDense, GPTDesync, GPTLadder, GPTLasivik, GPTParallel, _hip, set_virtual_tp  # noqa: E402
+from gpt_fast import GPTDense, GPTDesync, GPTGepolix, GPTLadder, GPTLasivik, GPTParallel, _hip, set_virtual_tp  # noqa: E402
 from gpt_fast.utils import _get_model_size, set_flash_attention  # noqa: E402
 
 default_device = "cuda" if torch.cuda.is_available() else "cpu"
@@ -38,6 +38,7 @@ _MODELS = {
     "gpt_parallel": GPTParallel,
     "gpt_ladder": GPTLadder,
     "gpt_lasivik": GPTLasivik,
+    "gpt_gepolix": GPTGepolix,
 }
 
 HBM_PEAK_GBPS = 8000.0  # MI355X HBM3E, vendor figure
@@ -452,7 +453,7 @@ def build_parser():
     p.add_argument("--checkpoint", type=Path, default=None,
                    help="folder with config.json and weights; the model is chosen by config.json")
     p.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16",
-                   help="float32: families that run in true 32-bit (gpt_lasivik)")
+                   help="float32: families that run in true 32-bit (gpt_lasivik, gpt_gepolix)")
     p.add_argument("--prompt_length", type=int, required=True, help="Input prompt length")
     p.add_argument("--num_samples", type=int, default=5, help="Number of samples.")
     p.add_argument("--max_new_tokens", type=int, default=200, help="Maximum number of new tokens.")

@@ -28,6 +28,8 @@ INCLUDES = {"ladder_step_fp8.hip": [os.path.join(CSRC, "ladder_step.hip")]}
 FAMILY_SOURCES = {
     "lasivik": ("attention.hip", "elementwise.hip", "gemm.hip", "gemv.hip", "latent_attention.hip", "linear_attention.hip",
                 "residual.hip", "sample.hip", "stream_gemm.hip"),
+    "gepolix": ("attention.hip", "elementwise.hip", "gemm.hip", "gemv.hip", "grouped_attention.hip", "latent_attention.hip", "moe.hip",
+                "residual.hip", "sample.hip", "ssd.hip", "stream_gemm.hip"),
 }
 
 FLAGS = [

@@ -263,8 +263,8 @@ struct WindowKeys {
   float scale;
 };
 
-// WIN (lr_window_attention): a sliding window, the score scale as an argument, and keys and values of one head per query
-// head as rows of a matrix, in the order lr_latent_window gives them; head sizes up to HD.
+// WIN (lr_window_attention): a sliding window, the score scale as an argument, and the kv heads' keys and values side by
+// side as rows of a matrix, in the order lr_latent_window gives them; head sizes up to HD.
 template <int HD, int NWH, bool WIN = false>
 __global__ __launch_bounds__(256) void k_attn_prefill_mfma(const u16* __restrict__ q, int64_t ldq,
                                                            const u16* __restrict__ kc, const u16* __restrict__ vc,
@@ -558,17 +558,22 @@ int window_attention_mfma(const lr_window_attention_t* d, lr_stream_t stream) {
   if (d->dtype != LR_BF16 || hd > 128 || d->dk % 8 || d->dv % 8 || d->ldq % 8 || d->ldk % 8 || d->ldy % 8 ||
       lr_misaligned(d->q) || lr_misaligned(d->k) || lr_misaligned(d->v) || lr_misaligned(d->y) || !(d->scale > 0.0f))
     return LR_E_UNSUPPORTED;
-  if ((int64_t)(d->n_keys + 64) * d->ldk * 2 >= 0x7fffffff || (int64_t)((d->S + 127) / 128) * d->H * d->B >= (1 << 24))
+  if ((int64_t)(d->n_keys + 64) * d->ldk * 2 >= 0x7fffffff || (int64_t)((d->S + 31) / 32) * d->H * d->B >= (1 << 24))
     return LR_E_UNSUPPORTED;
   const WindowKeys w = {d->window, d->n_keys, (int)d->ldk, d->dk, d->dv, d->scale};
-  const dim3 grid((unsigned)((int64_t)((d->S + 127) / 128) * d->H * d->B));
+  const int G = d->kv_heads > 0 ? d->kv_heads : d->H, share = d->H / G;
   hipStream_t s = (hipStream_t)stream;
-#define LR_WIN(HD)                                                                                                     \
-  k_attn_prefill_mfma<HD, 1, true><<<grid, dim3(256), 0, s>>>((const u16*)d->q, d->ldq, (const u16*)d->k,             \
-                                                              (const u16*)d->v, d->pos, (u16*)d->y, d->ldy, d->S, d->H, \
-                                                              d->H, d->Smax, w)
-  if (hd <= 64) LR_WIN(64);
-  else LR_WIN(128);
+#define LR_WIN(HD, NWH)                                                                                                \
+  k_attn_prefill_mfma<HD, NWH, true>                                                                                   \
+      <<<dim3((unsigned)((int64_t)((d->S + 32 * (4 / NWH) - 1) / (32 * (4 / NWH))) * (d->H / NWH) * d->B)), dim3(256), 0, s>>>( \
+          (const u16*)d->q, d->ldq, (const u16*)d->k, (const u16*)d->v, d->pos, (u16*)d->y, d->ldy, d->S, d->H, G, d->Smax, w)
+#define LR_WIN_HD(HD)                    \
+  if (share % 4 == 0) LR_WIN(HD, 4);     \
+  else if (share % 2 == 0) LR_WIN(HD, 2); \
+  else LR_WIN(HD, 1)
+  if (hd <= 64) { LR_WIN_HD(64); }
+  else { LR_WIN_HD(128); }
+#undef LR_WIN_HD
 #undef LR_WIN
   return lr_launch_status();
 }

@@ -265,7 +265,8 @@ extern "C" int lr_ladder_norms(const void* resid_in, const void* d1, const void*
 }
 
 // ------------------------------------------------------------------------------------ SwiGLU
-__global__ __launch_bounds__(256) void k_swiglu(const u16* __restrict__ h, int64_t ldh, u16* __restrict__ out, int I) {
+__global__ __launch_bounds__(256) void k_swiglu(const u16* __restrict__ h, int64_t ldh, u16* __restrict__ out, int64_t ldo,
+                                                int I) {
   const int row = blockIdx.y;
   const int c = (blockIdx.x * 256 + threadIdx.x) * 8;
   if (c >= I) return;
@@ -274,22 +275,28 @@ __global__ __launch_bounds__(256) void k_swiglu(const u16* __restrict__ h, int64
   unpack8(ld16(h + row * ldh + I + c), g);
 #pragma unroll
   for (int j = 0; j < 8; ++j) o[j] = swiglu_bf(u[j], g[j]);
-  st16(out + (int64_t)row * I + c, pack8(o));
+  st16(out + (int64_t)row * ldo + c, pack8(o));
 }
 
-extern "C" int lr_swiglu(const void* h, int64_t ldh, void* out, int rows, int I, lr_stream_t stream) {
+namespace lr_detail {
+int swiglu_rows(const void* h, int64_t ldh, void* out, int64_t ldo, int rows, int I, lr_stream_t stream) {
   LR_REQUIRE_PTR(h);
   LR_REQUIRE_PTR(out);
-  if (rows <= 0 || I <= 0 || ldh < 2 * (int64_t)I || rows > 65535 * 64) return LR_E_SHAPE;
-  if (I % 8 || ldh % 8) return LR_E_ALIGN;
+  if (rows <= 0 || I <= 0 || ldh < 2 * (int64_t)I || ldo < I || rows > 65535 * 64) return LR_E_SHAPE;
+  if (I % 8 || ldh % 8 || ldo % 8) return LR_E_ALIGN;
   // rows ride on grid.y, which is limited to 65535: fold larger row counts into several launches
   const int per = 65535;
   for (int r0 = 0; r0 < rows; r0 += per) {
     const int nr = rows - r0 < per ? rows - r0 : per;
     k_swiglu<<<dim3((I / 8 + 255) / 256, nr), dim3(256), 0, (hipStream_t)stream>>>(
-        (const u16*)h + (int64_t)r0 * ldh, ldh, (u16*)out + (int64_t)r0 * I, I);
+        (const u16*)h + (int64_t)r0 * ldh, ldh, (u16*)out + (int64_t)r0 * ldo, ldo, I);
   }
   return lr_launch_status();
+}
+}  // namespace lr_detail
+
+extern "C" int lr_swiglu(const void* h, int64_t ldh, void* out, int rows, int I, lr_stream_t stream) {
+  return lr_detail::swiglu_rows(h, ldh, out, I, rows, I, stream);
 }
 
 // ------------------------------------------------------------------------------------ RoPE + KV write

@@ -13,6 +13,10 @@
 int lr_gemv_dispatch(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy, int M, int N, int K,
                      int act_swiglu, int gemv_cfg, hipStream_t s);
 
+namespace lr_detail {
+int swiglu_rows(const void* h, int64_t ldh, void* out, int64_t ldo, int rows, int I, lr_stream_t stream);   // elementwise.hip
+}
+
 constexpr int BM = 128, BN = 128, BK = 64, LDT = BK + 8;  // LDT: padded LDS row length in elements
 
 template <bool SWIGLU>
@@ -148,12 +152,22 @@ constexpr int GM = 256, GN = 256;
 struct GemmRope {
   int S, Hq, Hkv, hd, Smax, block_size;
 };
-template <bool KTAIL, bool ROPE>
+// GROUP: the rows of a tile are entries of a list, tile (matrix, first entry, entries) as a device table says: input row
+// entry / xdiv, output row entry, weights of one of several matrices that lie `wstride` elements apart.
+struct GemmGroup {
+  const int32_t* tiles;    // [][3]
+  const int32_t* ntiles;
+  const int32_t* entries;
+  int xdiv;
+  int64_t wstride;
+};
+template <bool KTAIL, bool ROPE, bool GROUP = false>
 __global__ __launch_bounds__(256) void k_gemm_big(const u16* __restrict__ x, int64_t ldx, const u16* __restrict__ w,
                                                   u16* __restrict__ y, int64_t ldy, int M, int N, int K, int tm,
                                                   int tn, int pair_off, const u16* __restrict__ rtable,
                                                   const int32_t* __restrict__ rpos, u16* __restrict__ rk,
-                                                  u16* __restrict__ rv, int32_t* rerr, const GemmRope rp) {
+                                                  u16* __restrict__ rv, int32_t* rerr, const GemmRope rp,
+                                                  const GemmGroup gp = {}) {
   extern __shared__ __attribute__((aligned(16))) u16 gsm[];
   u16* xs = gsm;                      // [2][GM * LDT]
   u16* ws = gsm + 2 * GM * LDT;       // [2][GN * LDT]
@@ -161,7 +175,20 @@ __global__ __launch_bounds__(256) void k_gemm_big(const u16* __restrict__ x, int
   const int wm = wave >> 1, wn = wave & 1;
   // ---- tile of this workgroup
   int mt, nt;
-  {
+  int32_t* const entry = reinterpret_cast<int32_t*>(gsm + 2 * (GM + GN) * LDT);   // (GROUP) the tile's entries
+  if constexpr (GROUP) {   // an XCD takes a contiguous run of tiles, a row tile's column tiles one after the other
+    const int n = gridDim.x, xcd = blockIdx.x & 7, base = n >> 3, rem = n & 7;
+    const int id = xcd * base + (xcd < rem ? xcd : rem) + (blockIdx.x >> 3);
+    mt = id / tn;
+    nt = id - mt * tn;
+    if (mt >= gp.ntiles[0]) return;
+    const int32_t* tile = gp.tiles + 3 * mt;
+    w += tile[0] * gp.wstride;
+    M = tile[2];
+    entry[tid] = gp.entries[tile[1] + (tid < M ? tid : 0)];
+    mt = 0;
+    __syncthreads();
+  } else {
     const int id = blockIdx.x;
     if (tm % 32 == 0) {  // XCD-aware: XCD x owns a band of tm / 8 row tiles, walked 4 row tiles x all column tiles at a time
       const int xcd = id & 7, j = id >> 3;
@@ -197,7 +224,8 @@ __global__ __launch_bounds__(256) void k_gemm_big(const u16* __restrict__ x, int
 #pragma unroll
   for (int i = 0; i < 8; ++i) {
     const int r = srow0 + i * 32;
-    xoff[i] = m0 + r < M ? (int)((int64_t)r * ldx * 2) : (int)0x80000000;
+    const int xrow = GROUP ? entry[r] / gp.xdiv : r;
+    xoff[i] = m0 + r < M ? (int)((int64_t)xrow * ldx * 2) : (int)0x80000000;
     if (pair_off) {
       const int wv = i >> 2, b = i & 3;                      // r = wv * 128 + b * 32 + srow0
       const int pr = wv * 64 + (b & 1) * 32 + srow0;          // pair inside the tile
@@ -364,6 +392,7 @@ __global__ __launch_bounds__(256) void k_gemm_big(const u16* __restrict__ x, int
     }
     auto store_row = [&](int m, const uint4& v) {
       if (m < M) {
+        if constexpr (GROUP) m = entry[m];
         if (vec_ok && ncol0 + 7 < N) {
           *reinterpret_cast<uint4*>(y + (int64_t)m * ldy + ncol0) = v;
         } else {
@@ -452,6 +481,30 @@ static int launch_gemm_big(const void* x, int64_t ldx, const void* w, void* y, i
                : launch_gemm_big_as<false, false>(x, ldx, w, y, ldy, M, N, K, pair_off, nullptr, 0, s);
 }
 
+// Grouped products (lr_moe): rows of several matrices' tiles, see GemmGroup.  pair_off as in launch_gemm_big.
+namespace lr_detail {
+template <bool KTAIL>
+static int gemm_grouped_as(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy, int N, int K, int pair_off,
+                           const GemmGroup& gp, int max_tiles, hipStream_t s) {
+  constexpr size_t lds = (size_t)2 * (GM + GN) * LDT * sizeof(u16) + GM * sizeof(int32_t);
+  static std::atomic<unsigned long long> lds_raised{0};
+  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_gemm_big<KTAIL, false, true>), lds, lds_raised)) return LR_E_LAUNCH;
+  const int gn = pair_off ? GN / 2 : GN, tn = (N + gn - 1) / gn;
+  k_gemm_big<KTAIL, false, true><<<dim3((unsigned)(max_tiles * tn)), dim3(256), lds, s>>>(
+      (const u16*)x, ldx, (const u16*)w, (u16*)y, ldy, GM, N, K, max_tiles, tn, pair_off, nullptr, nullptr, nullptr, nullptr, nullptr,
+      GemmRope{}, gp);
+  return lr_launch_status();
+}
+int gemm_grouped(const void* x, int64_t ldx, int64_t xrows, const void* w, void* y, int64_t ldy, int N, int K, int pair_off, int64_t wstride,
+                 const int32_t* tiles, const int32_t* ntiles, const int32_t* entries, int xdiv, int max_tiles, hipStream_t s) {
+  if (xrows * ldx * 2 >= 0x7fffffff || ((int64_t)pair_off + GN) * K * 2 >= 0x7fffffff) return LR_E_UNSUPPORTED;
+  const GemmGroup gp = {tiles, ntiles, entries, xdiv, wstride};
+  return K % BK ? gemm_grouped_as<true>(x, ldx, w, y, ldy, N, K, pair_off, gp, max_tiles, s)
+                : gemm_grouped_as<false>(x, ldx, w, y, ldy, N, K, pair_off, gp, max_tiles, s);
+}
+int gemm_grouped_rows() { return GM; }
+}  // namespace lr_detail
+
 extern "C" int lr_linear_tuned(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy, int M, int N, int K,
                                int act_swiglu, int gemv_cfg, lr_stream_t stream) {
   LR_REQUIRE_PTR(x);
@@ -537,8 +590,7 @@ extern "C" int lr_linear_swiglu_out(const void* x, int64_t ldx, const void* w, v
   // other sizes: the projection into `scratch` [M, N], then the activation
   LR_REQUIRE_PTR(scratch);
   if (scratch_bytes < (size_t)M * N * sizeof(u16)) return LR_E_SHAPE;
-  if (ldy != I) return LR_E_UNSUPPORTED;  // lr_swiglu writes dense rows
   const int rc = lr_linear(x, ldx, w, scratch, N, M, N, K, 0, stream);
   if (rc != LR_OK) return rc;
-  return lr_swiglu(scratch, N, y, M, I, stream);
+  return lr_detail::swiglu_rows(scratch, N, y, ldy, M, I, stream);
 }

@@ -98,7 +98,7 @@ struct WinAttn {
   void* y;
   int64_t ldy, hy;
   const int32_t* pos;
-  int S, H, dk, dv, window, n_keys, windowed_rows, Smax;
+  int S, H, share, dk, dv, window, n_keys, windowed_rows, Smax;   // share: query heads per k / v head
   float scale;
 };
 
@@ -115,8 +115,8 @@ __global__ __launch_bounds__(64) void k_window_attention(const WinAttn a) {
   const TQ* q = reinterpret_cast<const TQ*>(a.q) + row * a.ldq + h * a.hq;
   for (int d = lane; d < a.dk; d += 64) qs[d] = ldf(q + d);
   __syncthreads();
-  const TK* kb = reinterpret_cast<const TK*>(a.k) + b * a.kb + h * a.kh;
-  const TK* vb = reinterpret_cast<const TK*>(a.v) + b * a.vb + h * a.vh;
+  const TK* kb = reinterpret_cast<const TK*>(a.k) + b * a.kb + h / a.share * a.kh;
+  const TK* vb = reinterpret_cast<const TK*>(a.v) + b * a.vb + h / a.share * a.vh;
   constexpr int DV = 16;
   float acc[DV];
 #pragma unroll
@@ -651,7 +651,7 @@ int latent_attention(const lr_latent_attention_t* d, hipStream_t s) {
     a.k = a.v = d->cache;
     a.kb = a.vb = (int64_t)d->Smax * d->ldr; a.kr = a.vr = d->ldr; a.kh = a.vh = 0;
     a.y = ol; a.ldy = a.ldq; a.hy = d->ldr; a.pos = d->pos;
-    a.S = d->S; a.H = d->H; a.dk = a.dv = d->ldr; a.window = d->window; a.n_keys = d->Smax; a.Smax = d->Smax;
+    a.S = d->S; a.H = d->H; a.share = 1; a.dk = a.dv = d->ldr; a.window = d->window; a.n_keys = d->Smax; a.Smax = d->Smax;
     a.scale = d->scale;
     rc = launch_window<float, T, float>(a, d->B, s);
   }
@@ -701,10 +701,12 @@ extern "C" int lr_window_attention(const lr_window_attention_t* d, lr_stream_t s
   if (d == nullptr || d->q == nullptr || d->k == nullptr || d->v == nullptr || d->y == nullptr || d->pos == nullptr)
     return LR_E_NULL;
   if (d->B <= 0 || d->S <= 0 || d->H <= 0 || d->dk <= 0 || d->dv <= 0 || d->window <= 0 || d->n_keys <= 0 ||
-      d->n_keys > d->Smax)
+      d->n_keys > d->Smax || d->kv_heads < 0)
     return LR_E_SHAPE;
-  if (d->ldq < (int64_t)d->H * d->dk || d->ldy < (int64_t)d->H * d->dv || d->ldk < (int64_t)d->H * d->dk ||
-      d->ldk < (int64_t)d->H * d->dv)
+  const int G = d->kv_heads > 0 ? d->kv_heads : d->H;
+  if (d->H % G) return LR_E_SHAPE;
+  if (d->ldq < (int64_t)d->H * d->dk || d->ldy < (int64_t)d->H * d->dv || d->ldk < (int64_t)G * d->dk ||
+      d->ldk < (int64_t)G * d->dv)
     return LR_E_SHAPE;
   if (d->B > 65535) return LR_E_UNSUPPORTED;
   {
@@ -718,7 +720,7 @@ extern "C" int lr_window_attention(const lr_window_attention_t* d, lr_stream_t s
   a.k = d->k; a.kb = (int64_t)d->n_keys * d->ldk; a.kr = d->ldk; a.kh = d->dk;
   a.v = d->v; a.vb = a.kb; a.vr = d->ldk; a.vh = d->dv;
   a.y = d->y; a.ldy = d->ldy; a.hy = d->dv; a.pos = d->pos;
-  a.S = d->S; a.H = d->H; a.dk = d->dk; a.dv = d->dv; a.window = d->window; a.n_keys = d->n_keys; a.windowed_rows = 1;
+  a.S = d->S; a.H = d->H; a.share = d->H / G; a.dk = d->dk; a.dv = d->dv; a.window = d->window; a.n_keys = d->n_keys; a.windowed_rows = 1;
   a.Smax = d->Smax; a.scale = d->scale;
   hipStream_t s = (hipStream_t)stream;
   if (d->dtype == LR_BF16) return launch_window<u16, u16, u16>(a, d->B, s);

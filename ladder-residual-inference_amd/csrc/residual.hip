@@ -75,6 +75,57 @@ __global__ __launch_bounds__(256) void k_residual_norm(const float* x, float alp
   }
 }
 
+// r = x + d + sum over a token's slots of weight * out (the experts of a mixture);  x_out = r and
+// x_compute = tanh(alpha r) gain + bias: a norm without statistics, so a row is cut into as many workgroups as it fills.
+template <typename T>
+__global__ __launch_bounds__(256) void k_residual_tanh(const float* x, const T* __restrict__ d, const T* __restrict__ eo,
+                                                       const float* __restrict__ ew, int top, const T* __restrict__ alpha,
+                                                       const T* __restrict__ gain, const T* __restrict__ bias, float* xo,
+                                                       T* __restrict__ xc, int dim) {
+  const int64_t row = blockIdx.x;
+  const int c = (blockIdx.y * 256 + threadIdx.x) * 4;
+  if (c >= dim) return;
+  const int64_t at = row * dim + c;
+  const float4 q = *reinterpret_cast<const float4*>(x + at);
+  float r[4] = {q.x, q.y, q.z, q.w};
+  if (d) {
+    Quad<T> t;
+    t.load(d + at);
+    float f[4];
+    t.get(f);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) r[j] += f[j];
+  }
+  if (eo) {
+    float s[4] = {0, 0, 0, 0};
+#pragma unroll 4
+    for (int k = 0; k < top; ++k) {
+      const float w = ew[row * top + k];
+      Quad<T> t;
+      t.load(eo + (row * top + k) * dim + c);
+      float f[4];
+      t.get(f);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) s[j] = fmaf(w, f[j], s[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) r[j] += s[j];
+  }
+  if (xo) st4(xo + at, r);
+  if (xc) {
+    Quad<T> tg, tb;
+    tg.load(gain + c);
+    tb.load(bias + c);
+    float g[4], b[4];
+    tg.get(g);
+    tb.get(b);
+    const float al = ldf(alpha);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) r[j] = fmaf(tanhf(al * r[j]), g[j], b[j]);
+    st4(xc + at, r);
+  }
+}
+
 // logits <- cap tanh(scale logits / cap), in place (cap <= 0: the scale alone)
 template <typename T>
 __global__ __launch_bounds__(256) void k_logit_cap(T* l, int64_t ld, int V, float scale, float cap) {
@@ -85,25 +136,40 @@ __global__ __launch_bounds__(256) void k_logit_cap(T* l, int64_t ld, int V, floa
   }
 }
 
-// y = x w^T in fp32: 64 x 64 tiles, four waves of 32 x 32, v_mfma_f32_16x16x4_f32; any M, N, K.
+// y = x w^T in fp32: 64 x 64 tiles, four waves of 32 x 32, v_mfma_f32_16x16x4_f32; any M, N, K.  GROUP: the rows of a tile
+// are entries of a list, tile (matrix, first entry, entries) as a device table says: input row entry / xdiv, output row
+// entry, weights of one of several matrices.
 constexpr int FT = 64, FK = 16, FL = FK + 4;
+template <bool GROUP>
 __global__ __launch_bounds__(256) void k_linear_f32(const float* __restrict__ x, int64_t ldx, const float* __restrict__ w,
-                                                    float* __restrict__ y, int64_t ldy, int M, int N, int K) {
+                                                    float* __restrict__ y, int64_t ldy, int M, int N, int K,
+                                                    const int32_t* __restrict__ tiles, const int32_t* __restrict__ ntiles,
+                                                    const int32_t* __restrict__ entries, int xdiv) {
   __shared__ __attribute__((aligned(16))) float xs[FT * FL], ws[FT * FL];
+  __shared__ int32_t rows[FT];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g4 = lane >> 4, l16 = lane & 15;
-  const int m0 = blockIdx.y * FT, n0 = blockIdx.x * FT, wm = (wave >> 1) * 32, wn = (wave & 1) * 32;
+  if constexpr (GROUP) {
+    if ((int)blockIdx.y >= ntiles[0]) return;
+    const int32_t* tile = tiles + 3 * blockIdx.y;
+    w += (int64_t)tile[0] * N * K;
+    M = tile[2];
+    if (tid < FT) rows[tid] = entries[tile[1] + (tid < M ? tid : 0)];
+    __syncthreads();
+  }
+  const int m0 = GROUP ? 0 : blockIdx.y * FT, n0 = blockIdx.x * FT, wm = (wave >> 1) * 32, wn = (wave & 1) * 32;
   f32x4_t acc[2][2];
 #pragma unroll
   for (int i = 0; i < 2; ++i)
 #pragma unroll
     for (int j = 0; j < 2; ++j) acc[i][j] = f32x4_t{0, 0, 0, 0};
   const int r = tid >> 2, c4 = (tid & 3) * 4;
+  const int64_t xrow = GROUP ? rows[r] / xdiv : m0 + r;
   for (int k0 = 0; k0 < K; k0 += FK) {
     float fx[4], fw[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int kk = k0 + c4 + j;
-      fx[j] = (m0 + r < M && kk < K) ? x[(int64_t)(m0 + r) * ldx + kk] : 0.0f;
+      fx[j] = (m0 + r < M && kk < K) ? x[xrow * ldx + kk] : 0.0f;
       fw[j] = (n0 + r < N && kk < K) ? w[(int64_t)(n0 + r) * K + kk] : 0.0f;
     }
     __syncthreads();
@@ -133,14 +199,14 @@ __global__ __launch_bounds__(256) void k_linear_f32(const float* __restrict__ x,
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int m = m0 + wm + 16 * i + 4 * g4 + e, n = n0 + wn + 16 * j + l16;
-        if (m < M && n < N) y[(int64_t)m * ldy + n] = acc[i][j][e];
+        if (m < M && n < N) y[(int64_t)(GROUP ? rows[m] : m) * ldy + n] = acc[i][j][e];
       }
 }
 
 __global__ __launch_bounds__(256) void k_swiglu_f32(const float* __restrict__ h, int64_t ldh, float* __restrict__ out,
-                                                    int I) {
+                                                    int64_t ldo, int I) {
   const float* row = h + (int64_t)blockIdx.x * ldh;
-  for (int c = threadIdx.x; c < I; c += 256) out[(int64_t)blockIdx.x * I + c] = silu_f(row[I + c]) * row[c];
+  for (int c = threadIdx.x; c < I; c += 256) out[(int64_t)blockIdx.x * ldo + c] = silu_f(row[I + c]) * row[c];
 }
 
 template <typename T>
@@ -200,6 +266,38 @@ extern "C" int lr_residual_rmsnorm(const float* x, float alpha, const void* d, c
   return lr_launch_status();
 }
 
+extern "C" int lr_residual_tanh(const float* x, const void* d, const void* expert_out, const float* expert_weights, int top,
+                                const void* alpha, const void* gain, const void* bias, float* x_out, void* x_compute, int rows,
+                                int dim, int dtype, lr_stream_t stream) {
+  LR_REQUIRE_PTR(x);
+  LR_OPTIONAL_PTR(d);
+  LR_OPTIONAL_PTR(expert_out);
+  LR_OPTIONAL_PTR(x_out);
+  LR_OPTIONAL_PTR(x_compute);
+  if (x_out == nullptr && x_compute == nullptr) return LR_E_NULL;
+  if (x_compute) {
+    LR_REQUIRE_PTR(gain);
+    LR_REQUIRE_PTR(bias);
+    if (alpha == nullptr) return LR_E_NULL;
+  }
+  if (expert_out && expert_weights == nullptr) return LR_E_NULL;
+  if (rows <= 0 || dim <= 0 || (expert_out && top <= 0)) return LR_E_SHAPE;
+  if (dim % 8) return LR_E_ALIGN;
+  if (dim > 1024 * 65535) return LR_E_UNSUPPORTED;
+  const dim3 grid(rows, (dim + 1023) / 1024), blk(256);
+  if (dtype == LR_BF16)
+    k_residual_tanh<u16><<<grid, blk, 0, (hipStream_t)stream>>>(x, (const u16*)d, (const u16*)expert_out, expert_weights, top,
+                                                               (const u16*)alpha, (const u16*)gain, (const u16*)bias, x_out,
+                                                               (u16*)x_compute, dim);
+  else if (dtype == LR_F32)
+    k_residual_tanh<float><<<grid, blk, 0, (hipStream_t)stream>>>(x, (const float*)d, (const float*)expert_out, expert_weights, top,
+                                                                 (const float*)alpha, (const float*)gain, (const float*)bias, x_out,
+                                                                 (float*)x_compute, dim);
+  else
+    return LR_E_UNSUPPORTED;
+  return lr_launch_status();
+}
+
 extern "C" int lr_logit_cap(void* logits, int64_t ldl, int rows, int V, float scale, float cap, int dtype,
                             lr_stream_t stream) {
   LR_REQUIRE_PTR(logits);
@@ -223,14 +321,24 @@ extern "C" int lr_linear_f32(const float* x, int64_t ldx, const float* w, float*
   if (M <= 0 || N <= 0 || K <= 0 || ldx < K || ldy < N) return LR_E_SHAPE;
   const dim3 grid((N + FT - 1) / FT, (M + FT - 1) / FT);
   if (grid.y > 65535) return LR_E_UNSUPPORTED;
-  k_linear_f32<<<grid, dim3(256), 0, (hipStream_t)stream>>>(x, ldx, w, y, ldy, M, N, K);
+  k_linear_f32<false><<<grid, dim3(256), 0, (hipStream_t)stream>>>(x, ldx, w, y, ldy, M, N, K, nullptr, nullptr, nullptr, 1);
   return lr_launch_status();
 }
 
-extern "C" int lr_swiglu_f32(const float* h, int64_t ldh, float* out, int rows, int I, lr_stream_t stream) {
+namespace lr_detail {
+int linear_f32_grouped(const float* x, int64_t ldx, const float* w, float* y, int64_t ldy, int N, int K, const int32_t* tiles,
+                       const int32_t* ntiles, const int32_t* entries, int xdiv, int max_tiles, hipStream_t s) {
+  if (max_tiles > 65535) return LR_E_UNSUPPORTED;
+  k_linear_f32<true><<<dim3((N + FT - 1) / FT, max_tiles), dim3(256), 0, s>>>(x, ldx, w, y, ldy, FT, N, K, tiles, ntiles, entries, xdiv);
+  return lr_launch_status();
+}
+int linear_f32_grouped_rows() { return FT; }
+}  // namespace lr_detail
+
+extern "C" int lr_swiglu_f32(const float* h, int64_t ldh, float* out, int64_t ldo, int rows, int I, lr_stream_t stream) {
   LR_REQUIRE_PTR(h);
   LR_REQUIRE_PTR(out);
-  if (rows <= 0 || I <= 0 || ldh < 2 * (int64_t)I) return LR_E_SHAPE;
-  k_swiglu_f32<<<dim3(rows), dim3(256), 0, (hipStream_t)stream>>>(h, ldh, out, I);
+  if (rows <= 0 || I <= 0 || ldh < 2 * (int64_t)I || ldo < I) return LR_E_SHAPE;
+  k_swiglu_f32<<<dim3(rows), dim3(256), 0, (hipStream_t)stream>>>(h, ldh, out, ldo, I);
   return lr_launch_status();
 }

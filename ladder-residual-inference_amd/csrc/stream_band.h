@@ -68,8 +68,10 @@ constexpr size_t stream_band_lds_bytes() {
 // 256 bytes, now 256 elements of K, which are expanded to bf16 (exactly: e4m3 is a subset of bf16) on their way
 // into the LDS piece; the sum is rounded to bf16, multiplied by the row's scale and rounded again, as
 // F.linear(x, w.to(bf16)) * scales does, before the epilogue sees it.
-template <int MT, int UNITS, bool W8 = false, bool XL = (MT >= XLDS_MIN_MT)>
-__device__ __forceinline__ void stream_band(const Proj& p, const int M, const int band, u16* sg_smem) {
+// GATHER: input row m is row rows[m] / xdiv of x, output row m is row rows[m] of y (`rows`: M of them, in LDS).
+template <int MT, int UNITS, bool W8 = false, bool XL = (MT >= XLDS_MIN_MT), bool GATHER = false>
+__device__ __forceinline__ void stream_band(const Proj& p, const int M, const int band, u16* sg_smem,
+                                            const int32_t* rows = nullptr, const int xdiv = 1) {
   static_assert(!W8 || MT == 16, "the e4m3 path is built for up to 16 input rows");
   constexpr int KCW = W8 ? 256 : 128;  // k elements per chunk
   constexpr int LRW = KCW + 8;         // LDS row length in elements
@@ -126,13 +128,15 @@ __device__ __forceinline__ void stream_band(const Proj& p, const int M, const in
 #pragma unroll
     for (int i = 0; i < MT / 4; ++i) {
       const int m = 4 * i + l4;
-      xoff[i] = m < M ? (int)((m * ldx + l16 * 8) * 2) : OOB;
+      const int xm = GATHER ? (m < M ? rows[m] / xdiv : 0) : m;
+      xoff[i] = m < M ? (int)((xm * ldx + l16 * 8) * 2) : OOB;
     }
   } else {
 #pragma unroll
     for (int mt = 0; mt < MTILES; ++mt) {
       const int m = mt * 16 + l16;
-      xoff[mt] = m < M ? (int)((m * ldx + l4 * 8) * 2) : OOB;
+      const int xm = GATHER ? (m < M ? rows[m] / xdiv : 0) : m;
+      xoff[mt] = m < M ? (int)((xm * ldx + l4 * 8) * 2) : OOB;
     }
   }
   u16* const my = sg_smem + wave * (WPIECE + XPIECE);
@@ -336,6 +340,7 @@ __device__ __forceinline__ void stream_band(const Proj& p, const int M, const in
     const int r = o % rows_out, m = o / rows_out;
     if (r >= nrows || m >= M) continue;
     const int mt = m >> 4, ln = ((r & 15) >> 2) * 16 + (m & 15), e = r & 3, u = r >> 4;
+    const int ym = GATHER ? rows[m] : m;
     float s0 = 0.0f, s1 = 0.0f;
 #pragma unroll
     for (int wv = 0; wv < NWV; ++wv) s0 += red[wv * WSTRIDE + ((u * MTILES + mt) * 4 + e) * 64 + ln];
@@ -349,11 +354,11 @@ __device__ __forceinline__ void stream_band(const Proj& p, const int M, const in
         u_ = round_bf(u_ * bf_to_f(p.scales[n0 + r]));
         g_ = round_bf(g_ * bf_to_f(p.scales[pair_off + n0 + r]));
       }
-      yg[(int64_t)m * ldy + n0 + r] = f_to_bf(swiglu_bf(u_, g_));
+      yg[(int64_t)ym * ldy + n0 + r] = f_to_bf(swiglu_bf(u_, g_));
     } else if constexpr (W8) {
-      yg[(int64_t)m * ldy + n0 + r] = f_to_bf(round_bf(s0) * bf_to_f(p.scales[n0 + r]));
+      yg[(int64_t)ym * ldy + n0 + r] = f_to_bf(round_bf(s0) * bf_to_f(p.scales[n0 + r]));
     } else {
-      yg[(int64_t)m * ldy + n0 + r] = f_to_bf(s0);
+      yg[(int64_t)ym * ldy + n0 + r] = f_to_bf(s0);
     }
   }
   LR_BAND_STAMP(5)

@@ -3,8 +3,9 @@
 from .gpt_dense_TP import GPTDense
 from .gpt_desync_TP import GPTDesync
 from .gpt_ladder_TP import GPTLadder
+from .gpt_gepolix import GPTGepolix
 from .gpt_lasivik import GPTLasivik
 from .gpt_parallel_TP import GPTParallel
 from .tp import maybe_init_dist, set_virtual_tp
 
-__all__ = ["GPTDense", "GPTDesync", "GPTLadder", "GPTLasivik", "GPTParallel", "maybe_init_dist", "set_virtual_tp"]
+__all__ = ["GPTDense", "GPTDesync", "GPTGepolix", "GPTLadder", "GPTLasivik", "GPTParallel", "maybe_init_dist", "set_virtual_tp"]

@@ -69,7 +69,7 @@ _PROTOS = {
                                     c_int, c_float, c_int, c_void_p]),
     "lr_logit_cap": (c_int, [c_void_p, c_int64, c_int, c_int, c_float, c_float, c_int, c_void_p]),
     "lr_linear_f32": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_void_p]),
-    "lr_swiglu_f32": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_int, c_void_p]),
+    "lr_swiglu_f32": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int, c_int, c_void_p]),
     "lr_argmax_f32": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_int, c_void_p]),
     "lr_linear_attention_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
     "lr_linear_attention": (c_int, [c_void_p, c_void_p]),
@@ -79,6 +79,21 @@ _PROTOS = {
     "lr_window_attention": (c_int, [c_void_p, c_void_p]),
     "lr_latent_attention_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
     "lr_latent_attention": (c_int, [c_void_p, c_void_p]),
+    "lr_residual_tanh": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                                 c_int, c_int, c_int, c_void_p]),
+    "lr_causal_conv": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
+                               c_int, c_int, c_void_p]),
+    "lr_ssd_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
+    "lr_ssd": (c_int, [c_void_p, c_void_p]),
+    "lr_ssd_step": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p]),
+    "lr_parts_norm": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p]),
+    "lr_bias_rope_cache": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                                   c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p]),
+    "lr_window_decode_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
+    "lr_window_decode": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_int, c_int, c_int,
+                                 c_int, c_int, c_float, c_void_p, c_size_t, c_void_p]),
+    "lr_moe_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
+    "lr_moe": (c_int, [c_void_p, c_void_p]),
 }
 
 
@@ -423,11 +438,12 @@ def module_linear_swiglu(h: torch.Tensor, mod, out: torch.Tensor, act: torch.Ten
 
 def swiglu(h: torch.Tensor, out: torch.Tensor):
     rows, two_i, ldh = _rows_ld(h)
-    assert out.is_contiguous() and out.numel() == rows * (two_i // 2)
+    assert out.numel() == rows * (two_i // 2)
     if h.dtype == torch.float32:
-        _check(load().lr_swiglu_f32(_dev(h, h.dtype), ldh, _dev(out, h.dtype), rows, two_i // 2, _stream()),
+        _check(load().lr_swiglu_f32(_dev(h, h.dtype), ldh, _dev(out, h.dtype), _rows_ld(out)[2], rows, two_i // 2, _stream()),
                "lr_swiglu_f32")
         return out
+    assert out.is_contiguous()
     _check(load().lr_swiglu(_dev(h), ldh, _dev(out), rows, two_i // 2, _stream()), "lr_swiglu")
     return out
 
@@ -712,22 +728,23 @@ def latent_window(cache, pos, rows, B, window: int):
 class _WindowAttention(ctypes.Structure):   # lr_window_attention_t
     _fields_ = [("q", c_void_p), ("ldq", c_int64), ("k", c_void_p), ("v", c_void_p), ("ldk", c_int64), ("y", c_void_p),
                 ("ldy", c_int64), ("pos", c_void_p)] + \
-               [(n, c_int32) for n in ("B", "S", "H", "dk", "dv", "window", "n_keys", "Smax", "dtype")] + \
+               [(n, c_int32) for n in ("B", "S", "H", "dk", "dv", "window", "n_keys", "Smax", "dtype", "kv_heads")] + \
                [("scale", c_float)]
 
 
-def window_attention(q, kv, y, pos, B, S, H, dk, dv, window: int, n_keys: int, Smax: int, scale: float):
-    """Sliding-window attention of S queries per sequence; kv [B * n_keys, >= H dk + H dv] = k | v of the rows
-    latent_window hands out."""
-    _, qc, ldq = _rows_ld(q)
+def window_attention(q, kv, y, pos, B, S, H, dk, dv, window: int, n_keys: int, Smax: int, scale: float, kv_heads: int = None):
+    """Sliding-window attention of S queries per sequence; kv [B * n_keys, >= G (dk + dv)] = k | v of G heads (kv_heads; None:
+    H), rows as latent_window hands them out, or a cache's own (n_keys == Smax)."""
+    G = H if kv_heads is None else kv_heads
+    rows, qc, ldq = _rows_ld(q)
     krows, kcols, ldk = _rows_ld(kv)
-    _, yc, ldy = _rows_ld(y)
-    assert qc >= H * dk and krows == B * n_keys and kcols >= H * (dk + dv) and yc >= H * dv
+    yrows, yc, ldy = _rows_ld(y)
+    assert rows == yrows == B * S and qc >= H * dk and krows == B * n_keys and kcols >= G * (dk + dv) and yc >= H * dv
     assert pos.dtype == torch.int32 and pos.numel() == S and q.dtype == kv.dtype == y.dtype
     es = kv.element_size()
-    d = _WindowAttention(q=_dev(q, q.dtype), ldq=ldq, k=_dev(kv, q.dtype), v=kv.data_ptr() + H * dk * es, ldk=ldk,
+    d = _WindowAttention(q=_dev(q, q.dtype), ldq=ldq, k=_dev(kv, q.dtype), v=kv.data_ptr() + G * dk * es, ldk=ldk,
                          y=_dev(y, q.dtype), ldy=ldy, pos=pos.data_ptr(), B=B, S=S, H=H, dk=dk, dv=dv, window=int(window),
-                         n_keys=n_keys, Smax=Smax, dtype=_DTYPES[q.dtype], scale=scale)
+                         n_keys=n_keys, Smax=Smax, dtype=_DTYPES[q.dtype], kv_heads=G, scale=scale)
     _check(load().lr_window_attention(ctypes.byref(d), _stream()), "lr_window_attention")
     return y
 
@@ -767,6 +784,173 @@ def latent_attention(q, uk, uv, cache, y, pos, scratch, B, S, H, dk, dv, window:
                          rank=rank, window=int(window), Smax=cache.shape[1], dtype=_DTYPES[dt], scale=scale, eps=eps)
     _check(load().lr_latent_attention(ctypes.byref(d), _stream()), "lr_latent_attention")
     return y
+
+
+# ------------------------------------------------------------------------------------------------
+# dynamic tanh, selective state space, grouped attention through a window, mixture of experts
+# ------------------------------------------------------------------------------------------------
+
+def residual_tanh(x, d, alpha, gain, bias, x_out, x_compute, experts=None):
+    """x_out = x + d + the weighted expert rows; x_compute = tanh(alpha x_out) gain + bias.  x, x_out fp32 [rows, dim], the rest in
+    the compute type; experts = (rows [rows * top, dim], weights fp32 [rows, top]) or None."""
+    dim = x.shape[-1]
+    rows = x.numel() // dim
+    dt = gain.dtype
+    for t in (x, d, x_out, x_compute):
+        assert t is None or (t.is_contiguous() and t.numel() == rows * dim)
+    assert gain.numel() == dim and bias.numel() == dim and alpha.numel() == 1 and gain.is_contiguous() and bias.is_contiguous()
+    eo, ew, top = None, None, 0
+    if experts is not None:
+        eo, ew = experts
+        top = ew.shape[1]
+        assert eo.is_contiguous() and ew.is_contiguous() and ew.shape[0] == rows and eo.numel() == rows * top * dim
+    _check(load().lr_residual_tanh(_dev(x, torch.float32), _opt(d, dt), _opt(eo, dt), _opt(ew, torch.float32), top, _dev(alpha, dt),
+                                   _dev(gain, dt), _dev(bias, dt), _opt(x_out, torch.float32), _opt(x_compute, dt), rows, dim,
+                                   _DTYPES[dt], _stream()), "lr_residual_tanh")
+
+
+def causal_conv(u, w, bias, ring, pos, out, B, S):
+    """silu of the causal convolution per channel of u [B * S, C] (lr_causal_conv); ring [>= B, taps, C]."""
+    rows, C, ldu = _rows_ld(u)
+    orows, oc, ldo = _rows_ld(out)
+    taps = w.shape[1]
+    dt = u.dtype
+    assert rows == orows == B * S and oc == C and w.is_contiguous() and tuple(w.shape) == (C, taps) and bias.numel() == C
+    assert ring.is_contiguous() and ring.shape[0] >= B and tuple(ring.shape[1:]) == (taps, C)
+    assert pos.dtype == torch.int32 and pos.is_cuda and pos.numel() == S
+    _check(load().lr_causal_conv(_dev(u, dt), ldu, _dev(w, dt), _dev(bias, dt), _dev(ring, dt), pos.data_ptr(), _dev(out, dt), ldo, B, S,
+                                 C, taps, _DTYPES[dt], _stream()), "lr_causal_conv")
+    return out
+
+
+class _Ssd(ctypes.Structure):   # lr_ssd_t
+    _fields_ = [(n, c_void_p) for n in ("z", "x", "b", "c", "dt")] + [("ld", c_int64), ("ldu", c_int64)] + \
+               [(n, c_void_p) for n in ("dt_bias", "a_log", "d", "pos", "state", "y")] + \
+               [("ldy", c_int64), ("err", c_void_p), ("scratch", c_void_p), ("scratch_bytes", c_size_t)] + \
+               [(n, c_int32) for n in ("B", "S", "H", "G", "N", "P", "dtype")]
+
+
+def ssd_scratch_bytes(B, S, H, N, P, dtype) -> int:
+    return int(load().lr_ssd_scratch_bytes(B, S, H, N, P, _DTYPES[dtype]))
+
+
+def _ssd_desc(z, u, dt_raw, dt_bias, a_log, d, pos, state, y, B, S, H, G, scratch):
+    dt = u.dtype
+    N, P = state.shape[2:]
+    (zr, zc, ld), (ur, uc, ldu), (dr, dc, ldd), (yr, yc, ldy) = (_rows_ld(t) for t in (z, u, dt_raw, y))
+    assert zr == ur == dr == yr == B * S and zc >= H * P and uc == H * P + 2 * G * N and dc >= H and yc >= H * P and ld == ldd
+    assert state.is_contiguous() and state.shape[0] >= B and state.shape[1] == H and state.dtype == torch.float32
+    assert pos.dtype == torch.int32 and pos.is_cuda and pos.numel() == S
+    for t in (dt_bias, a_log, d):
+        assert t.numel() == H and t.is_contiguous() and t.dtype == dt
+    es = u.element_size()
+    x = _dev(u, dt)
+    assert dt_raw.is_cuda and dt_raw.dtype == dt
+    return _Ssd(z=_dev(z, dt), x=x, b=x + H * P * es, c=x + (H * P + G * N) * es, dt=dt_raw.data_ptr(), ld=ld, ldu=ldu,
+                dt_bias=dt_bias.data_ptr(), a_log=a_log.data_ptr(), d=d.data_ptr(), pos=pos.data_ptr(), state=_dev(state, torch.float32),
+                y=_dev(y, dt), ldy=ldy, err=device_error_word(u.device).data_ptr(),
+                scratch=None if scratch is None else scratch.data_ptr(),
+                scratch_bytes=0 if scratch is None else scratch.numel() * scratch.element_size(), B=B, S=S, H=H, G=G, N=N, P=P,
+                dtype=_DTYPES[dt])
+
+
+def ssd(z, u, dt_raw, dt_bias, a_log, d, pos, state, y, B, S, H, G, scratch=None):
+    """Selective state space over S tokens of B sequences (lr_ssd).  u [B * S, H P + 2 G N] = x | b | c after the convolution;
+    state fp32 [>= B, H, N, P]; y [B * S, >= H P]."""
+    desc = _ssd_desc(z, u, dt_raw, dt_bias, a_log, d, pos, state, y, B, S, H, G, scratch)
+    _check(load().lr_ssd(ctypes.byref(desc), _stream()), "lr_ssd")
+    return y
+
+
+def ssd_step(z, u, dt_raw, conv_w, conv_b, ring, dt_bias, a_log, d, pos, state, y, B, H, G):
+    """One token per sequence, convolution included (lr_ssd_step); u is the convolution's input."""
+    desc = _ssd_desc(z, u, dt_raw, dt_bias, a_log, d, pos, state, y, B, 1, H, G, None)
+    dt, C, taps = u.dtype, u.shape[-1], conv_w.shape[1]
+    assert conv_w.is_contiguous() and conv_w.shape[0] == C and conv_b.numel() == C
+    assert ring.is_contiguous() and ring.shape[0] >= B and tuple(ring.shape[1:]) == (taps, C)
+    _check(load().lr_ssd_step(ctypes.byref(desc), _dev(conv_w, dt), _dev(conv_b, dt), _dev(ring, dt), taps, _stream()), "lr_ssd_step")
+    return y
+
+
+def parts_norm(y, gain, parts: int, heads: int, P: int, PP: int, eps: float):
+    """RMS norm of `parts` equal ranges of heads * P columns (heads padded to PP), in place."""
+    rows, cols, ld = _rows_ld(y)
+    assert cols >= heads * PP and gain.numel() == heads * PP and gain.is_contiguous()
+    _check(load().lr_parts_norm(_dev(y, y.dtype), ld, _dev(gain, y.dtype), rows, heads * P, parts, P, PP, float(eps), _DTYPES[y.dtype],
+                                _stream()), "lr_parts_norm")
+    return y
+
+
+def bias_rope_cache(proj, bias, rope, pos, cache, B, S, H, G, dk, dv):
+    """Bias, rotation and cache write of a projection [q | k | v] (lr_bias_rope_cache); cache [>= B, Smax, ldc], or (None, Smax) for a
+    projection of q alone."""
+    rows, cols, ld = _rows_ld(proj)
+    dt = proj.dtype
+    cache, Smax, ldc = (None, cache[1], 0) if isinstance(cache, tuple) else (cache, cache.shape[1], cache.shape[2])
+    assert rows == B * S and pos.dtype == torch.int32 and pos.is_cuda and pos.numel() == S
+    want = H * dk + (0 if cache is None else G * (dk + dv))
+    assert cols >= want and (bias is None or (bias.numel() >= want and bias.is_contiguous()))
+    assert cache is None or (cache.is_contiguous() and cache.shape[0] >= B)
+    rot, rope_len = 0, 0
+    if rope is not None:
+        assert rope.is_contiguous() and rope.shape[2] == 2
+        rope_len, rot = rope.shape[0], 2 * rope.shape[1]
+    _check(load().lr_bias_rope_cache(_dev(proj, dt), ld, _opt(bias, dt), _opt(rope, torch.float32), pos.data_ptr(), _opt(cache, dt), B, S,
+                                     H, G, dk, dv, rot, rope_len, ldc, Smax, _DTYPES[dt], device_error_word(proj.device).data_ptr(),
+                                     _stream()), "lr_bias_rope_cache")
+
+
+def window_decode_scratch_bytes(B, H, G, dv, window, Smax) -> int:
+    return int(load().lr_window_decode_scratch_bytes(B, H, G, dv, window, Smax))
+
+
+def window_decode(q, cache, y, pos, scratch, B, H, G, dk, dv, window: int, scale: float):
+    """Sliding-window attention of one query per sequence over a cache [>= B, Smax, >= G (dk + dv)] (lr_window_decode)."""
+    rows, qc, ldq = _rows_ld(q)
+    yrows, yc, ldy = _rows_ld(y)
+    assert rows == yrows == B and qc >= H * dk and yc >= H * dv and cache.is_contiguous() and cache.shape[0] >= B
+    assert pos.dtype == torch.int32 and pos.numel() == 1
+    _check(load().lr_window_decode(_dev(q), ldq, _dev(cache), pos.data_ptr(), _dev(y), ldy, B, H, G, dk, dv, cache.shape[2],
+                                   cache.shape[1], int(window), float(scale), scratch.data_ptr(),
+                                   scratch.numel() * scratch.element_size(), _stream()), "lr_window_decode")
+    return y
+
+
+class _Moe(ctypes.Structure):   # lr_moe_t
+    _fields_ = [("x", c_void_p), ("ldx", c_int64)] + \
+               [(n, c_void_p) for n in ("router", "router_bias", "w1", "w2", "out", "experts", "weights", "counts", "shared")] + \
+               [("ld_shared", c_int64), ("scratch", c_void_p), ("scratch_bytes", c_size_t)] + \
+               [(n, c_int32) for n in ("rows", "D", "I", "E", "top", "shared_cols", "dtype")]
+
+
+def moe_scratch_bytes(rows, E, top, I, shared: bool, dtype) -> int:
+    return int(load().lr_moe_scratch_bytes(rows, E, top, I, int(shared), _DTYPES[dtype]))
+
+
+def moe(x, router, router_bias, w1, w2, out, experts, weights, counts, scratch, shared=None):
+    """Mixture of experts (lr_moe): out [rows * top, D] a row per choice, experts / weights [rows, top] the choices.  `shared`: a
+    shared expert's activations [rows, cols], multiplied in place by the sigmoid of their gate (the router's last row)."""
+    rows, D, ldx = _rows_ld(x)
+    E, two_i, Dw = w1.shape
+    top = weights.shape[1]
+    dt = x.dtype
+    n = E + (shared is not None)
+    assert Dw == D and tuple(w2.shape) == (E, D, two_i // 2) and tuple(router.shape) == (n, D) and router_bias.numel() == E
+    for t in (router, router_bias, w1, w2, out, experts, weights, counts):
+        assert t.is_contiguous()
+    assert out.numel() == rows * top * D and tuple(experts.shape) == tuple(weights.shape) == (rows, top)
+    assert counts.numel() == E and counts.dtype == experts.dtype == torch.int32
+    sp, lds, sc = None, 0, 0
+    if shared is not None:
+        srows, sc, lds = _rows_ld(shared)
+        assert srows == rows
+        sp = _dev(shared, dt)
+    d = _Moe(x=_dev(x, dt), ldx=ldx, router=_dev(router, dt), router_bias=_dev(router_bias, dt), w1=_dev(w1, dt), w2=_dev(w2, dt),
+             out=_dev(out, dt), experts=experts.data_ptr(), weights=_dev(weights, torch.float32), counts=counts.data_ptr(), shared=sp,
+             ld_shared=lds, scratch=scratch.data_ptr(), scratch_bytes=scratch.numel() * scratch.element_size(), rows=rows, D=D,
+             I=two_i // 2, E=E, top=top, shared_cols=sc, dtype=_DTYPES[dt])
+    _check(load().lr_moe(ctypes.byref(d), _stream()), "lr_moe")
+    return out
 
 
 def _ladder_model_desc(model, attention_workgroups: int = 0):

@@ -20,6 +20,8 @@ Three steps, each usable on its own (all on plain state dicts, CPU tensors are f
 
   convert_lasivik_state_dict  a Lasivik checkpoint's names (`embed`, `l<i>.mix.*`, `l<i>.mlp.*`, `head`, ...) ->
                           GPTLasivik's, projections of the same input fused, padded columns and rows zero.
+  convert_gepolix_state_dict  a Gepolix checkpoint's names -> GPTGepolix's; heads padded, the projections that share an output
+                          side by side, experts stacked.
   load_pretrained         a folder with config.json and weights -> the model it describes, loaded.
 
 `model_args_from_hf_config` turns the fields of an HF config.json (hf_modeling_utils/configs/*.json)
@@ -31,7 +33,7 @@ from typing import Dict, List, Optional, Union
 import torch
 from torch import Tensor
 
-from .mixers import pad8
+from .mixers import pad8, pad16
 
 StateDict = Dict[str, Tensor]
 
@@ -116,11 +118,31 @@ def model_args_from_hf_config(cfg: Union[str, dict], **overrides) -> dict:
 
 
 # ------------------------------------------------------------------------------------------------
-# Lasivik names -> GPTLasivik names
+# Lasivik names -> GPTLasivik names, Gepolix names -> GPTGepolix names
 # ------------------------------------------------------------------------------------------------
 
-def is_lasivik_state_dict(sd: StateDict) -> bool:
+def is_listed_layers_state_dict(sd: StateDict) -> bool:
+    """The names of the families whose configuration lists the layers."""
     return "embed" in sd and "final.norm" in sd
+
+
+class _Taker:
+    """Hands out a checkpoint's tensors once each, shapes checked; raises on missing ones and on what is left over."""
+
+    def __init__(self, sd: StateDict):
+        self.left = dict(sd)
+
+    def __call__(self, name: str, *shape: int) -> Tensor:
+        if name not in self.left:
+            raise KeyError(f"checkpoint has no tensor {name!r}")
+        w = self.left.pop(name)
+        if tuple(w.shape) != shape:
+            raise ValueError(f"{name}: checkpoint {tuple(w.shape)}, configuration {shape}")
+        return w
+
+    def finish(self):
+        if self.left:
+            raise KeyError(f"tensors the configuration does not account for: {sorted(self.left)[:6]}")
 
 
 def lasivik_decay_ranks(sd: StateDict) -> Dict[int, int]:
@@ -140,19 +162,10 @@ def _padded(w: Tensor, *shape: int) -> Tensor:
 def convert_lasivik_state_dict(sd: StateDict, args) -> StateDict:
     """Checkpoint names -> GPTLasivik parameter names for LasivikArgs `args`.  Raises on tensors the configuration does
     not account for and on missing ones."""
-    left = dict(sd)
+    take = _Taker(sd)
     out: StateDict = {}
     D = args.dim
     W = args.width
-
-    def take(name: str, *shape: int) -> Tensor:
-        if name not in left:
-            raise KeyError(f"checkpoint has no tensor {name!r}")
-        w = left.pop(name)
-        if tuple(w.shape) != shape:
-            raise ValueError(f"{name}: checkpoint {tuple(w.shape)}, configuration {shape}")
-        return w
-
     wide = lambda w: _padded(w, w.shape[0], D)          # a projection of the residual stream
     out["tok_embeddings.weight"] = wide(take("embed", args.vocab_size, W))
     for i, layer in enumerate(args.layers):
@@ -183,8 +196,78 @@ def convert_lasivik_state_dict(sd: StateDict, args) -> StateDict:
             out[f"layers.{i}.ffn_norm.weight"] = _padded(take(f"l{i}.norm2", W), D)
     out["norm.weight"] = _padded(take("final.norm", W), D)
     out["output.weight"] = wide(take("head", args.vocab_size, W))
-    if left:
-        raise KeyError(f"tensors the configuration does not account for: {sorted(left)[:6]}")
+    take.finish()
+    return out
+
+
+def _pad_heads(w: Tensor, heads: int, size: int, to: int) -> Tensor:
+    """Dimension 0, heads * size long, as heads * to: zeros behind every head."""
+    if size == to:
+        return w
+    return _padded(w.reshape(heads, size, *w.shape[1:]), heads, to, *w.shape[1:]).reshape(heads * to, *w.shape[1:])
+
+
+def convert_gepolix_state_dict(sd: StateDict, args) -> StateDict:
+    """Checkpoint names -> GPTGepolix parameter names for GepolixArgs `args`.  Raises on tensors the configuration does not
+    account for and on missing ones."""
+    take = _Taker(sd)
+    out: StateDict = {}
+    D, W = args.dim, args.width
+    wide = lambda w: _padded(w, w.shape[0], D)          # a projection of the residual stream
+
+    def tanh(src: str, dst: str):
+        out[dst + ".alpha"] = take(src + ".alpha").reshape(1)
+        out[dst + ".weight"], out[dst + ".bias"] = _padded(take(src, W), D), _padded(take(src + ".b", W), D)
+
+    def up_gate(src: str, I: int) -> Tensor:
+        return torch.cat([_padded(take(src + n, I, W), pad8(I), D) for n in ("up", "gate")])
+
+    def down(src: str, I: int) -> Tensor:
+        return _padded(take(src + "down", W, I), D, pad8(I))
+
+    def mamba2(m, src: str, dst: str) -> Tensor:
+        H, G, P, N = m.heads, m.groups, m.vdim, m.state
+        Pp, Np = pad16(P), pad16(N)
+        head, group = (lambda w: _pad_heads(w, H, P, Pp)), (lambda w: _pad_heads(w, G, N, Np))
+        xbc = lambda w: torch.cat([f(p) for f, p in zip((head, group, group), w.split([H * P, G * N, G * N]))])
+        z, u, dt = take(src + "in", 2 * H * P + 2 * G * N + H, W).split([H * P, H * P + 2 * G * N, H])
+        out[dst + "in_proj.weight"] = wide(torch.cat([head(z), xbc(u), dt]))
+        out[dst + "conv_weight"] = xbc(take(src + "conv", H * P + 2 * G * N, m.taps))
+        out[dst + "conv_bias"] = xbc(take(src + "conv.b", H * P + 2 * G * N))
+        for name, t in (("dt_bias", "dt_bias"), ("a_log", "A_log"), ("d", "D")):
+            out[dst + name] = take(src + t, H)
+        out[dst + "norm.weight"] = head(take(src + "norm", H * P))
+        return head(take(src + "o", W, H * P).T).T
+
+    def attention(m, src: str, dst: str) -> Tensor:
+        rows = [("q", m.heads, m.dim)] + ([] if m.kv_from is not None else [("k", m.kv_heads, m.dim), ("v", m.kv_heads, m.vdim)])
+        heads = lambda suffix, *cols: torch.cat([_pad_heads(take(src + n + suffix, h * d, *cols), h, d, pad8(d)) for n, h, d in rows])
+        out[dst + "in_proj.weight"], out[dst + "in_proj.bias"] = wide(heads("", W)), heads(".b")
+        return _pad_heads(take(src + "o", W, m.heads * m.vdim).T, m.heads, m.vdim, pad8(m.vdim)).T
+
+    out["tok_embeddings.weight"] = wide(take("embed", args.vocab_size, W))
+    for i, layer in enumerate(args.layers):
+        dst, src, m = f"layers.{i}.", f"l{i}.mlp.", layer.mixer
+        tanh(f"l{i}.norm1", dst + "norm")
+        o = {"mamba2": mamba2, "attention": attention}[m.kind](m, f"l{i}.mix.", dst + "mixer.")
+        o = [_padded(o, D, o.shape[1])]
+        if layer.ffn is not None:
+            out[dst + "w1.weight"] = up_gate(src, layer.ffn)
+            o.append(down(src, layer.ffn))
+        x = layer.experts
+        if x is not None:
+            router = [wide(take(src + "router", x.experts, W))]
+            if x.shared is not None:
+                router.append(wide(take(src + "shared.sg", 1, W)))
+                out[dst + "w1.weight"] = up_gate(src + "shared.", x.shared)
+                o.append(down(src + "shared.", x.shared))
+            out[dst + "experts.router"], out[dst + "experts.router_bias"] = torch.cat(router), take(src + "router.b", x.experts)
+            out[dst + "experts.w1"] = torch.stack([up_gate(f"{src}e{e}.", x.ff) for e in range(x.experts)])
+            out[dst + "experts.w2"] = torch.stack([down(f"{src}e{e}.", x.ff) for e in range(x.experts)])
+        out[dst + "mixer.out_proj.weight"] = torch.cat(o, dim=1)
+    tanh("final.norm", "norm")
+    out["output.weight"] = wide(take("head", args.vocab_size, W))
+    take.finish()
     return out
 
 
@@ -268,14 +351,17 @@ def read_state_dict(path: str) -> StateDict:
 
 
 def load_checkpoint(model: torch.nn.Module, checkpoint: Union[str, StateDict], already_sharded: bool = False) -> List[str]:
-    """Load an un-sharded checkpoint (HF, Lasivik or gpt_fast names; a path or a state dict) into `model`,
+    """Load an un-sharded checkpoint (HF, Lasivik, Gepolix or gpt_fast names; a path or a state dict) into `model`,
     which was built for one tensor-parallel rank (model.config.tp_world_size / tp_rank).
     Returns the names of the tensors that were loaded.  Raises on missing or unexpected
     parameters; buffers the checkpoint does not carry (KV caches, masks) are left alone."""
     cfg = model.config
     sd = read_state_dict(checkpoint) if isinstance(checkpoint, (str, os.PathLike)) else dict(checkpoint)
-    if is_lasivik_state_dict(sd):
-        sd = convert_lasivik_state_dict(sd, cfg)
+    if is_listed_layers_state_dict(sd):
+        convert = {"lasivik": convert_lasivik_state_dict, "gepolix": convert_gepolix_state_dict}.get(model.family)
+        if convert is None:
+            raise ValueError(f"the checkpoint's names are those of a family of listed layers, not of {type(model).__name__}")
+        sd = convert(sd, cfg)
         already_sharded = True   # one rank holds all of it
     if is_hf_state_dict(sd):
         # an already sharded checkpoint holds this rank's heads only
@@ -312,14 +398,16 @@ def _folder_config(folder: str) -> dict:
 
 
 def pretrained_class(folder: str):
-    """The model class a checkpoint folder's config.json asks for: `architecture` "Lasivik" -> GPTLasivik; a Hugging Face
-    Llama or Llama-Ladder configuration -> GPTLadder (whose layers outside `ladder_layers` are dense)."""
+    """The model class a checkpoint folder's config.json asks for: `architecture` "Lasivik" -> GPTLasivik, "Gepolix" ->
+    GPTGepolix; a Hugging Face Llama or Llama-Ladder configuration -> GPTLadder (whose layers outside `ladder_layers` are dense)."""
+    from .gpt_gepolix import GPTGepolix
     from .gpt_ladder_TP import GPTLadder
     from .gpt_lasivik import GPTLasivik
 
     cfg = _folder_config(folder)
-    if cfg.get("architecture") == "Lasivik":
-        return GPTLasivik
+    listed = {"Lasivik": GPTLasivik, "Gepolix": GPTGepolix}.get(cfg.get("architecture"))
+    if listed is not None:
+        return listed
     if "hidden_size" in cfg:
         return GPTLadder
     raise ValueError(f"{folder}/config.json describes no model this package has")
@@ -327,14 +415,18 @@ def pretrained_class(folder: str):
 
 def load_pretrained(folder: str, device="cuda", dtype: torch.dtype = torch.bfloat16) -> torch.nn.Module:
     """The model a checkpoint folder (config.json and weights) describes, on `device` in `dtype`."""
-    from .config import LasivikArgs, ModelArgs
+    from .config import GepolixArgs, LasivikArgs, ModelArgs
 
     cls = pretrained_class(folder)
     if dtype not in cls.supported_dtypes:
         raise NotImplementedError(f"{cls.__name__} does not run in {dtype}")
     cfg, sd = _folder_config(folder), read_state_dict(folder)
-    args = LasivikArgs.from_config(cfg, lasivik_decay_ranks(sd)) if cls.family == "lasivik" else \
-        ModelArgs(**model_args_from_hf_config(cfg))
+    if cls.family == "lasivik":
+        args = LasivikArgs.from_config(cfg, lasivik_decay_ranks(sd))
+    elif cls.family == "gepolix":
+        args = GepolixArgs.from_config(cfg)
+    else:
+        args = ModelArgs(**model_args_from_hf_config(cfg))
     with torch.device("meta"):
         model = cls(args)
     model = model.to(dtype=dtype).to_empty(device=device)

@@ -196,9 +196,18 @@ def _build_family(family: str) -> Dict[str, dict]:
 # ------------------------------------------------------------------------------------------------
 
 @dataclass
+class ExpertArgs:
+    experts: int
+    top: int                        # experts a token uses
+    ff: int                         # width of each
+    shared: Optional[int] = None    # width of an expert every token uses besides
+
+
+@dataclass
 class LayerArgs:
     mixer: MixerArgs
     ffn: Optional[int]              # feed-forward width, None: the layer has none
+    experts: Optional[ExpertArgs] = None   # a mixture instead (ffn None)
 
 
 @dataclass
@@ -274,8 +283,103 @@ _LASIVIK = {
     "lasivik-8b": _lasivik_config(4096, 14336, 128256, 8, 32, 1024),
 }
 
+# ------------------------------------------------------------------------------------------------
+# Gepolix: a parallel hybrid of state spaces and windowed attention, dense or with experts
+# ------------------------------------------------------------------------------------------------
+
+@dataclass
+class GepolixArgs:
+    vocab_size: int
+    width: int                      # `dim`, the padded width, is what buffers and weights have
+    layers: List[LayerArgs]
+    norm_eps: float                 # of the mixers' own norms
+    block_size: int = 1 << 30       # no table limits the positions: the caches' length does
+    tp_world_size: int = 1
+
+    def __post_init__(self):
+        if _tp.get_tp_world_size() != 1:
+            raise NotImplementedError("Gepolix models run whole on one GPU: their mixers are not sharded over ranks")
+
+    @property
+    def dim(self) -> int:
+        return pad8(self.width)
+
+    @property
+    def n_layer(self) -> int:
+        return len(self.layers)
+
+    @property
+    def output_rows(self) -> int:
+        return self.vocab_size
+
+    @classmethod
+    def from_config(cls, cfg: dict) -> "GepolixArgs":
+        """From a parsed config.json."""
+        layers = []
+        for i, layer in enumerate(cfg["layers"]):
+            kind, m, mlp = layer["type"], layer["mixer"], layer.get("mlp")
+            if kind == "mamba2":
+                args = MixerArgs(kind=kind, heads=m["heads"], dim=0, vdim=m["vdim"], state=m["state"], groups=m["groups"],
+                                 norm_groups=m["norm_groups"], taps=m["conv"])
+                assert args.heads % args.groups == 0 and args.heads * args.vdim % args.norm_groups == 0, f"layer {i}"
+            elif kind == "attention":
+                args = MixerArgs(kind=kind, heads=m["heads"], dim=m["dim"], vdim=m["vdim"], kv_heads=m["kv_heads"],
+                                 kv_from=m.get("kv_from"), rot_dims=m["rot"]["dims"], rot_base=float(m["rot"]["base"]),
+                                 window=m["mask"]["size"], scale=float(m["scale"]), bias=True)
+                assert args.heads % args.kv_heads == 0, f"layer {i}"
+                j = args.kv_from
+                if j is not None:
+                    lender = layers[j].mixer if 0 <= j < i else None
+                    if lender is None or lender.kind != kind or lender.kv_from is not None:
+                        raise ValueError(f"layer {i}: layer {j} is no earlier layer with keys and values of its own")
+                    if (lender.kv_heads, lender.dim, lender.vdim) != (args.kv_heads, args.dim, args.vdim):
+                        raise ValueError(f"layer {i}: heads differ from layer {j}'s, whose keys and values it uses")
+            else:
+                raise ValueError(f"layer {i}: unknown mixer {kind!r}")
+            ffn = experts = None
+            if mlp is not None and mlp["kind"] == "dense":
+                ffn = mlp["ff"]
+            elif mlp is not None and mlp["kind"] == "moe":
+                shared = mlp.get("shared")
+                experts = ExpertArgs(mlp["router"]["experts"], mlp["router"]["top"], mlp["expert"]["ff"],
+                                     None if shared is None else shared["ff"])
+                assert 0 < experts.top <= experts.experts, f"layer {i}"
+            elif mlp is not None:
+                raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
+            layers.append(LayerArgs(args, ffn, experts))
+        return cls(vocab_size=cfg["vocab"], width=cfg["width"], layers=layers, norm_eps=float(cfg["norm"]["eps"]))
+
+
+def _gepolix_config(width: int, ff: int, vocab: int, periods: int, heads: int, kv_heads: int, window: int, groups: int, moe: dict) -> dict:
+    """A config.json of the design: (state space, state space with experts, attention, state space with experts) `periods` times;
+    every other attention layer reads the keys and values of the one before."""
+    ssm = dict(heads=2 * width // 64, vdim=64, state=128, groups=groups, norm_groups=groups, conv=4)
+    attention = dict(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, mask=dict(size=window), rot=dict(dims=128, base=500000.0),
+                     scale=128 ** -0.5)
+    dense = dict(kind="dense", ff=ff)
+    layers = []
+    for i in range(periods):
+        lent = dict(attention, kv_from=4 * i - 2) if i % 2 else attention
+        layers += [dict(type="mamba2", mixer=ssm, mlp=dense), dict(type="mamba2", mixer=ssm, mlp=moe),
+                   dict(type="attention", mixer=lent, mlp=dense), dict(type="mamba2", mixer=ssm, mlp=moe)]
+    return dict(architecture="Gepolix", vocab=vocab, width=width, norm=dict(eps=1e-5), layers=layers)
+
+
+def _moe(experts: int, top: int, ff: int, shared: int) -> dict:
+    return dict(kind="moe", router=dict(experts=experts, top=top), expert=dict(ff=ff), shared=dict(ff=shared))
+
+
+# benchmark shapes: layers of the size of the other families' "...-1b" and "...-8b", the experts together as wide as a dense
+# feed-forward
+_GEPOLIX = {
+    "gepolix-1b": _gepolix_config(2048, 8192, 128256, 4, 16, 4, 1024, 4, _moe(16, 4, 448, 1024)),
+    "gepolix-8b": _gepolix_config(4096, 14336, 128256, 8, 32, 8, 1024, 8, _moe(32, 6, 384, 2048)),
+}
+
 REGISTRIES = {f: _build_family(f) for f in ("ladder", "dense", "desync", "parallel")}
 REGISTRIES["lasivik"] = _LASIVIK
+REGISTRIES["gepolix"] = _GEPOLIX
+_LISTED = {"lasivik": LasivikArgs, "gepolix": GepolixArgs}   # families whose registry holds config.json dictionaries
 
 
 def args_from_name(family: str, name: str):
@@ -283,4 +387,4 @@ def args_from_name(family: str, name: str):
     if name not in reg:
         # the reference returns None here and fails later with an AttributeError (gpt_ladder_TP.py:59-62)
         raise KeyError(f"unknown {family} config '{name}'; known: {sorted(reg)}")
-    return LasivikArgs.from_config(reg[name]) if family == "lasivik" else ModelArgs(**reg[name])
+    return _LISTED[family].from_config(reg[name]) if family in _LISTED else ModelArgs(**reg[name])

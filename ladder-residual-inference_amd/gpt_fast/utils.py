@@ -69,6 +69,39 @@ class RMSNorm(nn.Module):
         return _hip.add_rmsnorm(x, None, None, self.weight, None, torch.empty_like(x), self.eps)
 
 
+class DynamicTanh(nn.Module):
+    """tanh(alpha x) weight + bias: a norm without statistics, alpha a single number."""
+
+    def __init__(self, dim: int):
+        super().__init__()
+        self.alpha = nn.Parameter(torch.ones(1))
+        self.weight = nn.Parameter(torch.ones(dim))
+        self.bias = nn.Parameter(torch.zeros(dim))
+
+    def into(self, x: Tensor, d: Optional[Tensor], x_out: Optional[Tensor], out: Tensor, experts=None):
+        """x_out = x + d + the experts' weighted rows, out = the norm of it, in one pass."""
+        _hip.residual_tanh(x, d, self.alpha, self.weight, self.bias, x_out, out, experts)
+
+
+class Experts(nn.Module):
+    """`n` gated feed-forwards of width ff, of which a token uses `top`.  w1 rows of an expert are [up; gate].  With a shared
+    expert the router has one row more, that expert's gate."""
+
+    def __init__(self, dim: int, n: int, top: int, ff: int, shared: bool):
+        super().__init__()
+        self.n, self.top, self.ff, self.shared = n, top, ff, shared
+        self.router = nn.Parameter(torch.zeros(n + shared, dim))
+        self.router_bias = nn.Parameter(torch.zeros(n))
+        self.w1 = nn.Parameter(torch.zeros(n, 2 * ff, dim))
+        self.w2 = nn.Parameter(torch.zeros(n, dim, ff))
+
+    def run(self, x: Tensor, shared_act: Optional[Tensor], out: Tensor, ids: Tensor, weights: Tensor, counts: Tensor, scratch: Tensor):
+        """A row per (token, choice) into `out`; shared_act (a shared expert's activations) times its gate.  Returns what
+        residual_tanh adds up."""
+        _hip.moe(x, self.router, self.router_bias, self.w1, self.w2, out, ids, weights, counts, scratch, shared_act)
+        return out, weights
+
+
 def apply_rope_scaling(freqs: torch.Tensor, rope_scaling: dict) -> torch.Tensor:
     """Llama-3.1 frequency scaling: keep short wavelengths, divide long ones by `factor`, blend the
     band in between.  Same element-wise fp32 evaluation order as the reference (utils.py:81-100)."""

@@ -251,7 +251,7 @@ def test_new_entry_points_validate_before_any_device_work():
     assert lib.lr_residual_rmsnorm(64, 1.0, None, 64, 0.0, 64, None, 1, 8, 8, 1e-5, 7, None) == UNSUP
     assert lib.lr_logit_cap(64, 4, 1, 8, 1.0, 1.0, 0, None) == SHAPE
     assert lib.lr_linear_f32(64, 4, 64, 64, 8, 1, 8, 8, None) == SHAPE
-    assert lib.lr_swiglu_f32(None, 4, 64, 1, 2, None) == NULL
+    assert lib.lr_swiglu_f32(None, 4, 64, 2, 1, 2, None) == NULL
 
     la = _hip._LinearAttention(q=64, k=64, v=64, g=64, ld=64, head_decay=64, pos=64, state=64, y=64, ldy=64, B=1, S=4, H=2, dk=16,
                                dv=16, rank=0, rot_dims=0, rope_len=0, dtype=0, tau=1.0, q_scale=1.0, k_scale=1.0, eps=1e-5)
