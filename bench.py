@@ -1,7 +1,8 @@
 """Headline benchmark: batch-1 greedy decode of one TP=8 rank shard of Ladder-70B on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch B] [--no-cpu-baseline]
-    python bench.py --lasivik [SIZE ...]     # another workload, see below
+    python bench.py --lasivik [SIZE ...]     # other workloads, see below
+    python bench.py --gepolix [SIZE ...]
 
 A "step" is one decode step (one new token per sequence) of the whole per-rank forward pass,
 replayed as a captured hipGraph: embedding -> 80 ladder blocks -> final add/norm -> vocab-shard
@@ -41,6 +42,7 @@ Measured in the same run and reported as extra keys (not the headline; --no-extr
                gpt_dense:ladder-1b, lasivik-8b / gpt_dense:ladder-8b; random weights): prefill and decode throughput at
                several batch sizes, and the kernels only one of the two has, each timed alone over data that does not
                fit the caches, with the fraction of its roofline.  One JSON line of its own.
+`--gepolix`   : the same for the Gepolix hybrid beside the Lasivik one (gepolix-1b / lasivik-1b, gepolix-8b / lasivik-8b).
 `prefill`     : Ladder-8B, batch 32 x 2048 prompt tokens, causal prefill with last-position logits:
                seconds, algorithmic TFLOP/s and the fraction of 2.5 PFLOP/s (dense bf16 MFMA peak)."""
 import argparse
@@ -240,6 +242,7 @@ def _graph_us(calls, reps=5):
     for c in calls[:2]:
         c()
     torch.cuda.synchronize()
+    calls = calls * max(1, 16 // len(calls))      # (the replay's own cost is spread over them)
     g = torch.cuda.CUDAGraph()
     with torch.cuda.graph(g):
         for c in calls:
@@ -259,6 +262,136 @@ def _kernel_row(name, us, bound, work):
     """`work`: bytes (bound hbm) or FLOP (bound mfma: bf16, mfma_f32)."""
     peak = {"hbm": HBM_PEAK_GBPS * 1e9, "mfma": MFMA_PEAK_TFLOPS * 1e12, "mfma_f32": FP32_MATRIX_PEAK_TFLOPS * 1e12}[bound]
     return {"kernel": name, "us": round(us, 2), "bound": bound, "work": int(work), "frac": round(work / (us * 1e-6) / peak, 4)}
+
+
+def _residual_norm_row(D, rows, copies):
+    import torch
+
+    from gpt_fast import _hip
+
+    n = copies(rows * D * 12)
+    rnd = lambda *s: torch.randn(*s, device="cuda")
+    xs, ds = [rnd(rows, D) for _ in range(n)], [rnd(rows, D).bfloat16() for _ in range(n)]
+    xc, gain = torch.empty(rows, D, dtype=torch.bfloat16, device="cuda"), rnd(D).bfloat16()
+    us = _graph_us([lambda i=i: _hip.residual_rmsnorm(xs[i], 2.0, ds[i], gain, xs[i], xc, 1e-5, gain_offset=1.0) for i in range(n)])
+    return _kernel_row("lr_residual_rmsnorm (fp32 residual)", us, "hbm", rows * D * (4 + 2 + 4 + 2))
+
+
+def gepolix_kernels(model, lasivik, B, T, decode):
+    """The kernels the Gepolix model does not share, then the like kernels of the Lasivik model, as in mixer_kernels."""
+    import torch
+
+    from gpt_fast import _hip
+
+    dev, BF = "cuda", torch.bfloat16
+    S = 1 if decode else T
+    rows, L, D = B * S, T + 8, model.config.dim
+    pos = torch.arange(T, T + 1, dtype=torch.int32, device=dev) if decode else torch.arange(T, dtype=torch.int32, device=dev)
+    rnd = lambda *s, dt=BF: torch.randn(*s, device=dev, dtype=torch.float32).to(dt)
+    copies = lambda nbytes: max(2, min(64, (600 << 20) // max(int(nbytes), 1))) if decode else 2
+    bytes_of = lambda t, n: [torch.empty(max(n, 16), dtype=torch.uint8, device=dev) for _ in range(t)]
+    out = []
+    blocks = {}
+    for blk in model.layers:
+        blocks.setdefault(blk.mixer.args.kind, blk)
+        blocks.setdefault("moe" if blk.experts is not None else "dense", blk)
+    # state space
+    m = blocks["mamba2"].mixer
+    a = m.args
+    proj, y = rnd(rows, (m.proj_cols + 7) // 8 * 8), torch.empty(rows, m.y_cols, dtype=BF, device=dev)
+    z, u, dt = proj[:, :m.inner], proj[:, m.inner:m.inner + m.conv_cols], proj[:, m.inner + m.conv_cols:m.proj_cols]
+    cw, cb = rnd(m.conv_cols, a.taps), rnd(m.conv_cols)
+    db, al, dd = rnd(a.heads), rnd(a.heads), rnd(a.heads)
+    carried = 2 * B * a.heads * m.N * m.P * 4
+    n = copies(carried)
+    states, rings = [torch.zeros(B, a.heads, m.N, m.P, device=dev) for _ in range(n)], torch.zeros(B, a.taps, m.conv_cols, dtype=BF, device=dev)
+    name = f"{a.heads} heads of {m.N} x {m.P}"
+    act_bytes = rows * 2 * (2 * m.inner + m.conv_cols + a.heads)
+    if decode:
+        us = _graph_us([lambda s=s: _hip.ssd_step(z, u, dt, cw, cb, rings, db, al, dd, pos, s, y, B, a.heads, a.groups) for s in states])
+        out.append(_kernel_row(f"lr_ssd_step ({name}; convolution included)", us, "hbm", carried + act_bytes))
+    else:
+        c = rnd(rows, m.conv_cols)
+        us = _graph_us([lambda: _hip.causal_conv(u, cw, cb, rings, pos, c, B, S)])
+        out.append(_kernel_row("lr_causal_conv", us, "hbm", 4 * rows * m.conv_cols))
+        scratch = bytes_of(1, _hip.ssd_scratch_bytes(B, S, a.heads, m.N, m.P, BF))[0]
+        us = _graph_us([lambda s=s: _hip.ssd(z, c, dt, db, al, dd, pos, s, y, B, S, a.heads, a.groups, scratch=scratch) for s in states])
+        out.append(_kernel_row(f"lr_ssd ({name})", us, "hbm", act_bytes))
+        # per token and head: the state is multiplied by C and added B x^T to; inside a chunk of 64 the scores and their sums
+        flop = rows * a.heads * (4 * m.N * m.P + 2 * 64 * (m.N + m.P) // 2)
+        out.append(dict(out[-1], bound="mfma", work=int(flop), frac=round(flop / (us * 1e-6) / (MFMA_PEAK_TFLOPS * 1e12), 4)))
+    gain = rnd(m.inner)
+    us = _graph_us([lambda: _hip.parts_norm(y, gain, a.norm_groups, a.heads, a.vdim, m.P, 1e-5)])
+    out.append(_kernel_row("lr_parts_norm", us, "hbm", 4 * rows * m.inner))
+    del states, proj, y, z, u, dt
+    # attention
+    m = blocks["attention"].mixer
+    a = m.args
+    seen = min(T + 1, a.window)
+    proj, y, bias = rnd(rows, m.proj_cols), torch.empty(rows, m.y_cols, dtype=BF, device=dev), rnd(m.proj_cols)
+    nbytes = B * m.kv_cols * 2 * seen
+    n = copies(nbytes)
+    caches = [rnd(B, L, m.kv_cols) for _ in range(n)]
+    rope = torch.zeros(L, a.rot_dims // 2, 2, device=dev)
+    q = proj[:, :a.heads * m.dk]
+    us = _graph_us([lambda c=c: _hip.bias_rope_cache(proj, bias, rope, pos, c, B, S, a.heads, a.kv_heads, m.dk, m.dv) for c in caches])
+    out.append(_kernel_row("lr_bias_rope_cache", us, "hbm", 4 * rows * m.proj_cols))
+    name = f"{a.heads} / {a.kv_heads} heads of {a.dim}, window {a.window}"
+    if decode:
+        scratch = bytes_of(1, _hip.window_decode_scratch_bytes(B, a.heads, a.kv_heads, m.dv, a.window, L))[0]
+        us = _graph_us([lambda c=c: _hip.window_decode(q, c, y, pos, scratch, B, a.heads, a.kv_heads, m.dk, m.dv, a.window, a.scale)
+                        for c in caches])
+        out.append(_kernel_row(f"lr_window_decode ({name}; two launches)", us, "hbm", nbytes))
+    else:
+        kv = caches[0].view(B * L, -1)
+        us = _graph_us([lambda: _hip.window_attention(q, kv, y, pos, B, S, a.heads, m.dk, m.dv, a.window, L, L, a.scale,
+                                                      kv_heads=a.kv_heads)])
+        keys = sum(min(i + 1, a.window) for i in range(T))
+        out.append(_kernel_row(f"lr_window_attention ({name})", us, "mfma", B * a.heads * keys * 2 * (a.dim + a.vdim)))
+    del caches, proj, y, q
+    # feed-forwards: the mixture; the dense one of the same model (as the Lasivik model's, two launches) for comparison
+    x = blocks["moe"].experts
+    xc = rnd(rows, D)
+    distinct = x.n * (1 - (1 - x.top / x.n) ** rows)
+    wbytes = int(distinct * 3 * x.ff * D * 2)
+    n = copies(x.n * 3 * x.ff * D * 2)
+    w1s, w2s = [rnd(x.n, 2 * x.ff, D) for _ in range(n)], [rnd(x.n, D, x.ff) for _ in range(n)]
+    router, rb = rnd(x.n + x.shared, D), rnd(x.n)
+    eo, ids, wts = torch.empty(rows * x.top, D, dtype=BF, device=dev), torch.empty(rows, x.top, dtype=torch.int32, device=dev), torch.empty(rows, x.top, device=dev)
+    counts, scratch = torch.zeros(x.n, dtype=torch.int32, device=dev), bytes_of(1, _hip.moe_scratch_bytes(rows, x.n, x.top, x.ff, BF))[0]
+    shared = rnd(rows, blocks["moe"].beside) if x.shared else None
+    gate = torch.empty(rows, device=dev)
+    us = _graph_us([lambda i=i: _hip.moe(_hip.moe_desc(xc, router, rb, w1s[i], w2s[i], eo, ids, wts, gate, counts, scratch, shared))
+                    for i in range(n)])
+    name = f"{x.n} experts of {x.ff}, top {x.top}"
+    if decode:
+        out.append(_kernel_row(f"lr_moe ({name}; router, up, down)", us, "hbm", wbytes + 2 * rows * x.top * D))
+    else:
+        out.append(_kernel_row(f"lr_moe ({name})", us, "mfma", 6 * rows * x.top * x.ff * D))
+    del w1s, w2s
+    I = blocks["dense"].beside
+    n = copies(3 * I * D * 2)
+    w1s, w2s = [rnd(2 * I, D) for _ in range(n)], [rnd(D, I) for _ in range(n)]
+    act, h, d = torch.empty(rows, I, dtype=BF, device=dev), torch.empty(rows, 2 * I, dtype=BF, device=dev), torch.empty(rows, D, dtype=BF, device=dev)
+
+    def dense_ff(i):
+        _hip.linear_swiglu_out(xc, w1s[i], act, h)
+        _hip.linear(act, w2s[i], d)
+    us = _graph_us([lambda i=i: dense_ff(i) for i in range(n)])
+    out.append(_kernel_row(f"dense feed-forward of {I} (two launches)", us, "hbm" if decode else "mfma", 6 * I * D if decode else 6 * rows * I * D))
+    del w1s, w2s, act, h
+    # residual and norm
+    n = copies(rows * D * (12 + 2 * x.top))
+    xs, ds, es = ([rnd(rows, D, dt=torch.float32) for _ in range(n)], [rnd(rows, D) for _ in range(n)],
+                  [rnd(rows * x.top, D) for _ in range(n)])
+    one, g, b = rnd(1), rnd(D), rnd(D)
+    us = _graph_us([lambda i=i: _hip.residual_tanh(xs[i], ds[i], one, g, b, xs[i], xc) for i in range(n)])
+    out.append(_kernel_row("lr_residual_tanh", us, "hbm", rows * D * 12))
+    us = _graph_us([lambda i=i: _hip.residual_tanh(xs[i], ds[i], one, g, b, xs[i], xc, (es[i], wts)) for i in range(n)])
+    out.append(_kernel_row("lr_residual_tanh, experts' rows added", us, "hbm", rows * D * (12 + 2 * x.top)))
+    del xs, ds, es, xc
+    torch.cuda.empty_cache()
+    return out + [dict(r, kernel="lasivik: " + r["kernel"]) for r in mixer_kernels(lasivik, None, B, T, decode)]
 
 
 def mixer_kernels(hybrid, dense, B, T, decode):
@@ -321,6 +454,9 @@ def mixer_kernels(hybrid, dense, B, T, decode):
         keys = sum(min(i + 1, a.window) for i in range(T))
         out.append(_kernel_row(f"lr_window_attention ({a.heads} heads of {a.dim}, window {a.window})", us, "mfma",
                                B * a.heads * keys * 2 * (a.dim + a.vdim)))
+    if dense is None:
+        out.append(_residual_norm_row(hybrid.config.dim, rows, copies))
+        return out
     # the dense model's counterpart
     d = dense.config
     Hq, Hkv, hd = d.n_head_local, d.n_kv_local, d.head_dim
@@ -337,42 +473,45 @@ def mixer_kernels(hybrid, dense, B, T, decode):
         out.append(_kernel_row(f"dense: lr_attn_prefill ({Hq} / {Hkv} heads of {hd})", us, "mfma", B * Hq * (T * (T + 1) // 2) * 4 * hd))
     del kcs, vcs
     # the norms, a launch per sublayer in both
+    out.append(_residual_norm_row(hybrid.config.dim, rows, copies))
     D = hybrid.config.dim
     n = copies(rows * D * 12)
-    xs, ds = [rnd(rows, D, dt=torch.float32) for _ in range(n)], [rnd(rows, D) for _ in range(n)]
+    bs, ds = [rnd(rows, D) for _ in range(n)], [rnd(rows, D) for _ in range(n)]
     xc, gain = torch.empty(rows, D, dtype=BF, device=dev), rnd(D)
-    us = _graph_us([lambda i=i: _hip.residual_rmsnorm(xs[i], 2.0, ds[i], gain, xs[i], xc, 1e-5, gain_offset=1.0) for i in range(n)])
-    out.append(_kernel_row("lr_residual_rmsnorm (fp32 residual)", us, "hbm", rows * D * (4 + 2 + 4 + 2)))
-    bs = [rnd(rows, D) for _ in range(n)]
     us = _graph_us([lambda i=i: _hip.add_rmsnorm(bs[i], ds[i], None, gain, bs[i], xc, 1e-5) for i in range(n)])
     out.append(_kernel_row("dense: lr_add_rmsnorm", us, "hbm", rows * D * 8))
     torch.cuda.empty_cache()
     return out
 
 
+GEPOLIX_PAIRS = {"1b": ("gpt_gepolix:gepolix-1b", "gpt_lasivik:lasivik-1b"), "8b": ("gpt_gepolix:gepolix-8b", "gpt_lasivik:lasivik-8b")}
 LASIVIK_PAIRS = {"1b": ("gpt_lasivik:lasivik-1b", "gpt_dense:ladder-1b"), "8b": ("gpt_lasivik:lasivik-8b", "gpt_dense:ladder-8b")}
 
 
-def lasivik_compare(sizes, T=1792, K=32, W=5):
+def family_compare(workload, pairs, kernels, sizes, T=1792, K=32, W=5):
+    """Prefill and decode throughput of the models of each pair, and their kernels alone.  One JSON line."""
     import torch
 
     import benchmark as bm
     from gpt_fast import _hip
 
     _hip.load()
-    out = {"workload": "lasivik beside dense", "prompt_len": T, "data": "synthetic", "dtype": "bf16", "models": [], "kernels": []}
+    out = {"workload": workload, "prompt_len": T, "data": "synthetic", "dtype": "bf16", "models": [], "kernels": []}
     for size in sizes:
-        models = [bm._load_model(name, "cuda", torch.bfloat16, seed=0, verbose=False) for name in LASIVIK_PAIRS[size]]
+        models = [bm._load_model(name, "cuda", torch.bfloat16, seed=0, verbose=False) for name in pairs[size]]
         g = torch.Generator(device="cuda")
         g.manual_seed(1)
         prompt = torch.randint(0, 100000, (T,), device="cuda", generator=g)
-        for name, model in zip(LASIVIK_PAIRS[size], models):
+        for name, model in zip(pairs[size], models):
             model.last_logits_only = True
             row = {"model": name, "parameters": sum(p.numel() for p in model.parameters()), "prefill": [], "decode": []}
             count = sum(p.numel() for n, p in model.named_parameters() if p.dim() == 2 and not n.startswith(("tok_emb", "output")))
+            for x in (blk.experts for blk in model.layers if getattr(blk, "experts", None) is not None):
+                count += (x.w1.numel() + x.w2.numel()) * x.top // x.n
             for B in (1, 8):
                 model.max_seq_length = -1
                 model.setup_caches(B, T + 8)
+                print(f"{name}: prefill, batch {B}", file=sys.stderr, flush=True)
                 rows, pos = prompt.view(1, -1).repeat(B, 1), torch.arange(T, device="cuda", dtype=torch.int32)
                 bm.prefill(model, rows, pos, greedy=True)
                 torch.cuda.synchronize()
@@ -394,7 +533,8 @@ def lasivik_compare(sizes, T=1792, K=32, W=5):
             out["models"].append(row)
         for B, decode in ((1, False), (8, False), (1, True), (8, True), (32, True)):
             out["kernels"].append({"size": size, "batch": B, "phase": "decode" if decode else "prefill",
-                                   "rows": mixer_kernels(models[0], models[1], B, T, decode)})
+                                   "rows": kernels(models[0], models[1], B, T, decode)})
+            print(f"{size} kernels: batch {B}, {'decode' if decode else 'prefill'}", file=sys.stderr, flush=True)
         del models, model
         torch.cuda.empty_cache()
     print(json.dumps(out), flush=True)
@@ -418,6 +558,8 @@ def main():
                     help="weight-only e4m3 projections (gpt_fast.quantize): a profiling aid, not the headline")
     ap.add_argument("--lasivik", nargs="*", choices=sorted(LASIVIK_PAIRS), metavar="SIZE",
                     help="the Lasivik family beside the dense one instead of the headline (sizes 1b and 8b; default both)")
+    ap.add_argument("--gepolix", nargs="*", choices=sorted(GEPOLIX_PAIRS), metavar="SIZE",
+                    help="the Gepolix family beside the Lasivik one instead of the headline (sizes 1b and 8b; default both)")
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="also run a plain 1 GiB device copy (reads 1 GiB, writes 1 GiB) a few times: under "
                          "rocprofv3 --pmc its FETCH_SIZE / WRITE_SIZE readings calibrate the counters' unit")
@@ -434,7 +576,9 @@ def main():
 
     assert torch.cuda.is_available(), "bench.py needs the MI355X"
     if args.lasivik is not None:
-        return lasivik_compare(args.lasivik or sorted(LASIVIK_PAIRS))
+        return family_compare("lasivik beside dense", LASIVIK_PAIRS, mixer_kernels, args.lasivik or sorted(LASIVIK_PAIRS))
+    if args.gepolix is not None:
+        return family_compare("gepolix beside lasivik", GEPOLIX_PAIRS, gepolix_kernels, args.gepolix or sorted(GEPOLIX_PAIRS))
     _hip.load()
     dev = "cuda"
     B, T, K, W = args.batch, args.prompt, args.steps, args.warmup

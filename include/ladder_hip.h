@@ -578,8 +578,8 @@ int lr_window_decode(const void* q, int64_t ldq, const void* cache, const int32_
  * index among equals), weights[row, :] = softmax over those; out[row * top + k, :] = w2[e] (silu(gate) * up) with
  * [up; gate] = w1[e] x, e = experts[row, k].  x [rows, D] (row stride ldx), router [E (+ 1), D], w1 [E, 2 I, D],
  * w2 [E, D, I], out [rows * top, D].  shared != NULL: router has one more row, without a bias, and shared [rows, shared_cols]
- * (row stride ld_shared) is multiplied by the sigmoid of its product with x.  counts: [E] int32, zero before the first call
- * and left zero.  E <= 512, top <= 64. */
+ * (row stride ld_shared) is multiplied by the sigmoid of its product with x, which goes to gate [rows].  counts: [E] int32,
+ * zero before the first call and left zero.  E <= 512, top <= 64.  routed != 0: experts, weights and gate are there already. */
 typedef struct lr_moe {
   const void* x;
   int64_t ldx;
@@ -587,15 +587,19 @@ typedef struct lr_moe {
   void* out;
   int32_t* experts;
   float* weights;
+  float* gate;
   int32_t* counts;
   void* shared;
   int64_t ld_shared;
   void* scratch;
   size_t scratch_bytes;
-  int32_t rows, D, I, E, top, shared_cols, dtype;
+  int32_t rows, D, I, E, top, shared_cols, dtype, routed;
 } lr_moe_t;
-size_t lr_moe_scratch_bytes(int rows, int E, int top, int I, int shared, int dtype);
+size_t lr_moe_scratch_bytes(int rows, int E, int top, int I, int dtype);
 int lr_moe(const lr_moe_t* desc, lr_stream_t stream);
+/* lr_linear_multi and, beside it in the same launch, the routing of lr_moe (which is then called with routed != 0): M == rows
+ * <= 64 tokens, bf16.  The projections must not write what the routing reads. */
+int lr_linear_multi_route(const lr_projection_t* projections, int n_projections, int M, const lr_moe_t* desc, lr_stream_t stream);
 
 #ifdef __cplusplus
 }

@@ -495,14 +495,136 @@ static int gemm_grouped_as(const void* x, int64_t ldx, const void* w, void* y, i
       GemmRope{}, gp);
   return lr_launch_status();
 }
+// Grouped products in 128 x 128 tiles, for problems with few 256-row tiles: the loop of k_gemm with gathered rows, buffer
+// loads instead of branches and, in pair mode, a wave's 64 weight rows as 32 up rows followed by their gate rows.
+__global__ __launch_bounds__(256) void k_gemm_grouped(const u16* __restrict__ x, int64_t ldx, const u16* __restrict__ w, u16* __restrict__ y,
+                                                      int64_t ldy, int N, int K, int tn, int pair_off, const GemmGroup gp) {
+  __shared__ __attribute__((aligned(16))) u16 xs[2][BM * LDT];
+  __shared__ __attribute__((aligned(16))) u16 ws[2][BN * LDT];
+  __shared__ int32_t entry[BM];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int wm = wave >> 1, wn = wave & 1;
+  int mt, nt, M;
+  {
+    const int n = gridDim.x, xcd = blockIdx.x & 7, base = n >> 3, rem = n & 7;
+    const int id = xcd * base + (xcd < rem ? xcd : rem) + (blockIdx.x >> 3);
+    mt = id / tn;
+    nt = id - mt * tn;
+    if (mt >= gp.ntiles[0]) return;
+    const int32_t* tile = gp.tiles + 3 * mt;
+    w += tile[0] * gp.wstride;
+    M = tile[2];
+    if (tid < BM) entry[tid] = gp.entries[tile[1] + (tid < M ? tid : 0)];
+    __syncthreads();
+  }
+  const int n0 = nt * (pair_off ? BN / 2 : BN);
+  const __amdgpu_buffer_rsrc_t xres = __builtin_amdgcn_make_buffer_rsrc(const_cast<u16*>(x), 0, 0x7fffffff, 0x00020000);
+  const __amdgpu_buffer_rsrc_t wres = __builtin_amdgcn_make_buffer_rsrc(const_cast<u16*>(w + (int64_t)n0 * K), 0, 0x7fffffff, 0x00020000);
+  const int srow0 = tid >> 3, scol = (tid & 7) * 8;
+  int xoff[4], woff[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int r = srow0 + 32 * i;
+    xoff[i] = r < M ? (int)((int64_t)(entry[r] / gp.xdiv) * ldx * 2) : (int)0x80000000;
+    if (pair_off) {
+      const int pr = (r >> 6) * 32 + (r & 31);
+      woff[i] = n0 + pr < N ? (int)((int64_t)(((r >> 5) & 1) * pair_off + pr) * K * 2) : (int)0x80000000;
+    } else {
+      woff[i] = n0 + r < N ? r * K * 2 : (int)0x80000000;
+    }
+  }
+  uint4 xr[4], wr[4];
+  auto fetch = [&](int k) {
+    const bool in = k + scol < K;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const u32x4_t a = __builtin_amdgcn_raw_buffer_load_b128(xres, in && xoff[i] >= 0 ? xoff[i] + (k + scol) * 2 : (int)0x80000000, 0, 0);
+      const u32x4_t b = __builtin_amdgcn_raw_buffer_load_b128(wres, in && woff[i] >= 0 ? woff[i] + (k + scol) * 2 : (int)0x80000000, 0, 0);
+      xr[i] = make_uint4(a.x, a.y, a.z, a.w);
+      wr[i] = make_uint4(b.x, b.y, b.z, b.w);
+    }
+  };
+  auto stage = [&](int buf) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      st16(&xs[buf][(srow0 + 32 * i) * LDT + scol], xr[i]);
+      st16(&ws[buf][(srow0 + 32 * i) * LDT + scol], wr[i]);
+    }
+  };
+  f32x16_t acc[2][2];
+#pragma unroll
+  for (int a = 0; a < 2; ++a)
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int v = 0; v < 16; ++v) acc[a][b][v] = 0.0f;
+  const int nk = (K + BK - 1) / BK, arow = lane & 31, akq = (lane >> 5) * 8;
+  fetch(0);
+  stage(0);
+  __syncthreads();
+  for (int kt = 0; kt < nk; ++kt) {
+    const int cur = kt & 1;
+    if (kt + 1 < nk) fetch((kt + 1) * BK);
+#pragma unroll
+    for (int kk = 0; kk < BK; kk += 16) {
+      bf16x8_t af[2], bfr[2];
+#pragma unroll
+      for (int a = 0; a < 2; ++a) af[a] = *reinterpret_cast<const bf16x8_t*>(&xs[cur][(wm * 64 + a * 32 + arow) * LDT + kk + akq]);
+#pragma unroll
+      for (int b = 0; b < 2; ++b) bfr[b] = *reinterpret_cast<const bf16x8_t*>(&ws[cur][(wn * 64 + b * 32 + arow) * LDT + kk + akq]);
+#pragma unroll
+      for (int a = 0; a < 2; ++a)
+#pragma unroll
+        for (int b = 0; b < 2; ++b) acc[a][b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bfr[b], af[a], acc[a][b], 0, 0, 0);
+    }
+    if (kt + 1 < nk) stage(cur ^ 1);
+    __syncthreads();
+  }
+  // The products were W-tile x X-tile^T: accumulator element v of a 32 x 32 tile is output column (v / 4) * 8 + (lane / 32) * 4
+  // + v % 4 of row lane % 32.  Outputs leave through LDS (a piece per wave) as whole rows.
+  u16* eb = &xs[0][0] + wave * 64 * LDT;      // (2 BM LDT elements in all; the operand tiles are dead)
+  auto emit = [&](auto PAIR) {
+    constexpr bool P = decltype(PAIR)::value;
+    constexpr int WN = P ? 32 : 64, LPR = WN / 8, RPI = 64 / LPR;
+#pragma unroll
+    for (int a = 0; a < 2; ++a)
+#pragma unroll
+      for (int b = 0; b < (P ? 1 : 2); ++b)
+#pragma unroll
+        for (int g = 0; g < 4; ++g) {
+          float o[4];
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            o[e] = P ? swiglu_bf(round_bf(acc[a][0][4 * g + e]), round_bf(acc[a][1][4 * g + e])) : acc[a][b][4 * g + e];
+          *reinterpret_cast<uint2*>(&eb[(a * 32 + (lane & 31)) * LDT + b * 32 + g * 8 + (lane >> 5) * 4]) =
+              make_uint2(pack_bf2(o[0], o[1]), pack_bf2(o[2], o[3]));
+        }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");      // a wave reads back only what it wrote itself
+    const int cl = (lane % LPR) * 8, n = n0 + wn * WN + cl;
+#pragma unroll
+    for (int r0 = 0; r0 < 64; r0 += RPI) {
+      const int ml = r0 + lane / LPR, m = wm * 64 + ml;
+      if (m < M && n < N)      // (N and ldy are multiples of 8)
+        st16(y + (int64_t)entry[m] * ldy + n, *reinterpret_cast<const uint4*>(&eb[ml * LDT + cl]));
+    }
+  };
+  if (pair_off) emit(std::true_type{});
+  else emit(std::false_type{});
+}
+
+// tile_rows: 128 or 256, the height the tile table was made for
 int gemm_grouped(const void* x, int64_t ldx, int64_t xrows, const void* w, void* y, int64_t ldy, int N, int K, int pair_off, int64_t wstride,
-                 const int32_t* tiles, const int32_t* ntiles, const int32_t* entries, int xdiv, int max_tiles, hipStream_t s) {
+                 const int32_t* tiles, const int32_t* ntiles, const int32_t* entries, int xdiv, int max_tiles, int tile_rows, hipStream_t s) {
   if (xrows * ldx * 2 >= 0x7fffffff || ((int64_t)pair_off + GN) * K * 2 >= 0x7fffffff) return LR_E_UNSUPPORTED;
   const GemmGroup gp = {tiles, ntiles, entries, xdiv, wstride};
+  if (tile_rows == BM) {
+    const int gn = pair_off ? BN / 2 : BN, tn = (N + gn - 1) / gn;
+    k_gemm_grouped<<<dim3((unsigned)(max_tiles * tn)), dim3(256), 0, s>>>((const u16*)x, ldx, (const u16*)w, (u16*)y, ldy, N, K, tn, pair_off, gp);
+    return lr_launch_status();
+  }
   return K % BK ? gemm_grouped_as<true>(x, ldx, w, y, ldy, N, K, pair_off, gp, max_tiles, s)
                 : gemm_grouped_as<false>(x, ldx, w, y, ldy, N, K, pair_off, gp, max_tiles, s);
 }
-int gemm_grouped_rows() { return GM; }
 }  // namespace lr_detail
 
 extern "C" int lr_linear_tuned(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy, int M, int N, int K,

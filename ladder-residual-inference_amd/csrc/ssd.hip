@@ -319,7 +319,7 @@ __device__ __forceinline__ void split8(const float* f, bf16x8_t& hi, bf16x8_t& l
 
 // NT: N in tiles of 16.  state_only: no outputs; the segment starts from zero and leaves its state and log-decay in scratch.
 template <int NT>
-__global__ __launch_bounds__(256) void k_ssd_chunk(const Ssd a, const int state_only) {
+__global__ __launch_bounds__(256, NT > 8 ? 1 : 2) void k_ssd_chunk(const Ssd a, const int state_only) {
   constexpr int NR = 16 * NT + 8, KN = NT / 2, NW = NT >= 4 ? NT / 4 : 1;   // NW: tiles of N per wave in the state update
   extern __shared__ __attribute__((aligned(16))) u16 su[];
   u16* Bs = su;                       // [CK][NR]       B by token
@@ -384,8 +384,9 @@ __global__ __launch_bounds__(256) void k_ssd_chunk(const Ssd a, const int state_
   // ---- staging: an item is eight columns of two neighbouring tokens, 32 pairs of tokens side by side
   constexpr int BI = NT / 4 > 0 ? NT / 4 : 1;        // items of B per thread (NT * 2 slices of 8, 32 pairs, 256 threads)
   const int kp = tid & 31, sl = tid >> 5;            // pair, slice (8 of them at once)
-  u32x4_t br[BI][2], xr[2];
+  u32x4_t br[BI][2], xr[2], cr[KN];
   float draw = 0.0f;
+  const int t = 16 * wave + l16;        // this lane's token in the products
   auto fetch = [&](int c0) {
     const int nt = min(len - c0, CK);
     const rsrc_t rb = buffer_of(B + (int64_t)c0 * a.ldu, (nt - 1) * lb + N * 2);
@@ -399,6 +400,12 @@ __global__ __launch_bounds__(256) void k_ssd_chunk(const Ssd a, const int state_
         br[i][e] = __builtin_amdgcn_raw_buffer_load_b128(rb, t < nt && c < N ? t * lb + c * 2 : NOWHERE, 0, 0);
       }
       xr[e] = __builtin_amdgcn_raw_buffer_load_b128(rx, t < nt && sl * 8 < pw ? t * lb + sl * 16 : NOWHERE, 0, 0);
+    }
+    if (!state_only) {
+      const rsrc_t rc = buffer_of(C + (int64_t)c0 * a.ldu, (nt - 1) * lb + N * 2);
+#pragma unroll
+      for (int k = 0; k < KN; ++k)
+        cr[k] = __builtin_amdgcn_raw_buffer_load_b128(rc, t < nt && 32 * k + 8 * g4 < N ? t * lb + (32 * k + 8 * g4) * 2 : NOWHERE, 0, 0);
     }
     if (wave == 0) {
       const u16 r = dt[(int64_t)(c0 + min(lane, nt - 1)) * a.ld];
@@ -458,18 +465,13 @@ __global__ __launch_bounds__(256) void k_ssd_chunk(const Ssd a, const int state_
   for (int c0 = 0; c0 < len; c0 += CK, buf ^= 1) {
     const int nt = min(len - c0, CK);
     const bool more = c0 + CK < len;
-    const int t = 16 * wave + l16;        // this lane's token in the products
     const float* cm = cum + buf * CK;
     const float* dm = dts + buf * CK;
     bf16x8_t cf[KN];
     uint2 zr[4], xq[4];
     if (!state_only) {
-      const rsrc_t rc = buffer_of(C + (int64_t)c0 * a.ldu, (nt - 1) * lb + N * 2);
 #pragma unroll
-      for (int k = 0; k < KN; ++k) {
-        const int c = 32 * k + 8 * g4;
-        cf[k] = __builtin_bit_cast(bf16x8_t, __builtin_amdgcn_raw_buffer_load_b128(rc, t < nt && c < N ? t * lb + c * 2 : NOWHERE, 0, 0));
-      }
+      for (int k = 0; k < KN; ++k) cf[k] = __builtin_bit_cast(bf16x8_t, cr[k]);
       const rsrc_t rz = buffer_of(z + (int64_t)c0 * a.ld, (nt - 1) * lz + pw * 2);
       const rsrc_t rx = buffer_of(x + (int64_t)c0 * a.ldu, (nt - 1) * lb + pw * 2);
 #pragma unroll
@@ -492,22 +494,29 @@ __global__ __launch_bounds__(256) void k_ssd_chunk(const Ssd a, const int state_
 #pragma unroll
       for (int n = 0; n < 4; ++n) {
         o[n] = f32x4_t{0, 0, 0, 0};
-        if (n < pt) {
+      }
+      // (columns beyond P are zeros: computed, not stored)
 #pragma unroll
-          for (int k = 0; k < KN; ++k) {
-            const bf16x8_t sh = *reinterpret_cast<const bf16x8_t*>(&Sh[(16 * n + l16) * NR + 32 * k + 8 * g4]);
-            const bf16x8_t sv = *reinterpret_cast<const bf16x8_t*>(&Sl[(16 * n + l16) * NR + 32 * k + 8 * g4]);
-            o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh, cf[k], o[n], 0, 0, 0);
-            o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sv, cf[k], o[n], 0, 0, 0);
-          }
-          o[n] *= et;
+      for (int k = 0; k < KN; ++k) {
+#pragma unroll
+        for (int n = 0; n < 4; ++n) {
+          const bf16x8_t sh = *reinterpret_cast<const bf16x8_t*>(&Sh[(16 * n + l16) * NR + 32 * k + 8 * g4]);
+          o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh, cf[k], o[n], 0, 0, 0);
+        }
+#pragma unroll
+        for (int n = 0; n < 4; ++n) {
+          const bf16x8_t sv = *reinterpret_cast<const bf16x8_t*>(&Sl[(16 * n + l16) * NR + 32 * k + 8 * g4]);
+          o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sv, cf[k], o[n], 0, 0, 0);
         }
       }
+#pragma unroll
+      for (int n = 0; n < 4; ++n) o[n] *= et;
       // ---- the chunk's own tokens, 32 keys at a time
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         if (2 * j <= wave) {
           float m[8];
+          const int tl = fresh(t) - 4 * g4;       // (compared here: as loop invariants the masks would not fit the scalar registers)
 #pragma unroll
           for (int e = 0; e < 2; ++e) {
             const int st = 2 * j + e;
@@ -525,22 +534,20 @@ __global__ __launch_bounds__(256) void k_ssd_chunk(const Ssd a, const int state_
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
               const float w = exp2_f(ct - cc[i]) * dd[i];
-              m[4 * e + i] = st <= wave && 16 * st + 4 * g4 + i <= t ? gt[i] * w : 0.0f;
+              m[4 * e + i] = 16 * st + i <= tl ? gt[i] * w : 0.0f;
             }
           }
           bf16x8_t mh, ml;
           split8(m, mh, ml);
 #pragma unroll
           for (int n = 0; n < 4; ++n) {
-            if (n < pt) {
-              // tokens 32 j + 4 g4 + {0 .. 3} and 16 further
-              const int r = 16 * n + l16;
-              const uint2 v0 = *reinterpret_cast<const uint2*>(&Xt[r * TR + 8 * turn(4 * j + (g4 >> 1), r) + 4 * (g4 & 1)]);
-              const uint2 v1 = *reinterpret_cast<const uint2*>(&Xt[r * TR + 8 * turn(4 * j + 2 + (g4 >> 1), r) + 4 * (g4 & 1)]);
-              const bf16x8_t xv = __builtin_bit_cast(bf16x8_t, u32x4_t{v0.x, v0.y, v1.x, v1.y});
-              o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xv, mh, o[n], 0, 0, 0);
-              o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xv, ml, o[n], 0, 0, 0);
-            }
+            // tokens 32 j + 4 g4 + {0 .. 3} and 16 further
+            const int r = 16 * n + l16;
+            const uint2 v0 = *reinterpret_cast<const uint2*>(&Xt[r * TR + 8 * turn(4 * j + (g4 >> 1), r) + 4 * (g4 & 1)]);
+            const uint2 v1 = *reinterpret_cast<const uint2*>(&Xt[r * TR + 8 * turn(4 * j + 2 + (g4 >> 1), r) + 4 * (g4 & 1)]);
+            const bf16x8_t xv = __builtin_bit_cast(bf16x8_t, u32x4_t{v0.x, v0.y, v1.x, v1.y});
+            o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xv, mh, o[n], 0, 0, 0);
+            o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xv, ml, o[n], 0, 0, 0);
           }
         }
       }
@@ -591,12 +598,9 @@ __global__ __launch_bounds__(256) void k_ssd_chunk(const Ssd a, const int state_
           bf16x8_t bh_, bl;
           split8(f, bh_, bl);
 #pragma unroll
-          for (int n = 0; n < 4; ++n) {
-            if (n < pt) {
-              S[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bh_, xv[n], S[m][n], 0, 0, 0);
-              S[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bl, xv[n], S[m][n], 0, 0, 0);
-            }
-          }
+          for (int n = 0; n < 4; ++n) S[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bh_, xv[n], S[m][n], 0, 0, 0);
+#pragma unroll
+          for (int n = 0; n < 4; ++n) S[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bl, xv[n], S[m][n], 0, 0, 0);
         }
       }
     }
@@ -613,13 +617,14 @@ __global__ __launch_bounds__(256) void k_ssd_chunk(const Ssd a, const int state_
   if (state_only) dst = a.seg_state + ((int64_t)bh * a.nseg + seg + 1) * N * P;
   else if (seg == a.nseg - 1) dst = a.state + (int64_t)bh * N * P;
   if (dst && mine) {
+    const int g4_ = fresh(g4);        // (the masks are formed here, not kept since the state was read)
 #pragma unroll
     for (int m = 0; m < NW; ++m)
 #pragma unroll
       for (int n = 0; n < 4; ++n)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const int r = 16 * (NW * wave + m) + 4 * g4 + i;
+          const int r = 16 * (NW * wave + m) + 4 * g4_ + i;
           if (r < N && n < pt) dst[(int64_t)r * P + pc + 16 * n + l16] = S[m][n][i];
         }
   }

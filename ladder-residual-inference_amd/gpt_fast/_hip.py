@@ -92,8 +92,9 @@ _PROTOS = {
     "lr_window_decode_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
     "lr_window_decode": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_int, c_int, c_int,
                                  c_int, c_int, c_float, c_void_p, c_size_t, c_void_p]),
-    "lr_moe_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
+    "lr_moe_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int]),
     "lr_moe": (c_int, [c_void_p, c_void_p]),
+    "lr_linear_multi_route": (c_int, [c_void_p, c_int, c_int, c_void_p, c_void_p]),
 }
 
 
@@ -918,18 +919,19 @@ def window_decode(q, cache, y, pos, scratch, B, H, G, dk, dv, window: int, scale
 
 class _Moe(ctypes.Structure):   # lr_moe_t
     _fields_ = [("x", c_void_p), ("ldx", c_int64)] + \
-               [(n, c_void_p) for n in ("router", "router_bias", "w1", "w2", "out", "experts", "weights", "counts", "shared")] + \
+               [(n, c_void_p) for n in ("router", "router_bias", "w1", "w2", "out", "experts", "weights", "gate", "counts", "shared")] + \
                [("ld_shared", c_int64), ("scratch", c_void_p), ("scratch_bytes", c_size_t)] + \
-               [(n, c_int32) for n in ("rows", "D", "I", "E", "top", "shared_cols", "dtype")]
+               [(n, c_int32) for n in ("rows", "D", "I", "E", "top", "shared_cols", "dtype", "routed")]
 
 
-def moe_scratch_bytes(rows, E, top, I, shared: bool, dtype) -> int:
-    return int(load().lr_moe_scratch_bytes(rows, E, top, I, int(shared), _DTYPES[dtype]))
+def moe_scratch_bytes(rows, E, top, I, dtype) -> int:
+    return int(load().lr_moe_scratch_bytes(rows, E, top, I, _DTYPES[dtype]))
 
 
-def moe(x, router, router_bias, w1, w2, out, experts, weights, counts, scratch, shared=None):
-    """Mixture of experts (lr_moe): out [rows * top, D] a row per choice, experts / weights [rows, top] the choices.  `shared`: a
-    shared expert's activations [rows, cols], multiplied in place by the sigmoid of their gate (the router's last row)."""
+def moe_desc(x, router, router_bias, w1, w2, out, experts, weights, gate, counts, scratch, shared=None):
+    """A mixture of experts for moe() and linear_multi_route(): out [rows * top, D] a row per choice, experts / weights [rows, top]
+    the choices.  `shared`: a shared expert's activations [rows, cols], multiplied in place by the sigmoid of their gate (the
+    router's last row)."""
     rows, D, ldx = _rows_ld(x)
     E, two_i, Dw = w1.shape
     top = weights.shape[1]
@@ -939,18 +941,31 @@ def moe(x, router, router_bias, w1, w2, out, experts, weights, counts, scratch, 
     for t in (router, router_bias, w1, w2, out, experts, weights, counts):
         assert t.is_contiguous()
     assert out.numel() == rows * top * D and tuple(experts.shape) == tuple(weights.shape) == (rows, top)
-    assert counts.numel() == E and counts.dtype == experts.dtype == torch.int32
+    assert counts.numel() == E and counts.dtype == experts.dtype == torch.int32 and gate.numel() >= rows
     sp, lds, sc = None, 0, 0
     if shared is not None:
         srows, sc, lds = _rows_ld(shared)
         assert srows == rows
         sp = _dev(shared, dt)
-    d = _Moe(x=_dev(x, dt), ldx=ldx, router=_dev(router, dt), router_bias=_dev(router_bias, dt), w1=_dev(w1, dt), w2=_dev(w2, dt),
-             out=_dev(out, dt), experts=experts.data_ptr(), weights=_dev(weights, torch.float32), counts=counts.data_ptr(), shared=sp,
-             ld_shared=lds, scratch=scratch.data_ptr(), scratch_bytes=scratch.numel() * scratch.element_size(), rows=rows, D=D,
-             I=two_i // 2, E=E, top=top, shared_cols=sc, dtype=_DTYPES[dt])
-    _check(load().lr_moe(ctypes.byref(d), _stream()), "lr_moe")
-    return out
+    return _Moe(x=_dev(x, dt), ldx=ldx, router=_dev(router, dt), router_bias=_dev(router_bias, dt), w1=_dev(w1, dt), w2=_dev(w2, dt),
+                out=_dev(out, dt), experts=experts.data_ptr(), weights=_dev(weights, torch.float32), gate=_dev(gate, torch.float32),
+                counts=counts.data_ptr(), shared=sp,
+                ld_shared=lds, scratch=scratch.data_ptr(), scratch_bytes=scratch.numel() * scratch.element_size(), rows=rows, D=D,
+                I=two_i // 2, E=E, top=top, shared_cols=sc, dtype=_DTYPES[dt], routed=0)
+
+
+def linear_multi_route(desc, *projections):
+    """linear_multi(*projections) and the routing of `desc` in one launch; up to 64 rows."""
+    arr, M, _keep = _projection_array(projections)
+    assert M == desc.rows
+    _check(load().lr_linear_multi_route(ctypes.cast(arr, c_void_p), len(projections), M, ctypes.byref(desc), _stream()),
+           "lr_linear_multi_route")
+    desc.routed = 1
+
+
+def moe(desc):
+    """The experts' rows of `desc` (lr_moe), routed first unless linear_multi_route has done so."""
+    _check(load().lr_moe(ctypes.byref(desc), _stream()), "lr_moe")
 
 
 def _ladder_model_desc(model, attention_workgroups: int = 0):

@@ -40,8 +40,9 @@ class ParallelWorkspace(HybridWorkspace):
             top = max(m.top for m in mix)
             self._expert_out = e(rows * top * model.config.dim)
             self._expert_ids, self._expert_weights = e(rows * top, dt=torch.int32), e(rows * top, dt=torch.float32)
+            self._gate = e(rows, dt=torch.float32)
             self._counts = torch.zeros(max(m.n for m in mix), dtype=torch.int32, device=device)
-            self._expert_scratch = e(max(_hip.moe_scratch_bytes(rows, m.n, m.top, m.ff, m.shared, dtype) for m in mix), dt=torch.uint8)
+            self._expert_scratch = e(max(_hip.moe_scratch_bytes(rows, m.n, m.top, m.ff, dtype) for m in mix), dt=torch.uint8)
 
     def joint(self, blk):
         """(both, mixer's columns, feed-forward's columns)"""
@@ -51,7 +52,7 @@ class ParallelWorkspace(HybridWorkspace):
     def expert_buffers(self, m: Experts, dim: int):
         n = self.rows * m.top
         return (self._expert_out[:n * dim].view(n, dim), self._expert_ids[:n].view(self.rows, m.top),
-                self._expert_weights[:n].view(self.rows, m.top), self._counts[:m.n], self._expert_scratch)
+                self._expert_weights[:n].view(self.rows, m.top), self._gate, self._counts[:m.n], self._expert_scratch)
 
 
 class ParallelBlock(nn.Module):
@@ -100,19 +101,32 @@ class GPTGepolix(GPTHybrid):
         norms = [blk.norm for blk in self.layers[1:]] + [self.norm]
         for blk, following in zip(self.layers, norms):
             both, y, act = ws.joint(blk)
-            proj = self._project_in(ws, blk, act)
+            m, experts, routed = blk.experts, None, None
+            if m is not None:
+                buffers = ws.expert_buffers(m, self.config.dim)
+                routed, experts = m.on(ws.xc, act if m.shared else None, *buffers), (buffers[0], buffers[2])
+            proj = self._project_in(ws, blk, act, routed)
             blk.mixer.mix(ws, pos, proj, y)
-            experts = None
-            if blk.experts is not None:
-                experts = blk.experts.run(ws.xc, act if blk.experts.shared else None, *ws.expert_buffers(blk.experts, self.config.dim))
+            if m is not None:
+                _hip.moe(routed)
             project(both, blk.mixer.out_proj, ws.d)
             following.into(ws.x, ws.d, ws.x, ws.xc, experts)
         return None, None
 
-    def _project_in(self, ws, blk, act):
-        """The mixer's projections of ws.xc; the feed-forward's activations into `act`."""
+    def _project_in(self, ws, blk, act, routed):
+        """The mixer's projections of ws.xc; the feed-forward's activations into `act`.  A decode batch takes one launch, routing
+        included."""
         proj = ws.proj[:, :blk.mixer.proj_cols]
         w = blk.mixer.in_proj.weight
+        if ws.xc.dtype == torch.bfloat16 and ws.rows <= 64:
+            todo = [(ws.xc, w, proj, _hip.EPI_NONE)]
+            if blk.w1 is not None:
+                todo.append((ws.xc, blk.w1.weight, act, _hip.EPI_SWIGLU))
+            if routed is not None:
+                _hip.linear_multi_route(routed, *todo)
+            else:
+                _hip.linear_multi(*todo)
+            return proj
         if blk.w1 is None:
             return project(ws.xc, blk.mixer.in_proj, proj)
         h = ws.h[:ws.rows * 2 * blk.beside].view(ws.rows, -1)
@@ -120,8 +134,6 @@ class GPTGepolix(GPTHybrid):
             _hip.linear(ws.xc, blk.w1.weight, h)
             _hip.swiglu(h, act)
             _hip.linear(ws.xc, w, proj)
-        elif 2 <= ws.rows <= 64:
-            _hip.linear_multi((ws.xc, w, proj, _hip.EPI_NONE), (ws.xc, blk.w1.weight, act, _hip.EPI_SWIGLU))
         else:
             _hip.linear_swiglu_out(ws.xc, blk.w1.weight, act, h)
             _hip.linear(ws.xc, w, proj)

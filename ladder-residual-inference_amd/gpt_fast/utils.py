@@ -95,11 +95,11 @@ class Experts(nn.Module):
         self.w1 = nn.Parameter(torch.zeros(n, 2 * ff, dim))
         self.w2 = nn.Parameter(torch.zeros(n, dim, ff))
 
-    def run(self, x: Tensor, shared_act: Optional[Tensor], out: Tensor, ids: Tensor, weights: Tensor, counts: Tensor, scratch: Tensor):
-        """A row per (token, choice) into `out`; shared_act (a shared expert's activations) times its gate.  Returns what
-        residual_tanh adds up."""
-        _hip.moe(x, self.router, self.router_bias, self.w1, self.w2, out, ids, weights, counts, scratch, shared_act)
-        return out, weights
+    def on(self, x: Tensor, shared_act: Optional[Tensor], out: Tensor, ids: Tensor, weights: Tensor, gate: Tensor, counts: Tensor,
+           scratch: Tensor):
+        """What _hip.moe and _hip.linear_multi_route work on: a row per (token, choice) into `out`; shared_act (a shared expert's
+        activations) times its gate."""
+        return _hip.moe_desc(x, self.router, self.router_bias, self.w1, self.w2, out, ids, weights, gate, counts, scratch, shared_act)
 
 
 def apply_rope_scaling(freqs: torch.Tensor, rope_scaling: dict) -> torch.Tensor:
