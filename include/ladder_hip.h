@@ -579,7 +579,7 @@ int lr_window_decode(const void* q, int64_t ldq, const void* cache, const int32_
  * [up; gate] = w1[e] x, e = experts[row, k].  x [rows, D] (row stride ldx), router [E (+ 1), D], w1 [E, 2 I, D],
  * w2 [E, D, I], out [rows * top, D].  shared != NULL: router has one more row, without a bias, and shared [rows, shared_cols]
  * (row stride ld_shared) is multiplied by the sigmoid of its product with x, which goes to gate [rows].  counts: [E] int32,
- * zero before the first call and left zero.  E <= 512, top <= 64.  routed != 0: experts, weights and gate are there already. */
+ * zero before the first call and left zero.  E <= 512.  routed != 0: experts, weights and gate are there already. */
 typedef struct lr_moe {
   const void* x;
   int64_t ldx;

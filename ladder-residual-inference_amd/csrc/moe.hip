@@ -98,12 +98,13 @@ __device__ __forceinline__ void route_rows(const Router& a, const int block, flo
   }
   __syncthreads();
   for (int r = wave; r < nr; r += NW) {
-    const float* z = logits + r * n;
+    float* z = logits + r * n;       // (a row is one wave's: the weights take the place of the logits as they are taken out)
     float v[EPL];
 #pragma unroll
     for (int i = 0; i < EPL; ++i) v[i] = lane + 64 * i < E ? z[lane + 64 * i] : -INFINITY;
-    float first = 0.0f, sum = 0.0f, mine = 0.0f;
-    int id = 0;
+    asm volatile("" ::: "memory");
+    float first = 0.0f, sum = 0.0f;
+    int32_t* ids = a.experts + (int64_t)(r0 + r) * a.top;
     for (int k = 0; k < a.top; ++k) {
       float m = v[0];
 #pragma unroll
@@ -124,12 +125,13 @@ __device__ __forceinline__ void route_rows(const Router& a, const int block, flo
       if (k == 0) first = m;
       const float w = expf(m - first);
       sum += w;
-      if (lane == k) { mine = w; id = at < 0 ? 0 : at; }      // (at < 0: logits that are no numbers)
+      if (lane == 0) {
+        z[k] = w;
+        ids[k] = at < 0 ? 0 : at;      // (at < 0: logits that are no numbers)
+      }
     }
-    if (lane < a.top) {
-      a.experts[(int64_t)(r0 + r) * a.top + lane] = id;
-      a.weights[(int64_t)(r0 + r) * a.top + lane] = mine / sum;
-    }
+    asm volatile("" ::: "memory");     // (a wave's LDS accesses complete in order)
+    for (int k = lane; k < a.top; k += 64) a.weights[(int64_t)(r0 + r) * a.top + k] = z[k] / sum;
     if (n > E && lane == 0) a.gate[r0 + r] = 1.0f / (1.0f + expf(-z[E]));
   }
 }
@@ -334,8 +336,8 @@ int launch_band(const Proj& p, int64_t wstride, const int32_t* experts, int n, i
   return lr_launch_status();
 }
 
-constexpr int BAND_ROWS = 64;         // tokens up to which the bands are taken
-bool by_bands(int rows, int dtype) { return dtype == LR_BF16 && rows <= BAND_ROWS; }
+constexpr int BAND_ROWS = 64, BAND_LIST = 4096;      // tokens and entries up to which the bands are taken
+bool by_bands(int rows, int top, int dtype) { return dtype == LR_BF16 && rows <= BAND_ROWS && (int64_t)rows * top <= BAND_LIST; }
 
 // Height of the grouped tiles: 256 rows where that still makes a tile for most CUs in both products.
 int tile_rows(int rows, int E, int top, int I, int D, int dtype) {
@@ -399,7 +401,7 @@ Layout layout(int rows, int E, int top, int I, int dtype) {
   Layout l;
   l.h = align16(n * I * es);
   l.ints = l.h + (dtype == LR_F32 ? align16(n * 2 * I * es) : 0);
-  l.total = l.ints + (by_bands(rows, dtype) ? 0 : align16(sizeof(int32_t) * ((size_t)E + 4 + 3 * (size_t)max_tiles(rows, E, top, 64) + n)));
+  l.total = l.ints + (by_bands(rows, top, dtype) ? 0 : align16(sizeof(int32_t) * ((size_t)E + 4 + 3 * (size_t)max_tiles(rows, E, top, 64) + n)));
   return l;
 }
 
@@ -425,7 +427,7 @@ static int check_moe(const lr_moe_t* d) {
   if (d->rows <= 0 || d->D <= 0 || d->E <= 0 || d->top <= 0 || d->top > d->E || d->I <= 0 || d->ldx < d->D) return LR_E_SHAPE;
   if (d->shared && (d->shared_cols <= 0 || d->ld_shared < d->shared_cols)) return LR_E_SHAPE;
   if (d->D % 8 || d->I % 8 || d->ldx % 8 || (d->shared && (d->ld_shared % 8 || d->shared_cols % 8))) return LR_E_ALIGN;
-  if (d->E > 64 * EPL || d->top > 64 || (int64_t)d->rows * d->top > (1 << 28)) return LR_E_UNSUPPORTED;
+  if (d->E > 64 * EPL || (int64_t)d->rows * d->top > (1 << 28)) return LR_E_UNSUPPORTED;
   return d->scratch_bytes < layout(d->rows, d->E, d->top, d->I, d->dtype).total ? LR_E_SHAPE : LR_OK;
 }
 
@@ -461,12 +463,12 @@ extern "C" int lr_moe(const lr_moe_t* d, lr_stream_t stream) {
     rc = d->dtype == LR_F32 ? route<float>(d, s) : route<u16>(d, s);
     if (rc != LR_OK) return rc;
   }
-  if (d->shared && !by_bands(d->rows, d->dtype)) {
+  if (d->shared && !by_bands(d->rows, d->top, d->dtype)) {
     rc = d->dtype == LR_F32 ? gate<float>(d, s) : gate<u16>(d, s);
     if (rc != LR_OK) return rc;
   }
 
-  if (by_bands(d->rows, d->dtype)) {
+  if (by_bands(d->rows, d->top, d->dtype)) {
     if ((int64_t)d->rows * d->ldx * 2 >= 0x7fffffff || (int64_t)n * I * 2 >= 0x7fffffff || ((int64_t)I + 64) * D * 2 >= 0x7fffffff)
       return LR_E_UNSUPPORTED;
     const bool by_slot = d->rows == 1;
