@@ -520,6 +520,12 @@ int lr_residual_tanh(const float* x, const void* d, const void* expert_out, cons
                      const void* alpha, const void* gain, const void* bias, float* x_out, void* x_compute, int rows, int dim,
                      int dtype, lr_stream_t stream);
 
+/* lr_residual_tanh with d = x w^T, up to 64 rows, in the product's launch: resid [M, N] += x w^T (+ the experts' weighted rows,
+ * [M * top, N]), fp32 throughout; x_compute [M, N] = tanh(alpha * resid) * gain + bias.  bf16. */
+int lr_linear_residual_tanh(const void* x, int64_t ldx, const void* w, int M, int N, int K, float* resid, const void* expert_out,
+                            const float* expert_weights, int top, const void* alpha, const void* gain, const void* bias,
+                            void* x_compute, lr_stream_t stream);
+
 /* Causal convolution per channel and silu over S consecutive tokens per sequence: out[t, c] =
  * silu(bias[c] + sum_j w[c, j] u[t - (taps - 1) + j, c]).  u [B*S, C] (row stride ldu), w [C, taps] (the last column is the
  * current token's), out [B*S, C] (row stride ldo; not u).  ring [Bmax, taps, C] holds a sequence's last inputs, a token's at

@@ -68,10 +68,19 @@ constexpr size_t stream_band_lds_bytes() {
 // 256 bytes, now 256 elements of K, which are expanded to bf16 (exactly: e4m3 is a subset of bf16) on their way
 // into the LDS piece; the sum is rounded to bf16, multiplied by the row's scale and rounded again, as
 // F.linear(x, w.to(bf16)) * scales does, before the epilogue sees it.
+// RESID: nothing is stored to y; the sums, and a token's experts' weighted rows if there are any, are added to the fp32 residual,
+// whose scaled tanh (lr_residual_tanh) goes out as the next layer's input.
+struct BandResidual {
+  float* x;                              // [M, N]
+  u16* xc;                               // [M, N]
+  const u16 *alpha, *gain, *bias, *eo;   // eo [M * top, N] or nullptr
+  const float* ew;                       // [M, top]
+  int top;
+};
 // GATHER: input row m is row rows[m] / xdiv of x, output row m is row rows[m] of y (`rows`: M of them, in LDS).
-template <int MT, int UNITS, bool W8 = false, bool XL = (MT >= XLDS_MIN_MT), bool GATHER = false>
+template <int MT, int UNITS, bool W8 = false, bool XL = (MT >= XLDS_MIN_MT), bool GATHER = false, bool RESID = false>
 __device__ __forceinline__ void stream_band(const Proj& p, const int M, const int band, u16* sg_smem,
-                                            const int32_t* rows = nullptr, const int xdiv = 1) {
+                                            const int32_t* rows = nullptr, const int xdiv = 1, const BandResidual rs = {}) {
   static_assert(!W8 || MT == 16, "the e4m3 path is built for up to 16 input rows");
   constexpr int KCW = W8 ? 256 : 128;  // k elements per chunk
   constexpr int LRW = KCW + 8;         // LDS row length in elements
@@ -344,7 +353,19 @@ __device__ __forceinline__ void stream_band(const Proj& p, const int M, const in
     float s0 = 0.0f, s1 = 0.0f;
 #pragma unroll
     for (int wv = 0; wv < NWV; ++wv) s0 += red[wv * WSTRIDE + ((u * MTILES + mt) * 4 + e) * 64 + ln];
-    if (pair_off) {
+    if constexpr (RESID) {
+      const int n = n0 + r;
+      const int64_t at = (int64_t)m * N + n;
+      float v = rs.x[at] + s0;
+      if (rs.eo) {
+        float t = 0.0f;
+#pragma unroll 4
+        for (int k = 0; k < rs.top; ++k) t = fmaf(rs.ew[m * rs.top + k], bf_to_f(rs.eo[((int64_t)m * rs.top + k) * N + n]), t);
+        v += t;
+      }
+      rs.x[at] = v;
+      rs.xc[at] = f_to_bf(fmaf(tanhf(bf_to_f(rs.alpha[0]) * v), bf_to_f(rs.gain[n]), bf_to_f(rs.bias[n])));
+    } else if (pair_off) {
       if (UNITS == 2) {
 #pragma unroll
         for (int wv = 0; wv < NWV; ++wv) s1 += red[wv * WSTRIDE + ((MTILES + mt) * 4 + e) * 64 + ln];

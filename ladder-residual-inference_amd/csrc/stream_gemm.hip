@@ -80,6 +80,55 @@ extern "C" int lr_linear_multi(const lr_projection_t* proj, int n_proj, int M, l
   return rc != LR_OK ? rc : lr_launch_status();
 }
 
+namespace {
+
+template <int MT, int UNITS, bool XL>
+__global__ __launch_bounds__(NWV * 64) void k_stream_residual(const Proj p, const int M, const BandResidual rs) {
+  extern __shared__ __attribute__((aligned(16))) u16 sg_smem[];
+  stream_band<MT, UNITS, false, XL, false, true>(p, M, blockIdx.x, sg_smem, nullptr, 1, rs);
+}
+
+template <int MT, int UNITS, bool XL>
+int launch_residual_units(const Proj& p, int M, const BandResidual& rs, hipStream_t s) {
+  constexpr size_t lds = stream_band_lds_bytes<MT, UNITS, false, XL>();
+  static std::atomic<unsigned long long> raised{0};
+  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_stream_residual<MT, UNITS, XL>), lds, raised)) return LR_E_LAUNCH;
+  k_stream_residual<MT, UNITS, XL><<<dim3((unsigned)p.nwg), dim3(NWV * 64), lds, s>>>(p, M, rs);
+  return lr_launch_status();
+}
+template <int MT, bool XL>
+int launch_residual(const Proj& p, int M, int units, const BandResidual& rs, hipStream_t s) {
+  return units == 2 ? launch_residual_units<MT, 2, XL>(p, M, rs, s) : launch_residual_units<MT, 1, XL>(p, M, rs, s);
+}
+
+}  // namespace
+
+extern "C" int lr_linear_residual_tanh(const void* x, int64_t ldx, const void* w, int M, int N, int K, float* resid, const void* expert_out,
+                                       const float* expert_weights, int top, const void* alpha, const void* gain, const void* bias,
+                                       void* x_compute, lr_stream_t stream) {
+  LR_REQUIRE_PTR(resid);
+  LR_REQUIRE_PTR(gain);
+  LR_REQUIRE_PTR(bias);
+  LR_REQUIRE_PTR(x_compute);
+  LR_OPTIONAL_PTR(expert_out);
+  if (alpha == nullptr || (expert_out && expert_weights == nullptr)) return LR_E_NULL;
+  if (M < 1 || (expert_out && top <= 0)) return LR_E_SHAPE;
+  if (M > 64) return LR_E_UNSUPPORTED;
+  const lr_projection_t q = {x, ldx, w, x_compute, N, N, K, LR_EPI_NONE, nullptr};
+  Proj pr[1] = {};
+  const int rc = sb_fill_projection(q, pr[0]);
+  if (rc != LR_OK) return rc;
+  const int ncu = lr_num_cus();
+  if (ncu < 1) return LR_E_LAUNCH;
+  const int units = pick_units_and_plan(pr, 1, M, ncu);
+  const BandResidual rs = {resid, (u16*)x_compute, (const u16*)alpha, (const u16*)gain, (const u16*)bias, (const u16*)expert_out,
+                           expert_weights, top};
+  hipStream_t s = (hipStream_t)stream;
+  if (M > 32) return launch_residual<64, true>(pr[0], M, units, rs, s);
+  if (M > 16) return launch_residual<32, true>(pr[0], M, units, rs, s);
+  return M >= XLDS_M16_FROM ? launch_residual<16, true>(pr[0], M, units, rs, s) : launch_residual<16, false>(pr[0], M, units, rs, s);
+}
+
 #ifdef LR_BAND_PROFILE
 // Profile builds only (not declared in the public header): following launches of this file's kernels record, per
 // wave, the six wall-clock stamps of stream_band.h into `device_buffer` (NULL switches it off).  Returns the

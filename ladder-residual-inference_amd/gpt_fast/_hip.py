@@ -81,6 +81,8 @@ _PROTOS = {
     "lr_latent_attention": (c_int, [c_void_p, c_void_p]),
     "lr_residual_tanh": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                  c_int, c_int, c_int, c_void_p]),
+    "lr_linear_residual_tanh": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
+                                        c_void_p, c_void_p, c_void_p, c_void_p]),
     "lr_causal_conv": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
                                c_int, c_int, c_void_p]),
     "lr_ssd_scratch_bytes": (c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
@@ -808,6 +810,22 @@ def residual_tanh(x, d, alpha, gain, bias, x_out, x_compute, experts=None):
     _check(load().lr_residual_tanh(_dev(x, torch.float32), _opt(d, dt), _opt(eo, dt), _opt(ew, torch.float32), top, _dev(alpha, dt),
                                    _dev(gain, dt), _dev(bias, dt), _opt(x_out, torch.float32), _opt(x_compute, dt), rows, dim,
                                    _DTYPES[dt], _stream()), "lr_residual_tanh")
+
+
+def linear_residual_tanh(h, w, x, alpha, gain, bias, x_compute, experts=None):
+    """residual_tanh with d = h w^T (lr_linear_residual_tanh), in place on x [rows <= 64, dim]; bf16."""
+    M, K, ldx = _rows_ld(h)
+    N, Kw = w.shape
+    assert w.is_contiguous() and Kw == K and tuple(x.shape) == tuple(x_compute.shape) == (M, N) and x.is_contiguous()
+    assert x_compute.is_contiguous() and gain.numel() == bias.numel() == N and alpha.numel() == 1
+    eo, ew, top = None, None, 0
+    if experts is not None:
+        eo, ew = experts
+        top = ew.shape[1]
+        assert eo.is_contiguous() and ew.is_contiguous() and ew.shape[0] == M and eo.numel() == M * top * N
+    _check(load().lr_linear_residual_tanh(_dev(h), ldx, _dev(w), M, N, K, _dev(x, torch.float32), _opt(eo, torch.bfloat16),
+                                          _opt(ew, torch.float32), top, _dev(alpha), _dev(gain), _dev(bias), _dev(x_compute), _stream()),
+           "lr_linear_residual_tanh")
 
 
 def causal_conv(u, w, bias, ring, pos, out, B, S):

@@ -8,7 +8,8 @@ without a shared expert) or absent.
 
 The parallel form is used throughout: one launch projects h for mixer and feed-forward (decode batches), and the mixer's
 output projection and the feed-forward's down projection are one product over the concatenated columns, whose fp32 sums are
-the layer's update.  The norm needs no statistics, so residual, experts' weighted sum and the next layer's norm are one pass.
+the layer's update.  The norm needs no statistics, so residual, experts' weighted sum and the next layer's norm are one pass,
+which in decode batches is the end of that product.
 The residual stream is fp32; projections, caches and activations are bf16, or fp32 when the model's parameters are.  States
 live in fp32.  A call at position 0 starts every sequence of the batch anew, so a cache slot is reused without being cleared;
 later calls continue where the previous one ended (input_pos must be consecutive)."""
@@ -109,8 +110,7 @@ class GPTGepolix(GPTHybrid):
             blk.mixer.mix(ws, pos, proj, y)
             if m is not None:
                 _hip.moe(routed)
-            project(both, blk.mixer.out_proj, ws.d)
-            following.into(ws.x, ws.d, ws.x, ws.xc, experts)
+            following.after(both, blk.mixer.out_proj, ws.d, ws.x, ws.xc, experts)
         return None, None
 
     def _project_in(self, ws, blk, act, routed):

@@ -83,6 +83,14 @@ class DynamicTanh(nn.Module):
         _hip.residual_tanh(x, d, self.alpha, self.weight, self.bias, x_out, out, experts)
 
 
+    def after(self, h: Tensor, lin: nn.Linear, d: Tensor, x: Tensor, out: Tensor, experts=None):
+        """into() with lin(h) added to x in place: one launch for a decode batch, through `d` otherwise."""
+        if h.dtype == torch.bfloat16 and h.shape[0] <= 64:
+            _hip.linear_residual_tanh(h, lin.weight, x, self.alpha, self.weight, self.bias, out, experts)
+        else:
+            self.into(x, _hip.linear(h, lin.weight, d), x, out, experts)
+
+
 class Experts(nn.Module):
     """`n` gated feed-forwards of width ff, of which a token uses `top`.  w1 rows of an expert are [up; gate].  With a shared
     expert the router has one row more, that expert's gate."""

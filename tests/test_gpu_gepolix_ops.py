@@ -70,6 +70,21 @@ def test_residual_tanh(hip, dtype, rows, dim, top):
     close(x, d64(keep) + d64(d), F32)
 
 
+@pytest.mark.parametrize("M", [1, 2, 8, 9, 16, 30, 64])
+@pytest.mark.parametrize("N,K,top", [(72, 200, 0), (2048, 136, 3), (5000, 1000, 1)])
+def test_linear_residual_tanh(hip, M, N, K, top):
+    h, w = rnd(M, K + 8, seed=1, dtype=BF)[:, :K], (rnd(N, K, seed=2) / K ** 0.5).to(BF)
+    x, gain, bias, alpha = rnd(M, N, seed=3), rnd(N, seed=4, dtype=BF), rnd(N, seed=5, dtype=BF), torch.tensor([0.75], dtype=BF, device=DEV)
+    experts = (rnd(M * top, N, seed=6, dtype=BF), torch.softmax(rnd(M, top, seed=7), -1)) if top else None
+    want = d64(x) + d64(h) @ d64(w).T
+    if top:
+        want += (d64(experts[1])[:, :, None] * d64(experts[0]).view(M, top, N)).sum(1)
+    out = torch.full((M, N), float("nan"), dtype=BF, device=DEV)
+    hip.linear_residual_tanh(h, w, x, alpha, gain, bias, out, experts)
+    close(x, want, F32)
+    close(out, O.dynamic_tanh(want, d64(alpha), d64(gain), d64(bias)), BF)
+
+
 # ------------------------------------------------------------------------------------------------ convolution
 
 @pytest.mark.parametrize("dtype", [F32, BF])
