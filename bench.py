@@ -352,8 +352,6 @@ def gepolix_kernels(model, lasivik, B, T, decode):
     # feed-forwards: the mixture; the dense one of the same model (as the Lasivik model's, two launches) for comparison
     x = blocks["moe"].experts
     xc = rnd(rows, D)
-    distinct = x.n * (1 - (1 - x.top / x.n) ** rows)
-    wbytes = int(distinct * 3 * x.ff * D * 2)
     n = copies(x.n * 3 * x.ff * D * 2)
     w1s, w2s = [rnd(x.n, 2 * x.ff, D) for _ in range(n)], [rnd(x.n, D, x.ff) for _ in range(n)]
     router, rb = rnd(x.n + x.shared, D), rnd(x.n)
@@ -361,11 +359,15 @@ def gepolix_kernels(model, lasivik, B, T, decode):
     counts, scratch = torch.zeros(x.n, dtype=torch.int32, device=dev), bytes_of(1, _hip.moe_scratch_bytes(rows, x.n, x.top, x.ff, BF))[0]
     shared = rnd(rows, blocks["moe"].beside) if x.shared else None
     gate = torch.empty(rows, device=dev)
-    us = _graph_us([lambda i=i: _hip.moe(_hip.moe_desc(xc, router, rb, w1s[i], w2s[i], eo, ids, wts, gate, counts, scratch, shared))
-                    for i in range(n)])
+    descs = [_hip.moe_desc(xc, router, rb, w1s[i], w2s[i], eo, ids, wts, gate, counts, scratch, shared) for i in range(n)]
+    _hip.moe(descs[0])
+    for d in descs:
+        d.routed = int(decode)      # a decode step routes beside its projections
+    us = _graph_us([lambda d=d: _hip.moe(d) for d in descs])
     name = f"{x.n} experts of {x.ff}, top {x.top}"
     if decode:
-        out.append(_kernel_row(f"lr_moe ({name}; router, up, down)", us, "hbm", wbytes + 2 * rows * x.top * D))
+        wbytes = len(ids.unique()) * 3 * x.ff * D * 2
+        out.append(_kernel_row(f"lr_moe ({name}; up, down)", us, "hbm", wbytes + 2 * rows * x.top * D))
     else:
         out.append(_kernel_row(f"lr_moe ({name})", us, "mfma", 6 * rows * x.top * x.ff * D))
     del w1s, w2s

@@ -20,7 +20,7 @@ struct RopeCache {
   int32_t* err;
 };
 
-// A workgroup per token; an item is a rotation pair, or two columns that pass.
+// A workgroup per token (few tokens: several); an item is a rotation pair, or two columns that pass.
 template <typename T>
 __global__ __launch_bounds__(256) void k_bias_rope_cache(const RopeCache a) {
   const int row = blockIdx.x, b = row / a.S, s = row - b * a.S;
@@ -35,7 +35,8 @@ __global__ __launch_bounds__(256) void k_bias_rope_cache(const RopeCache a) {
   const int heads = a.H + (a.cache ? a.G : 0);
   T* crow = a.cache ? reinterpret_cast<T*>(a.cache) + ((int64_t)b * a.Smax + p) * a.ldc : nullptr;
   auto value = [&](int c) { return ldf(x + c) + (bias ? ldf(bias + c) : 0.0f); };
-  for (int i = threadIdx.x; i < heads * dk2; i += 256) {
+  const int first = blockIdx.y * 256 + threadIdx.x, step = gridDim.y * 256;
+  for (int i = first; i < heads * dk2; i += step) {
     const int h = i / dk2, j = i - h * dk2;
     T* out = h < a.H ? x + h * a.dk : crow + (h - a.H) * a.dk;
     if (j < half) {
@@ -53,7 +54,7 @@ __global__ __launch_bounds__(256) void k_bias_rope_cache(const RopeCache a) {
   }
   if (crow) {
     const int v0 = (a.H + a.G) * a.dk;
-    for (int i = threadIdx.x; i < a.G * a.dv; i += 256) stf(crow + a.G * a.dk + i, value(v0 + i));
+    for (int i = first; i < a.G * a.dv; i += step) stf(crow + a.G * a.dk + i, value(v0 + i));
   }
 }
 
@@ -226,8 +227,10 @@ extern "C" int lr_bias_rope_cache(void* proj, int64_t ld, const void* bias, cons
   const int64_t cols = (int64_t)H * dk + (cache ? (int64_t)G * (dk + dv) : 0);
   if (ld < cols || (cache && ldc < G * (dk + dv)) || (int64_t)B * S > 0x7fffffff) return LR_E_SHAPE;
   const RopeCache a = {proj, ld, bias, rope, pos, cache, B * S, S, H, G, dk, dv, rot, rope_len, ldc, Smax, err};
-  if (dtype == LR_BF16) k_bias_rope_cache<u16><<<dim3(a.rows), dim3(256), 0, (hipStream_t)stream>>>(a);
-  else if (dtype == LR_F32) k_bias_rope_cache<float><<<dim3(a.rows), dim3(256), 0, (hipStream_t)stream>>>(a);
+  const int items = ((H + (cache ? G : 0)) * ((dk + 1) / 2) + 255) / 256;
+  const dim3 grid(a.rows, a.rows <= 64 ? (items < 16 ? items : 16) : 1);
+  if (dtype == LR_BF16) k_bias_rope_cache<u16><<<grid, dim3(256), 0, (hipStream_t)stream>>>(a);
+  else if (dtype == LR_F32) k_bias_rope_cache<float><<<grid, dim3(256), 0, (hipStream_t)stream>>>(a);
   else return LR_E_UNSUPPORTED;
   return lr_launch_status();
 }

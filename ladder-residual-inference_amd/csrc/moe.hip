@@ -44,37 +44,40 @@ __device__ __forceinline__ void route_rows(const Router& a, const int block, flo
   float* logits = part + NW * ET * 256;      // [16][n]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g4 = lane >> 4, l16 = lane & 15;
   const int r0 = block * 16, nr = min(16, a.rows - r0), D = a.D, E = a.E, n = a.n;
-  constexpr int V = 16 / sizeof(T), KS = 4 * V;      // values per load, columns per step
-  constexpr int U = ET > 2 ? 4 : 8;                  // steps whose loads are in flight together
-  const T* xr = reinterpret_cast<const T*>(a.x) + (int64_t)(r0 + min(l16, nr - 1)) * a.ldx;
+  // A wave takes blocks of 128 bytes of every row, a lane 32 consecutive bytes of them in two steps (the order of the columns
+  // inside a step is the same in both operands); BL blocks are in flight together.
+  constexpr int V = 16 / sizeof(T), BK_ = 8 * V, BL = 4;
+  constexpr int SZ = (int)sizeof(T);
+  const rsrc_t rx = buffer_of(reinterpret_cast<const T*>(a.x) + (int64_t)r0 * a.ldx, (int)(((nr - 1) * a.ldx + D) * SZ));
+  const int xo = l16 < nr ? (int)(l16 * a.ldx) * SZ : NOWHERE;
   for (int e0 = 0; e0 < n; e0 += 16 * ET) {
-    const T* wr[ET];
-#pragma unroll
-    for (int t = 0; t < ET; ++t) wr[t] = reinterpret_cast<const T*>(a.w) + (int64_t)min(e0 + 16 * t + l16, n - 1) * D;
+    const int ne = min(16 * ET, n - e0);
+    const rsrc_t rw = buffer_of(reinterpret_cast<const T*>(a.w) + (int64_t)e0 * D, ne * D * SZ);
     f32x4_t acc[ET];
 #pragma unroll
     for (int t = 0; t < ET; ++t) acc[t] = f32x4_t{0, 0, 0, 0};
-    for (int k = KS * wave; k < D; k += KS * NW * U) {
-      uint4 xv[U], wv[U][ET];
+    for (int k = BK_ * wave; k < D; k += BK_ * NW * BL) {
+      u32x4_t xv[2 * BL], wv[2 * BL][ET];
 #pragma unroll
-      for (int u = 0; u < U; ++u) {
-        const int c = min(k + KS * NW * u + V * g4, D - V);      // (beyond the row: its last columns, dropped below)
-        xv[u] = ld16(xr + c);
+      for (int u = 0; u < 2 * BL; ++u) {
+        const int c = k + BK_ * NW * (u >> 1) + 2 * V * g4 + V * (u & 1);
+        xv[u] = __builtin_amdgcn_raw_buffer_load_b128(rx, c < D && xo >= 0 ? xo + c * SZ : NOWHERE, 0, 0);
 #pragma unroll
-        for (int t = 0; t < ET; ++t) wv[u][t] = ld16(wr[t] + c);
+        for (int t = 0; t < ET; ++t)
+          wv[u][t] = __builtin_amdgcn_raw_buffer_load_b128(rw, c < D && 16 * t + l16 < ne ? ((16 * t + l16) * D + c) * SZ : NOWHERE, 0, 0);
       }
+      __builtin_amdgcn_sched_barrier(0);      // (all of them, before the first is used)
 #pragma unroll
-      for (int u = 0; u < U; ++u) {
-        if (k + KS * NW * u + V * g4 >= D) xv[u] = make_uint4(0, 0, 0, 0);
+      for (int u = 0; u < 2 * BL; ++u) {
 #pragma unroll
         for (int t = 0; t < ET; ++t) {
           if constexpr (sizeof(T) == 2) {
             acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, wv[u][t]), __builtin_bit_cast(bf16x8_t, xv[u]), acc[t], 0, 0, 0);
           } else {
-            acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(wv[u][t].x), __uint_as_float(xv[u].x), acc[t], 0, 0, 0);
-            acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(wv[u][t].y), __uint_as_float(xv[u].y), acc[t], 0, 0, 0);
-            acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(wv[u][t].z), __uint_as_float(xv[u].z), acc[t], 0, 0, 0);
-            acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(wv[u][t].w), __uint_as_float(xv[u].w), acc[t], 0, 0, 0);
+            acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(wv[u][t][0]), __uint_as_float(xv[u][0]), acc[t], 0, 0, 0);
+            acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(wv[u][t][1]), __uint_as_float(xv[u][1]), acc[t], 0, 0, 0);
+            acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(wv[u][t][2]), __uint_as_float(xv[u][2]), acc[t], 0, 0, 0);
+            acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(__uint_as_float(wv[u][t][3]), __uint_as_float(xv[u][3]), acc[t], 0, 0, 0);
           }
         }
       }
@@ -287,8 +290,8 @@ struct SharedAct {
   const float* gate;
 };
 constexpr int BAND_ENTRIES = 16;      // input rows per pass over a band's weights
-template <int UNITS>
-__global__ __launch_bounds__(NWV * 64) void k_expert_band(Proj p, const int64_t wstride, const int32_t* __restrict__ experts, const int n,
+template <int UNITS, int KW>
+__global__ __launch_bounds__(NWV * 64, 2) void k_expert_band(Proj p, const int64_t wstride, const int32_t* __restrict__ experts, const int n,
                                                           const int by_slot, const int xdiv, const int ny, const SharedAct sh) {
   extern __shared__ __attribute__((aligned(16))) u16 sg_smem[];
   int32_t* list = reinterpret_cast<int32_t*>(sg_smem + stream_band_lds_bytes<16, UNITS>() / sizeof(u16));   // [n]
@@ -322,28 +325,29 @@ __global__ __launch_bounds__(NWV * 64) void k_expert_band(Proj p, const int64_t 
   p.w += e * wstride;
   for (int i = 0; i < m; i += BAND_ENTRIES) {
     if (i) __syncthreads();
-    stream_band<16, UNITS, false, false, true>(p, min(BAND_ENTRIES, m - i), blockIdx.x, sg_smem, list + i, xdiv);
+    stream_band<16, UNITS, false, false, true, false, KW>(p, min(BAND_ENTRIES, m - i), blockIdx.x, sg_smem, list + i, xdiv);
   }
 }
 
-template <int UNITS>
+// KW: waves that share a band's columns (1: every wave has a band of its own, for short rows)
+template <int UNITS, int KW = NWV>
 int launch_band(const Proj& p, int64_t wstride, const int32_t* experts, int n, int E, bool by_slot, int xdiv, hipStream_t s, const SharedAct& sh = {}) {
   const size_t lds = stream_band_lds_bytes<16, UNITS>() + sizeof(int32_t) * n;
   static std::atomic<unsigned long long> raised{0};
-  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_expert_band<UNITS>), lds, raised)) return LR_E_LAUNCH;
+  if (!lr_raise_lds_limit(reinterpret_cast<const void*>(&k_expert_band<UNITS, KW>), lds, raised)) return LR_E_LAUNCH;
   const int ny = by_slot ? n : E;
-  k_expert_band<UNITS><<<dim3(p.nwg, ny + (sh.act ? 1 : 0)), dim3(NWV * 64), lds, s>>>(p, wstride, experts, n, by_slot, xdiv, ny, sh);
+  k_expert_band<UNITS, KW><<<dim3(p.nwg, ny + (sh.act ? 1 : 0)), dim3(NWV * 64), lds, s>>>(p, wstride, experts, n, by_slot, xdiv, ny, sh);
   return lr_launch_status();
 }
 
 constexpr int BAND_ROWS = 64, BAND_LIST = 4096;      // tokens and entries up to which the bands are taken
 bool by_bands(int rows, int top, int dtype) { return dtype == LR_BF16 && rows <= BAND_ROWS && (int64_t)rows * top <= BAND_LIST; }
 
-// Height of the grouped tiles: 256 rows where that still makes a tile for most CUs in both products.
+// Height of the grouped tiles: 256 rows where experts fill them and there are tiles for most CUs.
 int tile_rows(int rows, int E, int top, int I, int D, int dtype) {
   if (dtype == LR_F32) return lr_detail::linear_f32_grouped_rows();
   const int64_t n = (int64_t)rows * top, e = n < E ? n : E, tall = n / 256 + e / 2;
-  return tall * ((I + 127) / 128) >= 192 && tall * ((D + 255) / 256) >= 192 ? 256 : 128;
+  return n >= 256 * e && tall * ((I + 127) / 128) >= 160 && tall * ((D + 255) / 256) >= 160 ? 256 : 128;
 }
 int max_tiles(int rows, int E, int top, int height) {
   const int64_t n = (int64_t)rows * top, e = n < E ? n : E;
@@ -364,7 +368,7 @@ int launch_router(const Router& a, hipStream_t s) {
 template <typename T>
 int route(const lr_moe_t* d, hipStream_t s) {
   const Router a = router_of(d);
-  return a.n <= 16 ? launch_router<T, 1>(a, s) : a.n <= 32 ? launch_router<T, 2>(a, s) : launch_router<T, 4>(a, s);
+  return a.n <= 16 ? launch_router<T, 1>(a, s) : a.n <= 32 ? launch_router<T, 2>(a, s) : a.n <= 48 ? launch_router<T, 3>(a, s) : launch_router<T, 4>(a, s);
 }
 
 template <int MT, bool XL, int ET>
@@ -427,7 +431,7 @@ static int check_moe(const lr_moe_t* d) {
   if (d->rows <= 0 || d->D <= 0 || d->E <= 0 || d->top <= 0 || d->top > d->E || d->I <= 0 || d->ldx < d->D) return LR_E_SHAPE;
   if (d->shared && (d->shared_cols <= 0 || d->ld_shared < d->shared_cols)) return LR_E_SHAPE;
   if (d->D % 8 || d->I % 8 || d->ldx % 8 || (d->shared && (d->ld_shared % 8 || d->shared_cols % 8))) return LR_E_ALIGN;
-  if (d->E > 64 * EPL || (int64_t)d->rows * d->top > (1 << 28)) return LR_E_UNSUPPORTED;
+  if (d->E > 64 * EPL || d->ldx > (1 << 24) || d->D > (1 << 22) || (int64_t)d->rows * d->top > (1 << 28)) return LR_E_UNSUPPORTED;
   return d->scratch_bytes < layout(d->rows, d->E, d->top, d->I, d->dtype).total ? LR_E_SHAPE : LR_OK;
 }
 
@@ -448,7 +452,7 @@ extern "C" int lr_linear_multi_route(const lr_projection_t* proj, int n_proj, in
   const Router a = router_of(d);
   hipStream_t s = (hipStream_t)stream;
   return a.n <= 16 ? project_route<1>(pr[0], pr[1], M, a, s) : a.n <= 32 ? project_route<2>(pr[0], pr[1], M, a, s)
-                                                                         : project_route<4>(pr[0], pr[1], M, a, s);
+         : a.n <= 48 ? project_route<3>(pr[0], pr[1], M, a, s) : project_route<4>(pr[0], pr[1], M, a, s);
 }
 
 extern "C" int lr_moe(const lr_moe_t* d, lr_stream_t stream) {
@@ -474,19 +478,29 @@ extern "C" int lr_moe(const lr_moe_t* d, lr_stream_t stream) {
     const bool by_slot = d->rows == 1;
     Proj p = {};
     p.x = (const u16*)d->x; p.ldx = d->ldx; p.w = (const u16*)d->w1; p.y = (u16*)act; p.ldy = I; p.N = 2 * I; p.K = D; p.pair_off = I;
-    p.rpw = 16; p.nwg = (I + 15) / 16;
+    const int64_t busy = n < d->E ? n : d->E;      // experts, at most
+    p.rpw = busy * ((I + 15) / 16) < 256 ? 8 : 16;
+    p.nwg = (I + p.rpw - 1) / p.rpw;
     const SharedAct sh = {(u16*)d->shared, d->ld_shared, d->shared_cols, d->rows, d->gate};
     rc = launch_band<2>(p, (int64_t)2 * I * D, d->experts, n, d->E, by_slot, d->top, s, sh);
     if (rc != LR_OK) return rc;
     Proj o = {};
     o.x = (const u16*)act; o.ldx = I; o.w = (const u16*)d->w2; o.y = (u16*)d->out; o.ldy = D; o.N = D; o.K = I;
-    const int64_t busy = n < d->E ? n : d->E;
+    const int64_t w2 = (int64_t)I * D;
+    if (I <= 1024 && busy * ((D + 127) / 128) >= 256) {
+      o.rpw = 32; o.nwg = (D + 127) / 128;
+      return launch_band<2, 1>(o, w2, d->experts, n, d->E, by_slot, 1, s);
+    }
+    if (I <= 1024 && busy * ((D + 63) / 64) >= 256) {
+      o.rpw = 16; o.nwg = (D + 63) / 64;
+      return launch_band<1, 1>(o, w2, d->experts, n, d->E, by_slot, 1, s);
+    }
     if (busy * ((D + 31) / 32) >= 512) {
       o.rpw = 32; o.nwg = (D + 31) / 32;
-      return launch_band<2>(o, (int64_t)I * D, d->experts, n, d->E, by_slot, 1, s);
+      return launch_band<2>(o, w2, d->experts, n, d->E, by_slot, 1, s);
     }
     o.rpw = 16; o.nwg = (D + 15) / 16;
-    return launch_band<1>(o, (int64_t)I * D, d->experts, n, d->E, by_slot, 1, s);
+    return launch_band<1>(o, w2, d->experts, n, d->E, by_slot, 1, s);
   }
 
   const int height = tile_rows(d->rows, d->E, d->top, I, D, d->dtype), mt = max_tiles(d->rows, d->E, d->top, height);

@@ -214,12 +214,12 @@ __global__ __launch_bounds__(256) void k_ssd_walk(const Ssd a) {
 }
 
 // ---------------------------------------------------------------------------------------------- one token
-// 256 threads: four columns each, the rows of S side by side
-template <typename T>
+// 256 threads: four columns each, the rows of S side by side.  Everything from memory is asked for before anything is used.
+template <typename T, int TAPS>
 __global__ __launch_bounds__(256) void k_ssd_step(const Ssd a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const int bh = blockIdx.x, b = bh / a.H, h = bh - b * a.H, hpg = a.H / a.G, g = h / hpg, tid = threadIdx.x;
-  const int N = a.N, P = a.P, taps = a.taps;
+  const int N = a.N, P = a.P, taps = TAPS ? TAPS : a.taps;
   float* xs = sm;               // [P]
   float* bs = xs + P;           // [N]
   float* cs = bs + N;           // [N]
@@ -243,27 +243,51 @@ __global__ __launch_bounds__(256) void k_ssd_step(const Ssd a) {
     return;
   }
   // the convolution of this head's channels: x, then B and C of its group
-  const int slot = p % taps;
+  constexpr int W = TAPS ? TAPS : MAX_TAPS, IT = 3;      // (P + 2 N <= 768 channels)
+  const int nch = P + 2 * N, slot = p % taps;
   const T* cw = reinterpret_cast<const T*>(a.conv_w);
   const T* cb = reinterpret_cast<const T*>(a.conv_b);
   T* ring = reinterpret_cast<T*>(a.ring) + (int64_t)b * taps * a.C;
   const T* u = reinterpret_cast<const T*>(a.x) + (int64_t)b * a.ldu;       // channel 0 of the convolution
-  for (int i = tid; i < P + 2 * N; i += 256) {
-    const int ch = i < P ? h * P + i : (i < P + N ? a.H * P + g * N + i - P : a.H * P + (a.G + g) * N + i - P - N);
-    const T raw = u[ch];
-    float v = fmaf(ldf(cw + (int64_t)ch * taps + taps - 1), ldf(&raw), ldf(cb + ch));
-    for (int j = 1; j < taps; ++j) {
-      const float past = ldf(ring + (int64_t)((p - j + taps) % taps) * a.C + ch);
-      v = fmaf(ldf(cw + (int64_t)ch * taps + taps - 1 - j), p >= j ? past : 0.0f, v);
+  auto channel = [&](int i) { return i < P ? h * P + i : (i < P + N ? a.H * P + g * N + i - P : a.H * P + (a.G + g) * N + i - P - N); };
+  T raw[IT], cbias[IT], past[IT][W], w[IT][W];
+#pragma unroll
+  for (int k = 0; k < IT; ++k) {
+    if (256 * k >= nch) break;
+    const int ch = channel(min(tid + 256 * k, nch - 1));
+    raw[k] = u[ch];
+    cbias[k] = cb[ch];
+#pragma unroll
+    for (int j = 0; j < W; ++j) {      // j tokens back
+      if (j >= taps) break;
+      w[k][j] = cw[(int64_t)ch * taps + taps - 1 - j];
+      if (j > 0) past[k][j] = ring[(int64_t)((p - j + taps) % taps) * a.C + ch];
     }
-    sm[i] = silu_f(v);
-    if (taps > 1 && (i < P || h % hpg == 0)) ring[(int64_t)slot * a.C + ch] = raw;   // (a slot nobody reads in this step)
   }
-  const float dt = softplus_f(ldf(reinterpret_cast<const T*>(a.dt) + (int64_t)b * a.ld + h) +
-                              ldf(reinterpret_cast<const T*>(a.dt_bias) + h));
-  const float e = p > 0 ? expf(-expf(ldf(reinterpret_cast<const T*>(a.a_log) + h)) * dt) : 0.0f;
+  const T* dtp = reinterpret_cast<const T*>(a.dt) + (int64_t)b * a.ld + h;
+  const T draw = *dtp, dbias = reinterpret_cast<const T*>(a.dt_bias)[h], araw = reinterpret_cast<const T*>(a.a_log)[h];
+  const T Draw = reinterpret_cast<const T*>(a.d)[h];
   const T zraw = reinterpret_cast<const T*>(a.z)[(int64_t)b * a.ld + h * P + (tid < P ? tid : 0)];
-  const float D = ldf(reinterpret_cast<const T*>(a.d) + h);
+  __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+  for (int k = 0; k < IT; ++k) {
+    if (256 * k >= nch) break;
+    const int i = tid + 256 * k;
+    float v = fmaf(ldf(&w[k][0]), ldf(&raw[k]), ldf(&cbias[k]));
+#pragma unroll
+    for (int j = 1; j < W; ++j) {
+      if (j >= taps) break;
+      v = fmaf(ldf(&w[k][j]), p >= j ? ldf(&past[k][j]) : 0.0f, v);
+    }
+    if (i < nch) {
+      sm[i] = silu_f(v);
+      // (into a slot nobody reads in this step)
+      if (taps > 1 && (i < P || h % hpg == 0)) ring[(int64_t)slot * a.C + channel(i)] = raw[k];
+    }
+  }
+  const float dt = softplus_f(ldf(&draw) + ldf(&dbias));
+  const float e = p > 0 ? expf(-expf(ldf(&araw)) * dt) : 0.0f;
+  const float D = ldf(&Draw);
   __syncthreads();
   float4 xv = *reinterpret_cast<const float4*>(xs + vq * 4);
   const float dx[4] = {dt * xv.x, dt * xv.y, dt * xv.z, dt * xv.w};
@@ -825,8 +849,10 @@ extern "C" int lr_ssd_step(const lr_ssd_t* d, const void* conv_w, const void* co
   a.conv_w = conv_w; a.conv_b = conv_b; a.ring = ring; a.taps = taps; a.C = a.H * a.P + 2 * a.G * a.N;
   const size_t lds = sizeof(float) * ((size_t)a.P + 2 * a.N + (256 / (a.P / 4)) * a.P);
   hipStream_t s = (hipStream_t)stream;
-  if (d->dtype == LR_F32) k_ssd_step<float><<<dim3(a.B * a.H), dim3(256), lds, s>>>(a);
-  else k_ssd_step<u16><<<dim3(a.B * a.H), dim3(256), lds, s>>>(a);
+  const dim3 grid(a.B * a.H), blk(256);
+  if (d->dtype == LR_F32) k_ssd_step<float, 0><<<grid, blk, lds, s>>>(a);
+  else if (taps == 4) k_ssd_step<u16, 4><<<grid, blk, lds, s>>>(a);
+  else k_ssd_step<u16, 0><<<grid, blk, lds, s>>>(a);
   return lr_launch_status();
 }
 

@@ -77,9 +77,10 @@ struct BandResidual {
   const float* ew;                       // [M, top]
   int top;
 };
+// KW: waves that share a band's K, all of them or 1: then every wave has a band of its own (`band_` counts groups of NWV).
 // GATHER: input row m is row rows[m] / xdiv of x, output row m is row rows[m] of y (`rows`: M of them, in LDS).
-template <int MT, int UNITS, bool W8 = false, bool XL = (MT >= XLDS_MIN_MT), bool GATHER = false, bool RESID = false>
-__device__ __forceinline__ void stream_band(const Proj& p, const int M, const int band, u16* sg_smem,
+template <int MT, int UNITS, bool W8 = false, bool XL = (MT >= XLDS_MIN_MT), bool GATHER = false, bool RESID = false, int KW = NWV>
+__device__ __forceinline__ void stream_band(const Proj& p, const int M, const int band_, u16* sg_smem,
                                             const int32_t* rows = nullptr, const int xdiv = 1, const BandResidual rs = {}) {
   static_assert(!W8 || MT == 16, "the e4m3 path is built for up to 16 input rows");
   constexpr int KCW = W8 ? 256 : 128;  // k elements per chunk
@@ -110,6 +111,9 @@ __device__ __forceinline__ void stream_band(const Proj& p, const int M, const in
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l16 = lane & 15, l4 = lane >> 4;
+  static_assert(KW == NWV || (KW == 1 && !W8 && !XL), "");
+  const int band = KW == 1 ? band_ * NWV + wave : band_;
+  const int kwave = KW == 1 ? 0 : wave;
   LR_BAND_STAMP(0)
   const int n_out = pair_off ? pair_off : N;         // output columns
   const int n0 = band * rpw;                          // first row (pair) of the band
@@ -166,14 +170,14 @@ __device__ __forceinline__ void stream_band(const Proj& p, const int M, const in
   // 1.5 % faster per step, 64-row bands 8 % slower -- their inputs come from L2, which likes the common window.
   // Not kept: the order of a sum would then depend on how the rows are cut into bands.)
   auto issue_w = [&](int ci, u32x4_t (&dst)[NLD]) {
-    const int k0 = (ci * NWV + wave) * KCW;
+    const int k0 = (ci * KW + kwave) * KCW;
     const bool kok = k0 + l16 * (16 / WB) < K;
 #pragma unroll
     for (int i = 0; i < NLD; ++i)
       dst[i] = __builtin_amdgcn_raw_buffer_load_b128(wres, (kok && woff[i] != OOB) ? woff[i] : OOB, k0 * WB, AUX_WEIGHTS);
   };
   auto issue_x = [&](int ci, u32x4_t (&dst)[MTILES][KS]) {
-    const int k0 = (ci * NWV + wave) * KCW;
+    const int k0 = (ci * KW + kwave) * KCW;
     if (XLDS) {
       const bool kok = k0 + l16 * 8 < K;
 #pragma unroll
@@ -193,7 +197,7 @@ __device__ __forceinline__ void stream_band(const Proj& p, const int M, const in
   };
 
   const int nck = (K + KCW - 1) / KCW;
-  const int nch = wave < nck ? (nck - wave + NWV - 1) / NWV : 0;  // chunks of this wave
+  const int nch = kwave < nck ? (nck - kwave + KW - 1) / KW : 0;  // chunks of this wave
   // (the fences keep the requests in this order: the wait for chunk 0 counts the requests made after it, and the
   // scheduler, left alone, asks for chunk 0 last -- the loop then waited for all but the last 8 requests at the top
   // of every round of NS chunks)
@@ -345,14 +349,14 @@ __device__ __forceinline__ void stream_band(const Proj& p, const int M, const in
     LR_BAND_STAMP(5)
     return;
   }
-  for (int o = tid; o < rows_out * MT; o += NWV * 64) {
+  for (int o = KW == 1 ? lane : tid; o < rows_out * MT; o += KW * 64) {
     const int r = o % rows_out, m = o / rows_out;
     if (r >= nrows || m >= M) continue;
     const int mt = m >> 4, ln = ((r & 15) >> 2) * 16 + (m & 15), e = r & 3, u = r >> 4;
     const int ym = GATHER ? rows[m] : m;
     float s0 = 0.0f, s1 = 0.0f;
 #pragma unroll
-    for (int wv = 0; wv < NWV; ++wv) s0 += red[wv * WSTRIDE + ((u * MTILES + mt) * 4 + e) * 64 + ln];
+    for (int wv = 0; wv < KW; ++wv) s0 += red[(KW == 1 ? wave : wv) * WSTRIDE + ((u * MTILES + mt) * 4 + e) * 64 + ln];
     if constexpr (RESID) {
       const int n = n0 + r;
       const int64_t at = (int64_t)m * N + n;
@@ -368,7 +372,7 @@ __device__ __forceinline__ void stream_band(const Proj& p, const int M, const in
     } else if (pair_off) {
       if (UNITS == 2) {
 #pragma unroll
-        for (int wv = 0; wv < NWV; ++wv) s1 += red[wv * WSTRIDE + ((MTILES + mt) * 4 + e) * 64 + ln];
+        for (int wv = 0; wv < KW; ++wv) s1 += red[(KW == 1 ? wave : wv) * WSTRIDE + ((MTILES + mt) * 4 + e) * 64 + ln];
       }
       float u_ = round_bf(s0), g_ = round_bf(s1);
       if constexpr (W8) {
