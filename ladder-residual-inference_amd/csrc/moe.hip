@@ -479,8 +479,8 @@ extern "C" int lr_moe(const lr_moe_t* d, lr_stream_t stream) {
     Proj p = {};
     p.x = (const u16*)d->x; p.ldx = d->ldx; p.w = (const u16*)d->w1; p.y = (u16*)act; p.ldy = I; p.N = 2 * I; p.K = D; p.pair_off = I;
     const int64_t busy = n < d->E ? n : d->E;      // experts, at most
-    p.rpw = busy * ((I + 15) / 16) < 256 ? 8 : 16;
-    p.nwg = (I + p.rpw - 1) / p.rpw;
+    p.rpw = 16;
+    p.nwg = (I + 15) / 16;
     const SharedAct sh = {(u16*)d->shared, d->ld_shared, d->shared_cols, d->rows, d->gate};
     rc = launch_band<2>(p, (int64_t)2 * I * D, d->experts, n, d->E, by_slot, d->top, s, sh);
     if (rc != LR_OK) return rc;
