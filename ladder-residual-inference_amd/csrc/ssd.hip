@@ -137,7 +137,6 @@ __global__ __launch_bounds__(256) void k_causal_conv(const Conv a) {
 // ---------------------------------------------------------------------------------------------- token by token
 // One workgroup: 16 columns of P of one (sequence, head).  A thread: one column, every 16th of N.
 constexpr int WALK_T = 32;          // tokens whose inputs lie in LDS together
-constexpr int WALK_N = 16;          // values of N per thread, at most
 
 template <typename T, int NPT>
 __global__ __launch_bounds__(256) void k_ssd_walk(const Ssd a) {
